@@ -8,7 +8,7 @@ CPU or PyTorch fallback behind any of these calls.
 from __future__ import annotations
 
 import ctypes
-from ctypes import c_char_p, c_float, c_int, c_size_t, c_void_p
+from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_void_p
 from pathlib import Path
 
 LIBRARY_PATH = Path(__file__).resolve().parent / "libajq.so"
@@ -141,7 +141,61 @@ BENCH_SIGNATURES: dict[str, tuple] = {
     "ajqb_mfma_rate": (c_int, [c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p]),
 }
 
+# libajq_dense.so (include/ajq_dense.h): the operators of the dense model family
+DENSE_LIBRARY_PATH = Path(__file__).resolve().parent / "libajq_dense.so"
+
+AJQD_BF16 = 0
+AJQD_F32 = 1
+AJQD_ACTIVATIONS = {"relu": 0, "silu": 1, "gelu_tanh": 2}
+
+
+class LatentShape(ctypes.Structure):
+    """``ajqd_latent_shape``"""
+
+    _fields_ = [(n, c_int) for n in ("heads", "dimp", "rot", "rotp", "rank", "rankp")] + [("eps", c_float)]
+
+
+class WindowedAttentionArgs(ctypes.Structure):
+    """``ajqd_windowed_attention_args``"""
+
+    _fields_ = ([(n, c_void_p) for n in ("q", "k1", "k2", "v", "sink", "gates", "pos", "out")]
+                + [(n, c_int64) for n in ("k1_batch", "k2_batch", "v_batch")]
+                + [(n, c_int) for n in ("k1_row", "k1_head", "k2_row", "v_row", "v_head", "d1", "d2", "dv", "batch",
+                                        "heads", "seq", "rows", "prior", "window", "out_ld")]
+                + [("scale", c_float)])
+
+
+class DenseInArgs(ctypes.Structure):
+    """``ajqd_dense_in_args``"""
+
+    _fields_ = ([(n, c_void_p) for n in ("x", "n1", "n2", "gain1", "gain2", "w1", "w2", "y1", "gated")]
+                + [(n, c_int) for n in ("batch", "true_width", "width", "tiles1", "tiles2", "gated_ld", "act", "center")]
+                + [("eps", c_float)])
+
+
+_P, _I, _F, _L = c_void_p, c_int, c_float, c_int64
+DENSE_SIGNATURES: dict[str, tuple] = {
+    "ajqd_last_error": (c_char_p, []),
+    "ajqd_embed": (c_int, [_P, _I, _I, _P, _I, _P, _I, _I, _P, _P, _P, _P, _I, _I, _P]),
+    "ajqd_add_norms": (c_int, [_P, _P, _I, _P, _P, _P, _P, _F, _I, _P, _P, _I, _I, _I, _I, _P]),
+    "ajqd_latent_split": (c_int, [_P, _I, _I, ctypes.POINTER(LatentShape), _P, _P, _P, _I, _I, _I, _I, _P, _I, _I, _P, _I, _P,
+                                  _I, _P, _L, _P, _I, _P]),
+    "ajqd_ring_copy": (c_int, [_P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P]),
+    "ajqd_gated_activation": (c_int, [_P, _I, _P, _I, _I, _I, _I, _I, _P]),
+    "ajqd_matvec": (c_int, [_P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P]),
+    "ajqd_windowed_attention": (c_int, [ctypes.POINTER(WindowedAttentionArgs), _I, _I, _P]),
+    "ajqd_windowed_prefill_supported": (c_int, [_I, _I, _I]),
+    "ajqd_windowed_prefill": (c_int, [ctypes.POINTER(WindowedAttentionArgs), _P]),
+    "ajqd_dense_in": (c_int, [ctypes.POINTER(DenseInArgs), _P]),
+    "ajqd_dense_out": (c_int, [_P, _P, _P, _P, _P, _I, _I, _I, _P]),
+    "ajqd_latent_absorb": (c_int, [_P, _I, ctypes.POINTER(LatentShape), _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _P]),
+    "ajqd_latent_decode_chunks": (c_int, [_I, _I, _I, _I, _I]),
+    "ajqd_latent_decode": (c_int, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P]),
+    "ajqd_latent_expand": (c_int, [_P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P]),
+}
+
 _lib: ctypes.CDLL | None = None
+_dense_lib: ctypes.CDLL | None = None
 _bench_lib: ctypes.CDLL | None = None
 
 
@@ -178,6 +232,31 @@ def load() -> ctypes.CDLL:
         fn.argtypes = argtypes
     _lib = lib
     return lib
+
+
+def load_dense() -> ctypes.CDLL:
+    """The dense model family's operators, bound on first use (built by ``python -m ajllm_amd.build``)."""
+    global _dense_lib
+    if _dense_lib is not None:
+        return _dense_lib
+    if not DENSE_LIBRARY_PATH.exists():
+        raise RuntimeError(f"{DENSE_LIBRARY_PATH} is missing: build it with `python -m ajllm_amd.build` "
+                           "(the dense models have no fallback path)")
+    lib = ctypes.CDLL(str(DENSE_LIBRARY_PATH))
+    for name, (restype, argtypes) in DENSE_SIGNATURES.items():
+        fn = getattr(lib, name)
+        fn.restype = restype
+        fn.argtypes = argtypes
+    _dense_lib = lib
+    return lib
+
+
+def check_dense(status: int, what: str) -> None:
+    """``check`` for a status of libajq_dense.so."""
+    if status == 0:
+        return
+    message = f"{what}: {load_dense().ajqd_last_error().decode()}"
+    raise ValueError(message) if status in _ARGUMENT_ERRORS else RuntimeError(message)
 
 
 def check(status: int, what: str) -> None:

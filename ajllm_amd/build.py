@@ -1,4 +1,4 @@
-"""Compile the HIP sources in ``csrc/`` into ``libajq.so`` next to this file.
+"""Compile the HIP sources in ``csrc/`` into ``libajq.so`` and ``libajq_dense.so`` next to this file.
 
 Cross-compiles for gfx950 with hipcc; needs no GPU.  Run as
 ``python -m ajllm_amd.build`` or call :func:`build_library`.
@@ -15,6 +15,10 @@ from pathlib import Path
 PACKAGE_DIR = Path(__file__).resolve().parent
 SOURCE = PACKAGE_DIR / "csrc" / "ajq.hip"
 LIBRARY = PACKAGE_DIR / "libajq.so"
+# operators of the dense model family (include/ajq_dense.h): a library of its own, so that a dense model can be run
+# without waiting for the quantized matmuls to compile
+DENSE_SOURCE = PACKAGE_DIR / "csrc" / "ajq_dense.hip"
+DENSE_LIBRARY = PACKAGE_DIR / "libajq_dense.so"
 # measurement probes for bench.py (include/ajq_bench.h); the operator library does not depend on it
 BENCH_SOURCE = PACKAGE_DIR / "csrc" / "ajq_bench.hip"
 BENCH_LIBRARY = PACKAGE_DIR / "libajq_bench.so"
@@ -51,10 +55,22 @@ def build_library(verbose: bool = False, source: Path = SOURCE, library: Path = 
     return library
 
 
+def build_dense_library(verbose: bool = False) -> Path:
+    return build_library(verbose, DENSE_SOURCE, DENSE_LIBRARY)
+
+
+def ensure_dense_library() -> Path:
+    """The dense library, compiled now if it is not there yet."""
+    if not DENSE_LIBRARY.exists():
+        build_dense_library()
+    return DENSE_LIBRARY
+
+
 def build_bench_library(verbose: bool = False) -> Path:
     return build_library(verbose, BENCH_SOURCE, BENCH_LIBRARY)
 
 
 if __name__ == "__main__":
     print(build_library(verbose=True))
+    print(build_dense_library(verbose=True))
     print(build_bench_library(verbose=True))

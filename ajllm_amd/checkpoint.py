@@ -1,4 +1,5 @@
-"""Quantized checkpoints: the canonical tensors of every QuantLinear in one safetensors file.
+"""Checkpoints: quantized ones (the canonical tensors of every QuantLinear in one safetensors file), and folders with a
+``config.json`` and dense weights (``load_model``).
 
 The reference stores dense training checkpoints with ``torch.save`` as
 ``{"model_state_dict", "optimizer_state_dict", "step", "metadata"}``
@@ -114,6 +115,26 @@ def load_quantized(path: str | Path, device, verify: bool = True) -> tuple[model
     with torch.device(device):  # dense skeleton on the target device; its linears are swapped out next
         model = modeling.TransformerLM(**cfg)
     return load_quantized_into(model, tensors, manifest["scheme"], device), manifest
+
+
+def load_model(folder: str | Path, device, dtype: torch.dtype = torch.bfloat16) -> torch.nn.Module:
+    """The model a folder with ``config.json`` (which names its ``architecture``) and ``model.safetensors`` holds, on
+    ``device`` in ``dtype``.  Every tensor of the model must be in the file with the model's shape, and no other."""
+    folder = Path(folder)
+    config = json.loads((folder / "config.json").read_text())
+    if "architecture" not in config:
+        raise ValueError(f"{folder}/config.json names no architecture")
+    with torch.device("meta"):
+        model = modeling.build_model(config)
+    names = model.checkpoint_names()
+    with safe_open(str(folder / "model.safetensors"), framework="pt", device="cpu") as f:
+        present = set(f.keys())
+        missing, unexpected = set(names.values()) - present, present - set(names.values())
+        if missing or unexpected:
+            raise ValueError(f"checkpoint and model disagree: missing {sorted(missing)}, unexpected {sorted(unexpected)}")
+        state = {key: f.get_tensor(name).to(device=device, dtype=dtype) for key, name in names.items()}
+    model.load_state_dict(state, strict=True, assign=True)
+    return model.eval()
 
 
 @torch.no_grad()

@@ -1,0 +1,309 @@
+// Attention over keys that are made of a per-head part and a part all heads share, with a sliding window, an
+// attention sink and a per-head output gate:
+//
+//   s_j     = (qu . ku_j + qr . kr_j) * scale            over the visible rows j
+//   out     = gate * sum_j exp(s_j) v_j / (exp(sink) + sum_j exp(s_j))
+//
+// Three kernels:
+//   windowed_attention_kernel   any sizes, bf16 or fp32, one wave per (token, head): fp32 prompts and decoding
+//   windowed_prefill_kernel     prompts in bf16 on MFMA, keys and values expanded per head
+//   latent_decode_kernel        one token per sequence in bf16 on MFMA, in the latent space: the rows of the cache are
+//                               keys and values at once, all heads share them (see below)
+//
+// Scores, weights and sums are fp32; exponents are taken in base 2, scores multiplied by scale * log2(e).
+#pragma once
+#include "dense_kernels.h"
+#include "prefill_attention.h"
+
+namespace ajq {
+
+struct WindowedAttention {
+  const void* q;            // [B * T, H, d1 + d2]: unrotated part, rotated part
+  const void* k1;           // per-head key part: batch, row and head strides (elements); d1 wide
+  const void* k2;           // shared key part: batch and row strides; d2 wide
+  const void* v;            // batch, row and head strides; dv wide
+  const float* sink;        // [H] or null
+  const float* gates;       // [B * T, H] or null
+  const long long* pos;     // device-side position: the first min(*pos + 1, rows) rows are visible (a ring of cap rows)
+  void* out;                // [B * T, out_ld], head h at column h * dv
+  long long k1_batch, k2_batch, v_batch;
+  int k1_row, k1_head, k2_row, v_row, v_head;
+  int d1, d2, dv;           // multiples of 8
+  int batch, heads, seq;    // T new tokens per sequence
+  int rows, prior;          // rows a buffer holds per sequence; query t sits at row prior + t
+  int window;               // <= 0: none
+  int out_ld;
+  float scale;
+};
+
+constexpr float kLog2eF = 1.4426950408889634f;
+
+// One wave per (b, t, h).  Lanes take one key each for the scores of 64 keys and dv / 64 value columns each for the
+// sums.  LDS: q (d1 + d2), output sums (dv), 64 weights.
+template <typename T, typename O>
+__global__ __launch_bounds__(64) void windowed_attention_kernel(WindowedAttention a) {
+  extern __shared__ float sh[];
+  const int lane = threadIdx.x, h = blockIdx.y, m = blockIdx.x, b = m / a.seq, t = m % a.seq;
+  const int dq = a.d1 + a.d2;
+  float* q = sh;
+  float* acc = q + dq;
+  float* weight = acc + a.dv;
+  const T* qsrc = reinterpret_cast<const T*>(a.q) + ((size_t)m * a.heads + h) * dq;
+  for (int i = lane; i < dq; i += 64) q[i] = to_f32(qsrc[i]);
+  for (int i = lane; i < a.dv; i += 64) acc[i] = 0.f;
+  int lo = 0, hi;  // visible rows lo .. hi
+  if (a.pos) {
+    hi = (int)min(max(*a.pos, 0ll), (long long)a.rows - 1);
+  } else {
+    hi = a.prior + t;
+    if (a.window > 0) lo = max(0, hi - a.window + 1);
+  }
+  const T* k1 = reinterpret_cast<const T*>(a.k1) + (size_t)b * a.k1_batch + (size_t)h * a.k1_head;
+  const T* k2 = reinterpret_cast<const T*>(a.k2) + (size_t)b * a.k2_batch;
+  const T* v = reinterpret_cast<const T*>(a.v) + (size_t)b * a.v_batch + (size_t)h * a.v_head;
+  const float scale2 = a.scale * kLog2eF;
+  float mx = a.sink ? a.sink[h] * kLog2eF : -INFINITY, total = a.sink ? 1.f : 0.f;
+  __syncthreads();
+  for (int j0 = lo; j0 <= hi; j0 += 64) {
+    const int j = j0 + lane;
+    float s = -INFINITY;
+    if (j <= hi) {
+      float d = 0.f;
+      const T* kr = k1 + (size_t)j * a.k1_row;
+      for (int i = 0; i < a.d1; i += 4) {
+        const float4 k4 = load4(kr + i);
+        d = fmaf(q[i], k4.x, d); d = fmaf(q[i + 1], k4.y, d); d = fmaf(q[i + 2], k4.z, d); d = fmaf(q[i + 3], k4.w, d);
+      }
+      kr = k2 + (size_t)j * a.k2_row;
+      for (int i = 0; i < a.d2; i += 4) {
+        const float4 k4 = load4(kr + i);
+        const float* q2 = q + a.d1 + i;
+        d = fmaf(q2[0], k4.x, d); d = fmaf(q2[1], k4.y, d); d = fmaf(q2[2], k4.z, d); d = fmaf(q2[3], k4.w, d);
+      }
+      s = d * scale2;
+    }
+    const float m_new = fmaxf(mx, wave_max64(s));
+    const float corr = mx == -INFINITY ? 0.f : exp2f(mx - m_new);
+    const float w = s == -INFINITY ? 0.f : exp2f(s - m_new);
+    total = total * corr + wave_sum64(w);
+    mx = m_new;
+    weight[lane] = w;
+    __syncthreads();
+    const int n = min(64, hi - j0 + 1);
+    for (int i = lane; i < a.dv; i += 64) {
+      float o = acc[i] * corr;
+      for (int jj = 0; jj < n; ++jj) o = fmaf(weight[jj], to_f32(v[(size_t)(j0 + jj) * a.v_row + i]), o);
+      acc[i] = o;
+    }
+    __syncthreads();
+  }
+  const float factor = a.gates ? a.gates[(size_t)m * a.heads + h] : 1.f;
+  O* out = reinterpret_cast<O*>(a.out) + (size_t)m * a.out_ld + (size_t)h * a.dv;
+  for (int i = lane; i < a.dv; i += 64) out[i] = from_f32<O>(acc[i] / total * factor);
+}
+
+// Prompts, bf16.  The structure of attn_prefill_kernel (both products transposed so that no operand changes layout;
+// values read with transposing LDS reads; a row's reference exponent moves only when an exponent outgrows it), with
+//   * a workgroup of 4 waves on 64 U query rows of one (b, h), a wave U groups of 16;
+//   * keys of KS 32-column steps gathered from two places (the head's own columns, then the shared ones; columns past
+//     both are zero) and values of VT 16-column tiles, laid into LDS through registers one block of 64 keys ahead;
+//   * blocks from the first key the workgroup's first query sees to its last query's own;
+//   * the sink as the initial state of the running softmax: reference exponent sink, denominator 1.  Every row then
+//     has a finite reference from the start, also when a whole block lies outside its window.
+// LDS rows are padded: keys by 16 bytes, values by 32.
+template <int KS, int VT, int U>
+__global__ __launch_bounds__(256, (KS + VT > 18) ? 1 : 2) void windowed_prefill_kernel(WindowedAttention a) {
+  constexpr int KC = 4 * KS, VC = 2 * VT;                  // 16-byte chunks per key / value row
+  constexpr int KB = 64 * KS + 16, VB = 32 * VT + 32;      // bytes per LDS row
+  constexpr int kStage = kPfBK * (KB + VB);
+  constexpr int KP = KS, VP = (kPfBK * VC + 255) / 256;    // chunks per thread and block
+  extern __shared__ __attribute__((aligned(1024))) unsigned char lds[];
+  const uint32_t lds0 = (uint32_t)(uintptr_t)(pf_lds_char_t*)lds;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  constexpr int kBQ = 64 * U;
+  // an XCD takes a contiguous eighth of the (b, h) pairs, neighbouring query blocks of a pair (which share keys) together
+  const int qblocks = (a.seq + kBQ - 1) / kBQ, BH = a.batch * a.heads;
+  int qb, bh;
+  if ((BH & 7) == 0) {
+    const int m = (int)(blockIdx.x >> 3);
+    qb = m % qblocks;
+    bh = (int)(blockIdx.x & 7) * (BH >> 3) + m / qblocks;
+  } else {
+    qb = (int)blockIdx.x % qblocks;
+    bh = (int)blockIdx.x / qblocks;
+  }
+  const int b = bh / a.heads, h = bh % a.heads;
+  const int q0 = qb * kBQ;
+  const int total = a.prior + a.seq;
+  const int first_q = a.prior + q0, last_q = min(total, first_q + kBQ) - 1;  // rows of the workgroup's first / last query
+  const int window = a.window > 0 ? a.window : 0x3FFFFFFF;
+  const int lo = max(0, first_q - window + 1) & ~(kPfBK - 1);
+  const int nblk = (last_q - lo) / kPfBK + 1;
+  const int wave_first = first_q + 16 * U * wave, wave_last = wave_first + 16 * U - 1;
+
+  const uint16_t* k1 = reinterpret_cast<const uint16_t*>(a.k1) + (size_t)b * a.k1_batch + (size_t)h * a.k1_head;
+  const uint16_t* k2 = reinterpret_cast<const uint16_t*>(a.k2) + (size_t)b * a.k2_batch;
+  const uint16_t* vv = reinterpret_cast<const uint16_t*>(a.v) + (size_t)b * a.v_batch + (size_t)h * a.v_head;
+  const int c1 = a.d1 >> 3, c2 = c1 + (a.d2 >> 3), cv = a.dv >> 3;
+
+  u32x4_t kraw[KP], vraw[VP];
+  auto fetch = [&](int kb0) {
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int ci = threadIdx.x + 256 * i, c = ci % KC;
+      const int row = min(kb0 + ci / KC, total - 1);  // rows past the end repeat the last one; those keys are masked
+      kraw[i] = u32x4_t{0u, 0u, 0u, 0u};
+      if (c < c2) {
+        const uint16_t* src = c < c1 ? k1 + (size_t)row * a.k1_row + 8 * c : k2 + (size_t)row * a.k2_row + 8 * (c - c1);
+        kraw[i] = *reinterpret_cast<const u32x4_t*>(src);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int ci = threadIdx.x + 256 * i, c = ci % VC;
+      const int row = min(kb0 + ci / VC, total - 1);
+      vraw[i] = u32x4_t{0u, 0u, 0u, 0u};
+      if (ci < kPfBK * VC && c < cv) vraw[i] = *reinterpret_cast<const u32x4_t*>(vv + (size_t)row * a.v_row + 8 * c);
+    }
+  };
+  auto lay_down = [&](int stage) {
+    unsigned char* base = lds + stage * kStage;
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int ci = threadIdx.x + 256 * i;
+      *reinterpret_cast<u32x4_t*>(base + (ci / KC) * KB + 16 * (ci % KC)) = kraw[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int ci = threadIdx.x + 256 * i;
+      if (ci < kPfBK * VC) *reinterpret_cast<u32x4_t*>(base + kPfBK * KB + (ci / VC) * VB + 16 * (ci % VC)) = vraw[i];
+    }
+  };
+  // key fragment (16-key tile jb, step s): row 16 jb + r, columns 32 s + 8 g ..
+  uint32_t k_rd = lds0 + (uint32_t)(r * KB + 16 * g);
+  // value fragment of tile t: this lane addresses 8 bytes (piece r & 3) of key 4 g + (r >> 2)
+  uint32_t v_rd = lds0 + (uint32_t)(kPfBK * KB + (4 * g + (r >> 2)) * VB + 8 * (r & 3));
+
+  fetch(lo);
+  const float scale2 = a.scale * kLog2eF;
+  const float sink2 = a.sink ? a.sink[h] * kLog2eF : -1e30f;
+  float m_run[U], l_run[U];
+  f32x4_t o[U][VT];
+  int qrow[U];
+  u32x4_t qf[U][KS];
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    m_run[u] = sink2;
+    l_run[u] = (a.sink && g == 0) ? 1.f : 0.f;  // (lane sums of a row's four lanes meet at the end)
+#pragma unroll
+    for (int t = 0; t < VT; ++t) o[u][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const int t0 = q0 + 16 * U * wave + 16 * u + r;
+    qrow[u] = a.prior + t0;
+    const uint16_t* qp = reinterpret_cast<const uint16_t*>(a.q) +
+                         (((size_t)b * a.seq + min(t0, a.seq - 1)) * a.heads + h) * (a.d1 + a.d2);
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+      const int c = 4 * s + g;
+      qf[u][s] = u32x4_t{0u, 0u, 0u, 0u};
+      if (c < c2) qf[u][s] = *reinterpret_cast<const u32x4_t*>(qp + 8 * c);
+    }
+  }
+  lay_down(0);
+  if (nblk > 1) fetch(lo + kPfBK);
+  __syncthreads();
+  for (int j = 0; j < nblk; ++j) {
+    // block j is complete in stage j & 1; block j + 1 (in registers) goes into the other stage, last read before the
+    // previous barrier, while block j + 2 starts its flight from memory
+    const int kb0 = lo + j * kPfBK;
+    if (j + 1 < nblk) {
+      lay_down((j + 1) & 1);
+      if (j + 2 < nblk) fetch(kb0 + 2 * kPfBK);
+    }
+    const uint32_t stage = (uint32_t)((j & 1) * kStage);
+    if (kb0 <= wave_last && kb0 + kPfBK - 1 > wave_first - window) {
+      f32x4_t sc[U][4];
+#pragma unroll
+      for (int s = 0; s < KS; ++s) {
+        u32x4_t ka[4];
+#pragma unroll
+        for (int jb = 0; jb < 4; ++jb) ka[jb] = pf_read128(k_rd + stage + (uint32_t)(jb * 16 * KB + 64 * s));
+#pragma unroll
+        for (int jb = 0; jb < 4; ++jb)
+#pragma unroll
+          for (int u = 0; u < U; ++u)
+            sc[u][jb] = mfma16(ka[jb], qf[u][s], s == 0 ? f32x4_t{0.f, 0.f, 0.f, 0.f} : sc[u][jb]);
+      }
+      // masks only where the block reaches past the wave's first query or before its last query's window
+      if (kb0 + kPfBK - 1 > wave_first || kb0 <= wave_last - window) {
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+          for (int jb = 0; jb < 4; ++jb)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              const int key = kb0 + 16 * jb + 4 * g + i;
+              if (key > qrow[u] || key <= qrow[u] - window) sc[u][jb][i] = -INFINITY;
+            }
+      }
+      u32x4_t pf[U][2];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        float p[16], psum = 0.f;
+#pragma unroll
+        for (int e = 0; e < 16; ++e) {
+          p[e] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[u][e >> 2][e & 3], scale2, -m_run[u]));
+          psum += p[e];
+        }
+        if (__builtin_amdgcn_ballot_w64(psum > kPfTrigger) != 0) {
+          float mx = -INFINITY;
+#pragma unroll
+          for (int e = 0; e < 16; ++e) mx = fmaxf(mx, sc[u][e >> 2][e & 3] * scale2);
+          mx = quad_max(mx);
+          const float m_new = mx > m_run[u] + kPfSlack ? mx : m_run[u];
+          const float corr = __builtin_amdgcn_exp2f(m_run[u] - m_new);
+          psum = 0.f;
+#pragma unroll
+          for (int e = 0; e < 16; ++e) {
+            p[e] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[u][e >> 2][e & 3], scale2, -m_new));
+            psum += p[e];
+          }
+          m_run[u] = m_new;
+          l_run[u] *= corr;
+#pragma unroll
+          for (int t = 0; t < VT; ++t) o[u][t] *= corr;
+        }
+        l_run[u] += psum;
+        pf[u][0] = pack8_bf16(&p[0]);
+        pf[u][1] = pack8_bf16(&p[8]);
+      }
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+        for (int t = 0; t < VT; ++t) {
+          const uint32_t at = v_rd + stage + (uint32_t)(hf * 32 * VB + 32 * t);
+          const u32x2_t vlo = pf_read_tr(at), vhi = pf_read_tr(at + (uint32_t)(16 * VB));
+          const u32x4_t vf = {vlo.x, vlo.y, vhi.x, vhi.y};
+#pragma unroll
+          for (int u = 0; u < U; ++u) o[u][t] = mfma16(vf, pf[u][hf], o[u][t]);
+        }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const float l = quad_sum(l_run[u]);
+    const int t0 = qrow[u] - a.prior;
+    if (t0 >= a.seq) continue;
+    const size_t m = (size_t)b * a.seq + t0;
+    const float factor = (a.gates ? a.gates[m * a.heads + h] : 1.f) / l;
+    uint16_t* dst = reinterpret_cast<uint16_t*>(a.out) + m * a.out_ld + (size_t)h * a.dv + 4 * g;
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+      if (16 * t < a.dv)
+        *reinterpret_cast<u32x2_t*>(dst + 16 * t) =
+            u32x2_t{pack2_bf16(o[u][t][0] * factor, o[u][t][1] * factor), pack2_bf16(o[u][t][2] * factor, o[u][t][3] * factor)};
+  }
+}
+
+}  // namespace ajq

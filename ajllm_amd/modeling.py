@@ -19,7 +19,7 @@ Every ``Linear`` is the boundary a ``QuantLinear`` drops into (``quantize_model_
 from __future__ import annotations
 
 import math
-from typing import Any
+from typing import Any, Callable
 
 import torch
 from torch import nn
@@ -68,9 +68,25 @@ class RMSNorm(nn.Module):
         return ((x / rms) * self.weight).to(inputs.dtype)
 
 
-def build_norm(kind: str, d_model: int) -> nn.Module:
+class LayerNorm(nn.Module):
+    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * gain, no bias, computed in fp32 and cast back."""
+
+    def __init__(self, d_model: int, epsilon: float = 1e-5, device=None, dtype=None) -> None:
+        super().__init__()
+        self.epsilon = epsilon
+        self.weight = nn.Parameter(torch.ones(d_model, device=device, dtype=dtype))
+
+    def forward(self, inputs: torch.Tensor) -> torch.Tensor:
+        x = inputs.float()
+        x = x - x.mean(dim=-1, keepdim=True)
+        return ((x / torch.sqrt(x.square().mean(dim=-1, keepdim=True) + self.epsilon)) * self.weight).to(inputs.dtype)
+
+
+def build_norm(kind: str, d_model: int, epsilon: float = 1e-5) -> nn.Module:
     if kind == "rmsnorm":
-        return RMSNorm(d_model)
+        return RMSNorm(d_model, epsilon)
+    if kind == "layernorm":
+        return LayerNorm(d_model, epsilon)
     if kind == "none":
         return nn.Identity()
     raise ValueError(f"Unsupported normalization type: {kind}")
@@ -80,17 +96,34 @@ def silu(inputs: torch.Tensor) -> torch.Tensor:
     return inputs * torch.sigmoid(inputs)
 
 
-class SwiGLU(nn.Module):
-    """w2(silu(w1 x) * w3 x)"""
+ACTIVATIONS = {
+    "silu": silu,
+    "relu": torch.relu,
+    "gelu_tanh": lambda z: 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3))),
+}
 
-    def __init__(self, d_model: int, d_ff: int) -> None:
+
+class GatedFeedForward(nn.Module):
+    """w2(act(w1 x) * w3 x)"""
+
+    def __init__(self, d_model: int, d_ff: int, activation: str = "silu") -> None:
         super().__init__()
+        if activation not in ACTIVATIONS:
+            raise ValueError(f"Unsupported activation: {activation}")
+        self.activation = activation
         self.w1 = Linear(d_model, d_ff)
         self.w2 = Linear(d_ff, d_model)
         self.w3 = Linear(d_model, d_ff)
 
     def forward(self, inputs: torch.Tensor) -> torch.Tensor:
-        return self.w2(silu(self.w1(inputs)) * self.w3(inputs))
+        return self.w2(ACTIVATIONS[self.activation](self.w1(inputs)) * self.w3(inputs))
+
+
+class SwiGLU(GatedFeedForward):
+    """w2(silu(w1 x) * w3 x)"""
+
+    def __init__(self, d_model: int, d_ff: int) -> None:
+        super().__init__(d_model, d_ff, "silu")
 
 
 class SiLUFeedForward(nn.Module):
@@ -110,6 +143,8 @@ def build_feed_forward(kind: str, d_model: int, d_ff: int) -> nn.Module:
         return SwiGLU(d_model, d_ff)
     if kind == "silu":
         return SiLUFeedForward(d_model, d_ff)
+    if kind == "reglu":
+        return GatedFeedForward(d_model, d_ff, "relu")
     raise ValueError(f"Unsupported feed-forward type: {kind}")
 
 
@@ -184,6 +219,41 @@ class KVCache:
         view.position = self.position
         view.slots = self.slots
         return view
+
+
+class RingCache:
+    """Cache of a model whose layer runs keep one row per position and look a bounded number of positions back:
+    ``rings[run]`` is ``[B, capacity, width]``, position p in slot p % capacity, so a run holds its window and no more
+    (``capacities[run] = min(window, max_len)``; a run without a window keeps every position).  A layer that runs
+    several times has a ring per pass.
+
+    The two modes are ``KVCache``'s: dynamic (``length``, calls of any number of tokens) and static (one token per
+    call at the device-side ``position``, fixed shapes for a recorded graph; the caller advances it)."""
+
+    def __init__(self, capacities: list[int], widths: list[int], batch: int, max_len: int, device, dtype) -> None:
+        self.rings = [torch.zeros(batch, rows, width, device=device, dtype=dtype)
+                      for rows, width in zip(capacities, widths)]
+        self.batch = batch
+        self.length = 0
+        self.max_len = max_len
+        self.static = False
+        self.position = torch.zeros(1, dtype=torch.long, device=device)
+
+    def rows(self, start: int, stop: int) -> "RingCache":
+        """A cache over sequences ``start .. stop - 1`` of this one, sharing its storage (dynamic mode, empty)."""
+        view = object.__new__(RingCache)
+        view.rings = [ring[start:stop] for ring in self.rings]
+        view.batch = stop - start
+        view.length = 0
+        view.max_len = self.max_len
+        view.static = False
+        view.position = self.position
+        return view
+
+    def reset(self) -> None:
+        """Give the cache to another sequence: a position is read only after it has been written again."""
+        self.length = 0
+        self.static = False
 
 
 class MultiHeadSelfAttention(nn.Module):
@@ -365,8 +435,28 @@ class TransformerLM(nn.Module):
         return self.lm_head(hidden)
 
 
-def build_model(config: dict[str, Any], vocab_size: int) -> TransformerLM:
-    """Model from a reference-style config dict (keys as in the reference's model YAML)."""
+# architecture name -> builder(config); a model module registers its own
+ARCHITECTURES: dict[str, Callable[[dict[str, Any]], nn.Module]] = {}
+
+
+def register_architecture(name: str):
+    def add(builder):
+        ARCHITECTURES[name] = builder
+        return builder
+    return add
+
+
+def build_model(config: dict[str, Any], vocab_size: int | None = None) -> nn.Module:
+    """Model from a config dict: one that names an ``architecture`` goes to that architecture's builder, any other is
+    a reference-style dict (keys as in the reference's model YAML)."""
+    if "architecture" in config:
+        from . import latent  # noqa: F401  (registers its architectures)
+        name = config["architecture"]
+        if name not in ARCHITECTURES:
+            raise ValueError(f"Unsupported architecture: {name} (known: {', '.join(sorted(ARCHITECTURES))})")
+        return ARCHITECTURES[name](config)
+    if vocab_size is None:
+        raise ValueError("vocab_size is needed for a config without an architecture")
     position = config.get("position_encoding", {})
     normalization = config.get("normalization", {})
     feed_forward = config.get("feed_forward", {})
