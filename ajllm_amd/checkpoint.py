@@ -129,7 +129,7 @@ def load_model(folder: str | Path, device, dtype: torch.dtype = torch.bfloat16) 
     names = model.checkpoint_names()
     with safe_open(str(folder / "model.safetensors"), framework="pt", device="cpu") as f:
         present = set(f.keys())
-        missing, unexpected = set(names.values()) - present, present - set(names.values())
+        missing, unexpected = set(names.values()) - present, present - set(names.values()) - model.ignored_names()
         if missing or unexpected:
             raise ValueError(f"checkpoint and model disagree: missing {sorted(missing)}, unexpected {sorted(unexpected)}")
         state = {key: f.get_tensor(name).to(device=device, dtype=dtype) for key, name in names.items()}

@@ -1483,13 +1483,14 @@ int ajq_attn_step_partial(const float* qkv, const float* cosine, const float* si
 int ajq_greedy_pick(const float* logits, int B, int V, int ld, const float* embedding, int D, float* hidden,
                     int64_t* token, int64_t* out, int out_ld, const int64_t* step, int64_t* advance, uint32_t* ticket,
                     void* stream) {
-  if (!logits || !embedding || !hidden || !token || !out || !step)
-    return fail(AJQ_ERR_NULL, "ajq_greedy_pick: null pointer argument");
+  if (!logits || !token || !out || !step) return fail(AJQ_ERR_NULL, "ajq_greedy_pick: null pointer argument");
+  if ((embedding != nullptr) != (hidden != nullptr))
+    return fail(AJQ_ERR_NULL, "ajq_greedy_pick: embedding and hidden go together (both or neither)");
   if ((advance != nullptr) != (ticket != nullptr))
     return fail(AJQ_ERR_NULL, "ajq_greedy_pick: advance and ticket go together (both or neither)");
-  if (B < 1 || V < 1 || ld < V || ld % 4 != 0 || D < 4 || D % 4 != 0 || out_ld < 1)
+  if (B < 1 || V < 1 || ld < V || ld % 4 != 0 || (embedding && (D < 4 || D % 4 != 0)) || out_ld < 1)
     return fail(AJQ_ERR_SHAPE, "ajq_greedy_pick: unsupported shape (B=%d V=%d ld=%d D=%d out_ld=%d)", B, V, ld, D, out_ld);
-  if (!aligned16(logits) || !aligned16(embedding) || !aligned16(hidden))
+  if (!aligned16(logits) || (embedding && (!aligned16(embedding) || !aligned16(hidden))))
     return fail(AJQ_ERR_ALIGN, "ajq_greedy_pick: logits, embedding and hidden must be 16-byte aligned");
   hipLaunchKernelGGL(greedy_pick_kernel, dim3(B), dim3(1024), 0, (hipStream_t)stream, logits, V, ld, embedding, D, hidden,
                      reinterpret_cast<long long*>(token), reinterpret_cast<long long*>(out), out_ld,

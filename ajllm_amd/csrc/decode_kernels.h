@@ -521,7 +521,7 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(const float* __restrict_
 
 // Greedy choice at the end of a decode step, one workgroup of 1024 threads per sequence:
 // token = argmax(logits[b, 0..V)) (the lowest index among equal maxima, as torch.argmax),
-// written to token[b] and to out[b, *step]; then hidden[b, :] = embedding[token, :], the next
+// written to token[b] and to out[b, *step]; then (with an embedding) hidden[b, :] = embedding[token, :], the next
 // step's input.  With `advance` (two int64 counters, `step` may be one of them) the last workgroup
 // to finish adds one to both; `ticket` is a zeroed word the kernel leaves zeroed.
 __global__ __launch_bounds__(1024) void greedy_pick_kernel(const float* __restrict__ logits, int V, int ld,
@@ -594,6 +594,7 @@ __global__ __launch_bounds__(1024) void greedy_pick_kernel(const float* __restri
       }
     }
   }
+  if (!embedding) return;
   __syncthreads();
   const float4* e4 = reinterpret_cast<const float4*>(embedding + (size_t)chosen * D);
   float4* h4 = reinterpret_cast<float4*>(hidden + (size_t)b * D);

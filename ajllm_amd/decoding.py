@@ -14,12 +14,12 @@ import ctypes
 
 import torch
 
-from . import _lib, modeling
+from . import _lib, latent, modeling
 from .quant import QuantLinear, repack_w4, repack_w8, w4a16_matmul, w8a16_matmul
 
 
 class GraphDecoder:
-    def __init__(self, model: modeling.TransformerLM, batch: int, max_len: int,
+    def __init__(self, model: modeling.TransformerLM | latent.LatentLM, batch: int, max_len: int,
                  kv_dtype: torch.dtype | None = None) -> None:
         if max_len > model.context_length:
             raise ValueError(f"max_len {max_len} exceeds the model's context length {model.context_length}")
@@ -81,7 +81,8 @@ class GraphDecoder:
         """The next token of every row from ``logits`` ``[B, V]`` into ``self.token`` and ``self.out[:, step_index]``
         (greedy: the first maximum; otherwise ``_sample``)."""
         if self.temperature > 0:
-            self._sample(logits.float().contiguous())
+            vocab = logits.shape[1]
+            self._sample(torch.nn.functional.pad(logits.float(), (0, -vocab % 4)).contiguous(), vocab=vocab)
             return
         nxt = torch.argmax(logits, dim=-1, keepdim=True)
         self.out.index_copy_(1, self.step_index, nxt)
@@ -110,15 +111,18 @@ class GraphDecoder:
         for start in range(0, self.batch, step):
             rows = self.cache.rows(start, min(start + step, self.batch))
             parts.append(self.model(prompt[start:start + step], rows, last_token_only=True)[:, -1, :])
-        logits = torch.cat(parts, dim=0)
-        self.cache.length = prompt.shape[1]
+        self._prefilled(torch.cat(parts, dim=0), prompt.shape[1])
+
+    def _prefilled(self, logits: torch.Tensor, prompt_len: int) -> None:
+        """The prompt is in the cache, ``logits`` are its last position's: choose the first new token, go static."""
+        self.cache.length = prompt_len
         self.cache.static = True
-        self.cache.position.fill_(prompt.shape[1])
+        self.cache.position.fill_(prompt_len)
         self.step_index.zero_()
         self._choose(logits)
         self.step_index.add_(1)
         self.produced = 1
-        self.prompt_len = prompt.shape[1]
+        self.prompt_len = prompt_len
 
     def _all_rows_done(self, eos_token_id: int) -> int | None:
         """Number of tokens after which every row has produced ``eos_token_id`` (None: not yet)."""
@@ -529,14 +533,7 @@ class FusedDecoder(GraphDecoder):
             prompt = prompt.to(self.device)
             step = rows_per_pass or self.batch
             logits = torch.cat([self._prefill_rows(prompt[i:i + step], i) for i in range(0, self.batch, step)], dim=0)
-            self.cache.length = prompt.shape[1]
-            self.cache.static = True
-            self.cache.position.fill_(prompt.shape[1])
-            self.step_index.zero_()
-            self._choose(logits)
-            self.step_index.add_(1)
-            self.produced = 1
-            self.prompt_len = prompt.shape[1]
+            self._prefilled(logits, prompt.shape[1])
         torch.index_select(self.embedding, 0, self.token.view(-1), out=self.embedded)
 
     def _prefill_rows(self, prompt: torch.Tensor, first: int) -> torch.Tensor:
@@ -751,11 +748,66 @@ class FusedDecoder(GraphDecoder):
         return self.logits_full[:, : self.vocab]
 
 
+class LatentDecoder(GraphDecoder):
+    """GraphDecoder for a ``latent.LatentLM``, whose step is this library's kernels already: the choice of the token
+    and the step's two counters are one launch as well (``ajq_greedy_pick`` / ``ajq_sample_pick``), and eight steps make
+    a graph.  A prompt may be given in portions of ``tokens_per_pass``."""
+
+    def __init__(self, model: latent.LatentLM, batch: int, max_len: int, kv_dtype: torch.dtype | None = None) -> None:
+        super().__init__(model, batch, max_len, kv_dtype)
+        self.steps_per_graph = 8
+        # cache position and output column advance together, at the end of a step (see FusedDecoder)
+        self.counters = torch.zeros(2, dtype=torch.long, device=self.device)
+        self.ticket = torch.zeros(1, dtype=torch.int32, device=self.device)
+        self.cache.position = self.counters[0:1]
+        self.step_index = self.counters[1:2]
+
+    @torch.no_grad()
+    def prefill(self, prompt: torch.Tensor, rows_per_pass: int | None = None, tokens_per_pass: int | None = None) -> None:
+        if tokens_per_pass is None or tokens_per_pass >= prompt.shape[1]:
+            super().prefill(prompt, rows_per_pass)
+            return
+        if prompt.shape[0] != self.batch or prompt.shape[1] >= self.max_len or tokens_per_pass < 1:
+            raise ValueError("prompt must be [batch, T] with T < max_len")
+        self.cache.static = False
+        prompt = prompt.to(self.device)
+        step, seq, parts = rows_per_pass or self.batch, prompt.shape[1], []
+        for first in range(0, self.batch, step):
+            rows = self.cache.rows(first, min(first + step, self.batch))
+            for at in range(0, seq, tokens_per_pass):
+                last = at + tokens_per_pass >= seq
+                logits = self.model(prompt[first:first + step, at:at + tokens_per_pass], rows, want=[min(tokens_per_pass, seq - at) - 1] if last else [])
+            parts.append(logits[:, -1, :])
+        self._prefilled(torch.cat(parts, dim=0), seq)
+
+    @torch.no_grad()
+    def _step(self) -> None:
+        logits = self._logits()
+        if self.temperature > 0:
+            _lib.check(_lib.load().ajq_sample_pick(
+                logits.data_ptr(), self.batch, logits.shape[1], logits.stride(0), self.temperature,
+                1.0 if self.top_p is None else float(self.top_p), self.uniforms.data_ptr(), self.uniforms.shape[0], None, 0, None,
+                self.token.data_ptr(), self.out.data_ptr(), self.out.shape[1], self.step_index.data_ptr(), self.counters.data_ptr(),
+                self.ticket.data_ptr(), None, _stream()), "sample_pick")
+            return
+        _lib.check(_lib.load().ajq_greedy_pick(
+            logits.data_ptr(), self.batch, logits.shape[1], logits.stride(0), None, 0, None, self.token.data_ptr(),
+            self.out.data_ptr(), self.out.shape[1], self.step_index.data_ptr(), self.counters.data_ptr(), self.ticket.data_ptr(),
+            _stream()), "greedy_pick")
+
+
+def decoder_for(model: torch.nn.Module, fused: bool = False) -> type[GraphDecoder]:
+    """The decoder class that serves ``model``."""
+    if isinstance(model, latent.LatentLM):
+        return LatentDecoder
+    return FusedDecoder if fused else GraphDecoder
+
+
 @torch.no_grad()
-def greedy_decode_graph(model: modeling.TransformerLM, prompt: torch.Tensor, max_new_tokens: int,
+def greedy_decode_graph(model: torch.nn.Module, prompt: torch.Tensor, max_new_tokens: int,
                         fused: bool = False, kv_dtype: torch.dtype | None = None) -> torch.Tensor:
     """``[B, T + new]`` like ``modeling.greedy_decode``, with the per-token step replayed from a graph."""
-    cls = FusedDecoder if fused else GraphDecoder
+    cls = decoder_for(model, fused)
     decoder = cls(model, prompt.shape[0], prompt.shape[1] + max_new_tokens, kv_dtype)
     decoder.prefill(prompt)
     new = decoder.generate(max_new_tokens)

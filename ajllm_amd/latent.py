@@ -239,6 +239,10 @@ class LatentLM(nn.Module):
                 names[key] = f"l{index}.{parts[part]}"
         return names
 
+    def ignored_names(self) -> set[str]:
+        """Tensors a checkpoint may hold that no layer reads: the second norm of a layer without a feed-forward."""
+        return {f"l{i}.norm2" for i, layer in enumerate(self.layers) if layer.feed_forward is None}
+
     def new_cache(self, batch: int, max_len: int | None = None, dtype: torch.dtype | None = None) -> RingCache:
         """An empty cache.  Rows are kept in the activations' dtype."""
         weight = self.token_embeddings.weight

@@ -329,7 +329,8 @@ int ajq_attn_prefill(const float* q, const void* kcache, const void* vcache, int
  * the lowest index among equal maxima: next = argmax(logits[:, -1]) of generate,
  * src/ajllm/generation/generator.py:20-27, sampling.py:9-10), also stored at out[b, *step] (row
  * stride out_ld), and hidden[b, :] = embedding[token[b], :] (Embedding.forward,
- * src/ajllm/modeling/layers.py:52-53), the next step's input.  token, out, step: int64. */
+ * src/ajllm/modeling/layers.py:52-53), the next step's input (embedding and hidden may both be NULL: not
+ * looked up).  token, out, step: int64. */
 int ajq_greedy_pick(const float* logits, int B, int V, int ld, const float* embedding, int D, float* hidden,
                     int64_t* token, int64_t* out, int out_ld, const int64_t* step, int64_t* advance, uint32_t* ticket,
                     void* stream);
