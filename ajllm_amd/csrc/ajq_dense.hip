@@ -93,8 +93,8 @@ int prefill_ks(int d) { const int s = (d + 31) / 32; return s <= 4 ? s : s <= 6 
 int prefill_vt(int dv) { const int t = (dv + 15) / 16; return t <= 2 ? 2 : t <= 4 ? 4 : t <= 6 ? 6 : t <= 8 ? 8 : t <= 16 ? 16 : 0; }
 template <int KS, int VT>
 int launch_prefill(const WindowedAttention& w, hipStream_t stream) {
-  constexpr int U = KS + VT > 18 ? 1 : 2;
-  constexpr int bytes = 2 * kPfBK * (64 * KS + 16 + 32 * VT + 32);
+  constexpr int U = KS + VT > 16 ? 1 : 2;
+  constexpr int bytes = 2 * kPfBK * 128 * prefill_panels(KS, VT);
   auto kernel = windowed_prefill_kernel<KS, VT, U>;
   if (int e = allow_lds(kernel, bytes, "ajqd_windowed_prefill")) return e;
   const long long blocks = (long long)((w.seq + 64 * U - 1) / (64 * U)) * w.batch * w.heads;
@@ -113,7 +113,9 @@ int launch_prefill_vt(int vt, const WindowedAttention& w, hipStream_t stream) {
   }
 }
 
-int latent_tiles(int rankp) { const int t = (rankp + 63) / 64; return t <= 1 ? 1 : t <= 2 ? 2 : t <= 4 ? 4 : t <= 8 ? 8 : 0; }
+// ---- decode attention: (column steps, latent tiles per wave) that hold the widths
+int latent_tiles(int rankp) { const int t = (rankp + 63) / 64; return t <= 2 ? 2 : t <= 4 ? 4 : t <= 8 ? 8 : 0; }
+int latent_steps(int width) { const int s = (width + 31) / 32; return s <= 4 ? 4 : s <= 6 ? 6 : s <= 10 ? 10 : s <= 18 ? 18 : 0; }
 int gemv_waves(int k) { return k >= 2048 ? 8 : k >= 256 ? 4 : 1; }
 
 }  // namespace
@@ -280,7 +282,11 @@ int ajqd_dense_in(const ajqd_dense_in_args* a, void* stream) {
   d.w1 = (const uint16_t*)a->w1; d.w2 = (const uint16_t*)a->w2; d.y1 = a->y1; d.gated = (uint16_t*)a->gated;
   d.batch = a->batch; d.D = a->true_width; d.Dp = a->width; d.tiles1 = a->tiles1; d.tiles2 = a->tiles2;
   d.gated_ld = a->gated_ld; d.act = a->act; d.center = a->center; d.eps = a->eps;
-  const dim3 grid(a->tiles1 + a->tiles2, (a->batch + kGemvBatch - 1) / kGemvBatch);
+  // more than 16 sequences: two batch tiles and (from two tiles of rows on) two row tiles per workgroup
+  const bool wide = a->batch > kGemvBatch;
+  const int block = wide ? 2 * kGemvBatch : kGemvBatch;
+  const int rt = wide && a->tiles1 != 1 && a->tiles2 != 1 ? 2 : 1;
+  const dim3 grid((a->tiles1 + rt - 1) / rt + (a->tiles2 + rt - 1) / rt, (a->batch + block - 1) / block);
   const int bytes = a->x ? 2 * a->batch * (a->width + 8) : 0;
   auto go = [&](auto kernel, int threads) {
     if (int e = allow_lds(kernel, bytes, "ajqd_dense_in")) return e;
@@ -288,10 +294,14 @@ int ajqd_dense_in(const ajqd_dense_in_args* a, void* stream) {
     return check_launch("ajqd_dense_in");
   };
   const int waves = gemv_waves(a->width);
-  if (a->x) return waves == 8 ? go(dense_in_kernel<8, true>, 512) : waves == 4 ? go(dense_in_kernel<4, true>, 256)
-                                                                               : go(dense_in_kernel<1, true>, 64);
-  return waves == 8 ? go(dense_in_kernel<8, false>, 512) : waves == 4 ? go(dense_in_kernel<4, false>, 256)
-                                                                      : go(dense_in_kernel<1, false>, 64);
+  if (a->x) return waves == 8 ? go(dense_in_kernel<8, true, 1, 1>, 512) : waves == 4 ? go(dense_in_kernel<4, true, 1, 1>, 256)
+                                                                                     : go(dense_in_kernel<1, true, 1, 1>, 64);
+  if (rt == 2) return waves == 8 ? go(dense_in_kernel<8, false, 2, 2>, 512) : waves == 4 ? go(dense_in_kernel<4, false, 2, 2>, 256)
+                                                                                         : go(dense_in_kernel<1, false, 2, 2>, 64);
+  if (wide) return waves == 8 ? go(dense_in_kernel<8, false, 1, 2>, 512) : waves == 4 ? go(dense_in_kernel<4, false, 1, 2>, 256)
+                                                                                      : go(dense_in_kernel<1, false, 1, 2>, 64);
+  return waves == 8 ? go(dense_in_kernel<8, false, 1, 1>, 512) : waves == 4 ? go(dense_in_kernel<4, false, 1, 1>, 256)
+                                                                            : go(dense_in_kernel<1, false, 1, 1>, 64);
 }
 
 int ajqd_dense_out(const void* in, const void* w, float* x, const float* again, const float* step, int batch, int k,
@@ -300,12 +310,21 @@ int ajqd_dense_out(const void* in, const void* w, float* x, const float* again, 
   if (batch < 1 || k < 8 || k % 8 || width < 16 || width % 16)
     return fail(AJQ_ERR_SHAPE, "ajqd_dense_out: unsupported shape (batch=%d k=%d width=%d)", batch, k, width);
   DenseOut d{(const uint16_t*)in, (const uint16_t*)w, x, again, step, batch, k, width};
-  const dim3 grid(width / 16, (batch + kGemvBatch - 1) / kGemvBatch);
+  const bool wide = batch > kGemvBatch;
+  const int block = wide ? 2 * kGemvBatch : kGemvBatch;
+  const int rt = wide && width % 32 == 0 && width >= 8192 ? 2 : 1;
+  const dim3 grid(width / (16 * rt), (batch + block - 1) / block);
+  auto go = [&](auto kernel, int threads) {
+    hipLaunchKernelGGL(kernel, grid, dim3(threads), 0, (hipStream_t)stream, d);
+    return check_launch("ajqd_dense_out");
+  };
   const int waves = gemv_waves(k);
-  if (waves == 8) hipLaunchKernelGGL(dense_out_kernel<8>, grid, dim3(512), 0, (hipStream_t)stream, d);
-  else if (waves == 4) hipLaunchKernelGGL(dense_out_kernel<4>, grid, dim3(256), 0, (hipStream_t)stream, d);
-  else hipLaunchKernelGGL(dense_out_kernel<1>, grid, dim3(64), 0, (hipStream_t)stream, d);
-  return check_launch("ajqd_dense_out");
+  if (rt == 2) return waves == 8 ? go(dense_out_kernel<8, 2, 2>, 512) : waves == 4 ? go(dense_out_kernel<4, 2, 2>, 256)
+                                                                                   : go(dense_out_kernel<1, 2, 2>, 64);
+  if (wide) return waves == 8 ? go(dense_out_kernel<8, 1, 2>, 512) : waves == 4 ? go(dense_out_kernel<4, 1, 2>, 256)
+                                                                                : go(dense_out_kernel<1, 1, 2>, 64);
+  return waves == 8 ? go(dense_out_kernel<8, 1, 1>, 512) : waves == 4 ? go(dense_out_kernel<4, 1, 1>, 256)
+                                                                      : go(dense_out_kernel<1, 1, 1>, 64);
 }
 
 int ajqd_latent_absorb(const float* y, int ldy, const ajqd_latent_shape* shape, const void* ukt, const float* latent_gain,
@@ -320,14 +339,14 @@ int ajqd_latent_absorb(const float* y, int ldy, const ajqd_latent_shape* shape, 
   const int groups = (shape->rankp / 16 + 3) / 4;
   LatentAbsorb d{y, (const uint16_t*)ukt, latent_gain, cosine, sine, positions64(pos), (uint16_t*)q, (uint16_t*)ring,
                  batch, ldy, table_rows, cap, groups, device_shape(shape)};
-  hipLaunchKernelGGL(latent_absorb_kernel, dim3(shape->heads * groups + 1, (batch + kGemvBatch - 1) / kGemvBatch), dim3(256), 0,
+  hipLaunchKernelGGL(latent_absorb_kernel, dim3(shape->heads * groups + 4, (batch + kGemvBatch - 1) / kGemvBatch), dim3(256), 0,
                      (hipStream_t)stream, d);
   return check_launch("ajqd_latent_absorb");
 }
 
 int ajqd_latent_decode_chunks(int batch, int heads, int rankp, int rotp, int cap) {
   if (batch < 1 || heads < 1 || cap < 1 || rankp < 16 || rankp % 16 || rotp < 8 || rotp % 8 || !latent_tiles(rankp) ||
-      latent_decode_lds(rankp + rotp) > kLdsLimit - 1024)
+      !latent_steps(rankp + rotp))
     return 0;
   const int tiles = batch * ((heads + 15) / 16);
   int s = (256 + tiles - 1) / tiles;
@@ -341,22 +360,24 @@ int ajqd_latent_decode(const void* q, const void* ring, const int64_t* pos, floa
   if (!q || !ring || !pos || !partial) return fail(AJQ_ERR_NULL, "ajqd_latent_decode: null pointer argument");
   if (ajqd_latent_decode_chunks(batch, heads, rankp, rotp, cap) == 0)
     return fail(AJQ_ERR_UNSUPPORTED, "ajqd_latent_decode: widths %d + %d are not built", rankp, rotp);
-  if (chunks < 1 || chunks > kLatentMaxChunks || batch > 65535 || !(scale > 0.f))
+  if (chunks < 1 || chunks > kLatentMaxChunks || !(scale > 0.f))
     return fail(AJQ_ERR_SHAPE, "ajqd_latent_decode: unsupported shape (batch=%d chunks=%d)", batch, chunks);
-  LatentDecode d{(const uint16_t*)q, (const uint16_t*)ring, positions64(pos), partial, heads, rankp, rankp + rotp, cap, chunks,
-                 scale * kLog2eF};
-  const dim3 grid((heads + 15) / 16, chunks, batch);
-  const int bytes = latent_decode_lds(rankp + rotp);
+  LatentDecode d{(const uint16_t*)q, (const uint16_t*)ring, positions64(pos), partial, batch, heads, rankp, rankp + rotp, cap,
+                 chunks, scale * kLog2eF};
+  const long long blocks = (long long)((heads + 15) / 16) * chunks * batch;
+  if (blocks > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_latent_decode: too many workgroups");
+  const int bytes = latent_decode_lds(rankp);
   auto go = [&](auto kernel) {
     if (int e = allow_lds(kernel, bytes, "ajqd_latent_decode")) return e;
-    hipLaunchKernelGGL(kernel, grid, dim3(256), bytes, (hipStream_t)stream, d);
+    hipLaunchKernelGGL(kernel, dim3((unsigned)blocks), dim3(256), bytes, (hipStream_t)stream, d);
     return check_launch("ajqd_latent_decode");
   };
-  switch (latent_tiles(rankp)) {
-    case 1: return go(latent_decode_kernel<1>);
-    case 2: return go(latent_decode_kernel<2>);
-    case 4: return go(latent_decode_kernel<4>);
-    default: return go(latent_decode_kernel<8>);
+  const int tiles = latent_tiles(rankp);
+  switch (latent_steps(rankp + rotp)) {
+    case 4: return go(latent_decode_kernel<4, 2>);  // (at most 128 columns: two tiles per wave)
+    case 6: return tiles == 2 ? go(latent_decode_kernel<6, 2>) : go(latent_decode_kernel<6, 4>);
+    case 10: return tiles == 2 ? go(latent_decode_kernel<10, 2>) : tiles == 4 ? go(latent_decode_kernel<10, 4>) : go(latent_decode_kernel<10, 8>);
+    default: return tiles == 2 ? go(latent_decode_kernel<18, 2>) : tiles == 4 ? go(latent_decode_kernel<18, 4>) : go(latent_decode_kernel<18, 8>);
   }
 }
 
@@ -367,10 +388,10 @@ int ajqd_latent_expand(const float* partial, const float* sink, const float* gat
       out_ld < heads * vdimp || out_ld % 4)
     return fail(AJQ_ERR_SHAPE, "ajqd_latent_expand: unsupported shape (batch=%d heads=%d chunks=%d rankp=%d vdimp=%d)", batch,
                 heads, chunks, rankp, vdimp);
-  const int groups = (vdimp / 16 + 3) / 4, bytes = 2 * kGemvBatch * (rankp + 8);
-  if (int e = allow_lds(latent_expand_kernel, bytes + 4096, "ajqd_latent_expand")) return e;
+  if (rankp > 32 * kExpandSteps) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_latent_expand: latents of %d are not built", rankp);
+  const int groups = (vdimp / 16 + 7) / 8, bytes = 2 * kExpandBatch * (rankp + 8);
   LatentExpand d{partial, sink, gate, (const uint16_t*)uv, (uint16_t*)out, batch, heads, chunks, rankp, vdimp, gate_ld, out_ld, groups};
-  hipLaunchKernelGGL(latent_expand_kernel, dim3(heads * groups, (batch + kGemvBatch - 1) / kGemvBatch), dim3(256), bytes,
+  hipLaunchKernelGGL(latent_expand_kernel, dim3(heads * groups, (batch + kExpandBatch - 1) / kExpandBatch), dim3(512), bytes,
                      (hipStream_t)stream, d);
   return check_launch("ajqd_latent_expand");
 }

@@ -15,36 +15,45 @@
 // row, two steps a cache line.
 #pragma once
 #include "dense_kernels.h"
-#include "prefill_attention.h"
+#include "latent_attention.h"
 
 namespace ajq {
 
 constexpr int kGemvBatch = 16;
 
-// acc += W[rows of the tile, steps begin .. end) x; `wrow` points at this lane's row, `x(step)` gives its B fragment
-// (batch column r, k = 32 step + 8 g ..), both zero past K.
-template <typename XFn>
-__device__ __forceinline__ f32x4_t tile_steps(const uint16_t* __restrict__ wrow, int K, int begin, int end, int g, f32x4_t acc,
-                                              XFn&& x) {
-  constexpr int kUnroll = 8;
+// acc[n][t] += W[rows of row tile n, steps begin .. end) x_t; `wrow` points at this lane's row of the first tile (a tile is
+// 16 K elements further), `x(t, step)` gives the B fragment of batch tile t (batch column r, k = 32 step + 8 g ..), both
+// zero past K.  A weight fragment meets BT batch tiles, an activation fragment RT row tiles.
+template <int RT, int BT, typename XFn>
+__device__ __forceinline__ void tile_steps(const uint16_t* __restrict__ wrow, int K, int begin, int end, int g,
+                                           f32x4_t (&acc)[RT][BT], XFn&& x) {
+  constexpr int kUnroll = 8 / RT;
   const u32x4_t zero = {0u, 0u, 0u, 0u};
   for (int s0 = begin; s0 < end; s0 += kUnroll) {
-    u32x4_t w[kUnroll], v[kUnroll];
+    u32x4_t w[kUnroll][RT], v[kUnroll][BT];
 #pragma unroll
     for (int i = 0; i < kUnroll; ++i) {
       const int k = 32 * (s0 + i) + 8 * g;
-      w[i] = zero;
-      if (s0 + i < end && k < K) w[i] = *reinterpret_cast<const u32x4_t*>(wrow + k);
+#pragma unroll
+      for (int n = 0; n < RT; ++n) {
+        w[i][n] = zero;
+        if (s0 + i < end && k < K) w[i][n] = *reinterpret_cast<const u32x4_t*>(wrow + (size_t)n * 16 * K + k);
+      }
     }
 #pragma unroll
-    for (int i = 0; i < kUnroll; ++i) {
-      v[i] = zero;
-      if (s0 + i < end && 32 * (s0 + i) + 8 * g < K) v[i] = x(s0 + i);
-    }
+    for (int i = 0; i < kUnroll; ++i)
 #pragma unroll
-    for (int i = 0; i < kUnroll; ++i) acc = mfma16(w[i], v[i], acc);
+      for (int t = 0; t < BT; ++t) {
+        v[i][t] = zero;
+        if (s0 + i < end && 32 * (s0 + i) + 8 * g < K) v[i][t] = x(t, s0 + i);
+      }
+#pragma unroll
+    for (int i = 0; i < kUnroll; ++i)
+#pragma unroll
+      for (int n = 0; n < RT; ++n)
+#pragma unroll
+        for (int t = 0; t < BT; ++t) acc[n][t] = mfma16(w[i][n], v[i][t], acc[n][t]);
   }
-  return acc;
 }
 
 // the K range of one of kWaves waves, in pairs of steps (a cache line of a weight row stays with one wave)
@@ -55,21 +64,29 @@ __device__ __forceinline__ void wave_steps(int K, int wave, int waves, int& begi
   end = min(steps, begin + per);
 }
 
-// sum of the waves' tiles; valid in wave 0
-template <int kWaves>
-__device__ __forceinline__ f32x4_t meet(f32x4_t acc, float* red, int wave, int lane) {
-  if (kWaves == 1) return acc;
+// sum of the waves' tiles; tile (n, t) is valid in wave n BT + t
+template <int kWaves, int RT, int BT>
+__device__ __forceinline__ void meet(f32x4_t (&acc)[RT][BT], float* red, int wave, int lane) {
+  if (kWaves == 1) return;
+  static_assert(kWaves == 1 || RT * BT <= kWaves, "a wave per tile");
   float4* slot = reinterpret_cast<float4*>(red);
-  if (wave > 0) slot[(wave - 1) * 64 + lane] = float4{acc[0], acc[1], acc[2], acc[3]};
-  __syncthreads();
-  if (wave == 0) {
 #pragma unroll
-    for (int w = 0; w < kWaves - 1; ++w) {
-      const float4 o = slot[w * 64 + lane];
-      acc[0] += o.x; acc[1] += o.y; acc[2] += o.z; acc[3] += o.w;
+  for (int i = 0; i < RT * BT; ++i) {
+    const f32x4_t& v = acc[i / BT][i % BT];
+    if (wave != i) slot[(i * kWaves + wave) * 64 + lane] = float4{v[0], v[1], v[2], v[3]};
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < RT * BT; ++i) {
+    if (wave != i) continue;
+    f32x4_t& v = acc[i / BT][i % BT];
+#pragma unroll
+    for (int w = 0; w < kWaves; ++w) {
+      if (w == i) continue;
+      const float4 o = slot[(i * kWaves + w) * 64 + lane];
+      v[0] += o.x; v[1] += o.y; v[2] += o.z; v[3] += o.w;
     }
   }
-  return acc;
 }
 
 struct DenseIn {
@@ -87,19 +104,23 @@ struct DenseIn {
 };
 
 // kNorm: the norm is formed here, for the rows of one batch block (dynamic LDS: rows x (Dp + 8) bf16).
-template <int kWaves, bool kNorm>
+// RT: row tiles per workgroup (grid.x counts workgroups of the first matrix, then of the second), BT: batch tiles.
+template <int kWaves, bool kNorm, int RT, int BT>
 __global__ __launch_bounds__(64 * kWaves) void dense_in_kernel(DenseIn a) {
   extern __shared__ __attribute__((aligned(16))) uint16_t normed[];
-  __shared__ float red[kWaves > 1 ? (kWaves - 1) * 256 : 4];
+  __shared__ __attribute__((aligned(16))) float red[kWaves > 1 ? RT * BT * kWaves * 256 : 4];
   __shared__ float stat[kWaves];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
-  const int b0 = blockIdx.y * kGemvBatch, nb = min(kGemvBatch, a.batch - b0);
-  const bool second = (int)blockIdx.x >= a.tiles1;
-  const int tile = second ? (int)blockIdx.x - a.tiles1 : (int)blockIdx.x;
-  const uint16_t* wrow = (second ? a.w2 : a.w1) + (size_t)(16 * tile + r) * a.Dp;
+  const int b0 = blockIdx.y * kGemvBatch * BT, nb = min(kGemvBatch * BT, a.batch - b0);
+  const int groups1 = (a.tiles1 + RT - 1) / RT;
+  const bool second = (int)blockIdx.x >= groups1;
+  const int tiles = second ? a.tiles2 : a.tiles1;
+  // the last workgroup of an odd matrix overlaps its neighbour: the same rows give the same values twice
+  const int tile0 = max(0, min(RT * (second ? (int)blockIdx.x - groups1 : (int)blockIdx.x), tiles - RT));
+  const uint16_t* wrow = (second ? a.w2 : a.w1) + (size_t)(16 * tile0 + r) * a.Dp;
   int begin, end;
   wave_steps(a.Dp, wave, kWaves, begin, end);
-  f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+  f32x4_t acc[RT][BT] = {};
   if constexpr (kNorm) {
     const float* gain = second ? a.gain2 : a.gain1;
     constexpr int kThreads = 64 * kWaves, kKeep = 4;
@@ -157,30 +178,33 @@ __global__ __launch_bounds__(64 * kWaves) void dense_in_kernel(DenseIn a) {
       for (int i = 4 * (threadIdx.x + kThreads * kKeep); i < a.Dp; i += 4 * kThreads) put(i, load4(x + i));
     }
     __syncthreads();
-    const uint16_t* xr = normed + min(r, nb - 1) * stride + 8 * g;
-    acc = tile_steps(wrow, a.Dp, begin, end, g, acc, [&](int s) {
-      return r < nb ? *reinterpret_cast<const u32x4_t*>(xr + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
+    tile_steps<RT, BT>(wrow, a.Dp, begin, end, g, acc, [&](int t, int s) {
+      const int row = 16 * t + r;
+      return row < nb ? *reinterpret_cast<const u32x4_t*>(normed + row * stride + 8 * g + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
     });
   } else {
-    const uint16_t* xr = (second ? a.n2 : a.n1) + (size_t)(b0 + min(r, nb - 1)) * a.Dp + 8 * g;
-    acc = tile_steps(wrow, a.Dp, begin, end, g, acc, [&](int s) {
-      return r < nb ? *reinterpret_cast<const u32x4_t*>(xr + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
+    const uint16_t* xr = (second ? a.n2 : a.n1) + (size_t)b0 * a.Dp + 8 * g;
+    tile_steps<RT, BT>(wrow, a.Dp, begin, end, g, acc, [&](int t, int s) {
+      const int row = 16 * t + r;
+      return row < nb ? *reinterpret_cast<const u32x4_t*>(xr + (size_t)row * a.Dp + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
     });
   }
-  acc = meet<kWaves>(acc, red, wave, lane);
-  if (wave != 0) return;
-  if (!second) {
-    if (r < nb) *reinterpret_cast<float4*>(a.y1 + (size_t)(b0 + r) * (16 * a.tiles1) + 16 * tile + 4 * g) =
-        float4{acc[0], acc[1], acc[2], acc[3]};
-    return;
-  }
-  // rows 0 .. 7 of the tile (lanes g < 2) are gates, rows 8 .. 15 (lanes g >= 2, 32 lanes on) the matching up rows
-  float v[4];
+  meet<kWaves, RT, BT>(acc, red, wave, lane);
 #pragma unroll
-  for (int i = 0; i < 4; ++i) v[i] = activate(a.act, acc[i]) * __shfl_xor(acc[i], 32);
-  if (g < 2 && r < nb)
-    *reinterpret_cast<u32x2_t*>(a.gated + (size_t)(b0 + r) * a.gated_ld + 8 * tile + 4 * g) =
-        u32x2_t{pack2_bf16(v[0], v[1]), pack2_bf16(v[2], v[3])};
+  for (int i = 0; i < RT * BT; ++i) {
+    if (kWaves > 1 && wave != i) continue;
+    const f32x4_t& sum = acc[i / BT][i % BT];
+    const int row = 16 * (i % BT) + r, tile = tile0 + i / BT;
+    if (!second) {
+      if (row < nb) store4(a.y1 + (size_t)(b0 + row) * (16 * a.tiles1) + 16 * tile + 4 * g, float4{sum[0], sum[1], sum[2], sum[3]});
+      continue;
+    }
+    // rows 0 .. 7 of the tile (lanes g < 2) are gates, rows 8 .. 15 (lanes g >= 2, 32 lanes on) the matching up rows
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = activate(a.act, sum[e]) * __shfl_xor(sum[e], 32);
+    if (g < 2 && row < nb) store4(a.gated + (size_t)(b0 + row) * a.gated_ld + 8 * tile + 4 * g, float4{v[0], v[1], v[2], v[3]});
+  }
 }
 
 struct DenseOut {
@@ -191,34 +215,46 @@ struct DenseOut {
   const float* step;        // [Dp] or null, added too
   int batch, K, Dp;
 };
-template <int kWaves>
+template <int kWaves, int RT, int BT>
 __global__ __launch_bounds__(64 * kWaves) void dense_out_kernel(DenseOut a) {
-  __shared__ float red[kWaves > 1 ? (kWaves - 1) * 256 : 4];
+  __shared__ __attribute__((aligned(16))) float red[kWaves > 1 ? RT * BT * kWaves * 256 : 4];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
-  const int b0 = blockIdx.y * kGemvBatch, nb = min(kGemvBatch, a.batch - b0);
-  const uint16_t* wrow = a.w + (size_t)(16 * blockIdx.x + r) * a.K;
-  const uint16_t* xr = a.in + (size_t)(b0 + min(r, nb - 1)) * a.K + 8 * g;
+  const int b0 = blockIdx.y * kGemvBatch * BT, nb = min(kGemvBatch * BT, a.batch - b0);
+  const int first = blockIdx.x * RT * 16;  // (RT divides the row tiles: x is updated in place)
+  const uint16_t* wrow = a.w + (size_t)(first + r) * a.K;
+  const uint16_t* xr = a.in + (size_t)b0 * a.K + 8 * g;
   int begin, end;
   wave_steps(a.K, wave, kWaves, begin, end);
-  const size_t at = (size_t)(b0 + min(r, nb - 1)) * a.Dp + 16 * blockIdx.x + 4 * g;
-  float4 v = float4{0.f, 0.f, 0.f, 0.f};
-  if (wave == 0) {  // what the product is added to, requested ahead of it
-    v = load4(a.x + at);
+  // what the product of tile i = (row tile, batch tile) is added to, requested ahead of it by the wave that will write it
+  auto place = [&](int i) { return (size_t)(b0 + min(16 * (i % BT) + r, nb - 1)) * a.Dp + first + 16 * (i / BT) + 4 * g; };
+  float4 old[kWaves > 1 ? 1 : RT * BT];
+#pragma unroll
+  for (int i = 0; i < RT * BT; ++i) {
+    if (kWaves > 1 && wave != i) continue;
+    float4 v = load4(a.x + place(i));
     if (a.again) {
-      const float4 e = load4(a.again + at);
+      const float4 e = load4(a.again + place(i));
       v.x += e.x; v.y += e.y; v.z += e.z; v.w += e.w;
     }
     if (a.step) {
-      const float4 e = load4(a.step + 16 * blockIdx.x + 4 * g);
+      const float4 e = load4(a.step + first + 16 * (i / BT) + 4 * g);
       v.x += e.x; v.y += e.y; v.z += e.z; v.w += e.w;
     }
+    old[kWaves > 1 ? 0 : i] = v;
   }
-  f32x4_t acc = tile_steps(wrow, a.K, begin, end, g, f32x4_t{0.f, 0.f, 0.f, 0.f}, [&](int s) {
-    return r < nb ? *reinterpret_cast<const u32x4_t*>(xr + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
+  f32x4_t acc[RT][BT] = {};
+  tile_steps<RT, BT>(wrow, a.K, begin, end, g, acc, [&](int t, int s) {
+    const int row = 16 * t + r;
+    return row < nb ? *reinterpret_cast<const u32x4_t*>(xr + (size_t)row * a.K + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
   });
-  acc = meet<kWaves>(acc, red, wave, lane);
-  if (wave != 0 || r >= nb) return;
-  store4(a.x + at, float4{v.x + acc[0], v.y + acc[1], v.z + acc[2], v.w + acc[3]});
+  meet<kWaves, RT, BT>(acc, red, wave, lane);
+#pragma unroll
+  for (int i = 0; i < RT * BT; ++i) {
+    if ((kWaves > 1 && wave != i) || 16 * (i % BT) + r >= nb) continue;
+    const float4 v = old[kWaves > 1 ? 0 : i];
+    const f32x4_t& sum = acc[i / BT][i % BT];
+    store4(a.x + place(i), float4{v.x + sum[0], v.y + sum[1], v.z + sum[2], v.w + sum[3]});
+  }
 }
 
 struct LatentAbsorb {
@@ -233,7 +269,7 @@ struct LatentAbsorb {
   int batch, ldy, table_rows, cap, groups;  // groups: workgroups per head (4 tiles of 16 latent columns each)
   LatentShape s;
 };
-// Grid (H * groups + 1, batch blocks); the last workgroup of a batch block makes the cache rows.
+// Grid (H * groups + 4, batch blocks); the last four workgroups of a batch block make the cache rows, a wave each.
 __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAbsorb a) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
   const int b0 = blockIdx.y * kGemvBatch, nb = min(kGemvBatch, a.batch - b0);
@@ -242,8 +278,9 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAbsorb a) {
   const int p = clamped_position(a.pos, 0, a.table_rows);
   const float* cs = a.cosine + (size_t)p * (s.rot >> 1);
   const float* sn = a.sine + (size_t)p * (s.rot >> 1);
-  if ((int)blockIdx.x == s.heads * a.groups) {
-    for (int b = wave; b < nb; b += 4) {  // a wave per sequence
+  if ((int)blockIdx.x >= s.heads * a.groups) {
+    const int b = 4 * ((int)blockIdx.x - s.heads * a.groups) + wave;
+    if (b < nb) {
       const float* lat = a.y + (size_t)(b0 + b) * a.ldy + s.heads * dq;
       float ss = 0.f;
       for (int i = 4 * lane; i < s.rankp; i += 256) {  // padding columns are zero
@@ -272,137 +309,140 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAbsorb a) {
   if (16 * tile >= s.rankp) return;
   const uint16_t* wrow = a.ukt + ((size_t)h * s.rankp + 16 * tile + r) * s.dimp;
   const float* xr = a.y + (size_t)(b0 + min(r, nb - 1)) * a.ldy + h * dq + 8 * g;
-  const f32x4_t acc = tile_steps(wrow, s.dimp, 0, (s.dimp + 31) >> 5, g, f32x4_t{0.f, 0.f, 0.f, 0.f}, [&](int st) {
+  f32x4_t acc[1][1] = {};
+  tile_steps<1, 1>(wrow, s.dimp, 0, (s.dimp + 31) >> 5, g, acc, [&](int, int st) {
     if (r >= nb) return u32x4_t{0u, 0u, 0u, 0u};
     const float4 u = load4(xr + 32 * st), v = load4(xr + 32 * st + 4);
     return u32x4_t{pack2_bf16(u.x, u.y), pack2_bf16(u.z, u.w), pack2_bf16(v.x, v.y), pack2_bf16(v.z, v.w)};
   });
   if (r < nb)
-    *reinterpret_cast<u32x2_t*>(a.q + ((size_t)(b0 + r) * s.heads + h) * width + 16 * tile + 4 * g) =
-        u32x2_t{pack2_bf16(acc[0], acc[1]), pack2_bf16(acc[2], acc[3])};
+    store4(a.q + ((size_t)(b0 + r) * s.heads + h) * width + 16 * tile + 4 * g,
+           float4{acc[0][0][0], acc[0][0][1], acc[0][0][2], acc[0][0][3]});
 }
 
 // One chunk of cache rows against 16 heads of one sequence, in the latent space: row j of the ring
-// (latent rankp | rotated rotp) is the key, its latent part the value, for every head.  Blocks of 64 rows are staged in LDS
-// once for both products: S^T = K Q^T (a wave takes 16 keys), then U^T += C^T P^T with the latents read by transposing
-// LDS reads (a wave takes every fourth 16-column tile of the latent).  Grid (head tiles, chunks S, B).
-// Partial result of (b, h, chunk): (maximum, denominator, 0, 0, rankp sums), base-2 exponents.
+// (latent rankp | rotated rotp) is the key, its latent part the value, for every head.  Blocks of 64 rows, a wave 16 of them:
+// the rows are loaded in the layout of the first product's A operand (S^T = K Q^T; KS column steps, queries in registers as
+// well), from there laid into LDS for the second (U^T += C^T P^T, latents read by transposing LDS reads, a wave takes every
+// fourth 16-column tile, RT of them), while the next block is on its way.
+// Partial result of (b, h, chunk): (maximum, denominator, 0, 0, rankp sums), base-2 exponents; zeros for an empty chunk.
+// Grid: chunks of sequences x head tiles; the head tiles of a chunk are 8 workgroups apart, on one XCD and its L2.
 struct LatentDecode {
   const uint16_t* q;        // [B, H, width]
   const uint16_t* ring;     // [B, cap, width]
   const long long* pos;
   float* partial;           // [B, H, S, rankp + 4]
-  int heads, rankp, width, cap, chunks;
+  int batch, heads, rankp, width, cap, chunks;
   float scale2;
 };
-__host__ __device__ constexpr int latent_row_bytes(int width) { return ((width + 31) / 32) * 64 + 16; }
 constexpr int kLatentRows = 64;
 constexpr int kLatentPBytes = (kLatentRows + 8) * 2;
-__host__ __device__ constexpr int latent_decode_lds(int width) {
-  return (kLatentRows + 16) * latent_row_bytes(width) + 16 * kLatentPBytes;
-}
-template <int RT>
-__global__ __launch_bounds__(256) void latent_decode_kernel(LatentDecode a) {
+// bytes of a latent row in LDS: 32 past a multiple of 256, so that eight rows of one 32-byte segment meet every bank once
+__host__ __device__ constexpr int latent_row_bytes(int rankp) { return 2 * rankp + ((32 - 2 * rankp) & 255); }
+__host__ __device__ constexpr int latent_decode_lds(int rankp) { return kLatentRows * latent_row_bytes(rankp) + 16 * kLatentPBytes; }
+template <int KS, int RT>
+__global__ __launch_bounds__(256, 2) void latent_decode_kernel(LatentDecode a) {
   extern __shared__ __attribute__((aligned(1024))) unsigned char lds[];
   __shared__ float smax[4][16], ssum[4][16];
   const uint32_t lds0 = (uint32_t)(uintptr_t)(pf_lds_char_t*)lds;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r = lane & 15, g = lane >> 4;
-  const int b = blockIdx.z, h0 = 16 * blockIdx.x, chunk = blockIdx.y;
-  const int rb = latent_row_bytes(a.width), steps = (a.width + 31) >> 5, kc = 4 * steps, cw = a.width >> 3;
+  const int head_tiles = (a.heads + 15) >> 4, units = a.batch * a.chunks;
+  int unit, tile;
+  if ((units & 7) == 0) {
+    const int m = (int)(blockIdx.x >> 3);
+    tile = m % head_tiles;
+    unit = 8 * (m / head_tiles) + (int)(blockIdx.x & 7);
+  } else {
+    tile = (int)blockIdx.x % head_tiles;
+    unit = (int)blockIdx.x / head_tiles;
+  }
+  const int b = unit / a.chunks, chunk = unit % a.chunks, h0 = 16 * tile;
+  const int rb = latent_row_bytes(a.rankp), cw = a.width >> 3;
   const int valid = (int)min(max(*a.pos, 0ll), (long long)a.cap - 1) + 1;  // rows the ring holds
   const int per = (((valid + a.chunks - 1) / a.chunks) + kLatentRows - 1) & ~(kLatentRows - 1);
   const int begin = chunk * per, end = min(valid, begin + per);
   float* head_out = a.partial + (((size_t)b * a.heads + min(h0 + r, a.heads - 1)) * a.chunks + chunk) * (a.rankp + 4);
-  if (begin >= end) {
-    if (wave == 0 && g == 0 && h0 + r < a.heads) *reinterpret_cast<float4*>(head_out) = float4{-INFINITY, 0.f, 0.f, 0.f};
-    return;
-  }
   const u32x4_t zero = {0u, 0u, 0u, 0u};
-  const uint32_t q_at = (uint32_t)(kLatentRows * rb), p_at = q_at + (uint32_t)(16 * rb);
-  for (int ci = threadIdx.x; ci < 16 * kc; ci += 256) {
-    const int row = ci / kc, c = ci % kc;
-    u32x4_t v = zero;
-    if (h0 + row < a.heads && c < cw)
-      v = *reinterpret_cast<const u32x4_t*>(a.q + ((size_t)b * a.heads + h0 + row) * a.width + 8 * c);
-    *reinterpret_cast<u32x4_t*>(lds + q_at + row * rb + 16 * c) = v;
-  }
-  const uint16_t* ring = a.ring + (size_t)b * a.cap * a.width;
   float m = -INFINITY, l = 0.f;
-  f32x4_t u[RT];
+  f32x4_t u[RT] = {};
+  if (begin < end) {
+    const uint16_t* ring = a.ring + (size_t)b * a.cap * a.width;
+    u32x4_t kf[KS], qf[KS];
+    // rows past the end repeat the last one (those keys are masked), chunks past the width the last one (zero query columns)
+    auto fetch = [&](int j0) {
+      const uint32_t row = (uint32_t)min(j0 + 16 * wave + r, end - 1) * (uint32_t)a.width;
 #pragma unroll
-  for (int t = 0; t < RT; ++t) u[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  for (int j0 = begin; j0 < end; j0 += kLatentRows) {
-    constexpr int kFly = 6;
-    for (int c0 = 0; c0 < kLatentRows * kc; c0 += 256 * kFly) {
-      u32x4_t v[kFly];
+      for (int s = 0; s < KS; ++s) kf[s] = *reinterpret_cast<const u32x4_t*>(ring + row + (uint32_t)min(32 * s + 8 * g, a.width - 8));
+    };
+    fetch(begin);
+    const uint16_t* qsrc = a.q + ((size_t)b * a.heads + min(h0 + r, a.heads - 1)) * a.width + 8 * g;
 #pragma unroll
-      for (int i = 0; i < kFly; ++i) {
-        const int ci = c0 + 256 * i + threadIdx.x, row = ci / kc, c = ci % kc;
-        v[i] = zero;
-        if (row < kLatentRows && j0 + row < end && c < cw)
-          v[i] = *reinterpret_cast<const u32x4_t*>(ring + (size_t)(j0 + row) * a.width + 8 * c);
-      }
-#pragma unroll
-      for (int i = 0; i < kFly; ++i) {
-        const int ci = c0 + 256 * i + threadIdx.x, row = ci / kc, c = ci % kc;
-        if (row < kLatentRows) *reinterpret_cast<u32x4_t*>(lds + row * rb + 16 * c) = v[i];
-      }
+    for (int s = 0; s < KS; ++s) {
+      qf[s] = zero;
+      if (4 * s + g < cw) qf[s] = *reinterpret_cast<const u32x4_t*>(qsrc + 32 * s);
     }
-    __syncthreads();
-    f32x4_t sc = {0.f, 0.f, 0.f, 0.f};
-    const uint32_t k_rd = lds0 + (uint32_t)((16 * wave + r) * rb + 16 * g), q_rd = lds0 + q_at + (uint32_t)(r * rb + 16 * g);
-
-    for (int s = 0; s < steps; ++s) sc = mfma16(pf_read128(k_rd + 64u * s), pf_read128(q_rd + 64u * s), sc);
-    // sc[i]: key j0 + 16 wave + 4 g + i, head h0 + r
-    float mx = -INFINITY;
+    const uint32_t p_at = (uint32_t)(kLatentRows * rb);
+    for (int j0 = begin; j0 < end; j0 += kLatentRows) {
+      f32x4_t sc[2] = {};
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      sc[i] = j0 + 16 * wave + 4 * g + i < end ? sc[i] * a.scale2 : -INFINITY;
-      mx = fmaxf(mx, sc[i]);
-    }
-    mx = quad_max(mx);
-    if (g == 0) smax[wave][r] = mx;
-    __syncthreads();
-    // (finite: the block's first row is valid)
-    const float m_new = fmaxf(fmaxf(fmaxf(smax[0][r], smax[1][r]), fmaxf(smax[2][r], smax[3][r])), m);
-    const float corr = exp2f(m - m_new);
-    m = m_new;
-    float p[4];
+      for (int s = 0; s < KS; ++s) sc[s & 1] = mfma16(kf[s], qf[s], sc[s & 1]);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) p[i] = exp2f(sc[i] - m);
-    l = l * corr + ((p[0] + p[1]) + (p[2] + p[3]));
-    *reinterpret_cast<u32x2_t*>(lds + p_at + r * kLatentPBytes + 2 * (16 * wave + 4 * g)) =
-        u32x2_t{pack2_bf16(p[0], p[1]), pack2_bf16(p[2], p[3])};
+      for (int s = 0; s < KS; ++s)
+        if (4 * s + g < (a.rankp >> 3)) *reinterpret_cast<u32x4_t*>(lds + (16 * wave + r) * rb + 64 * s + 16 * g) = kf[s];
+      if (j0 + kLatentRows < end) fetch(j0 + kLatentRows);
+      // score i: key j0 + 16 wave + 4 g + i, head h0 + r
+      float p[4], mx = -INFINITY;
 #pragma unroll
-    for (int t = 0; t < RT; ++t) u[t] *= corr;
-    __syncthreads();
+      for (int i = 0; i < 4; ++i) {
+        p[i] = j0 + 16 * wave + 4 * g + i < end ? (sc[0][i] + sc[1][i]) * a.scale2 : -INFINITY;
+        mx = fmaxf(mx, p[i]);
+      }
+      mx = quad_max(mx);
+      if (g == 0) smax[wave][r] = mx;
+      __syncthreads();
+      // (finite: the block's first row is valid)
+      const float m_new = fmaxf(fmaxf(fmaxf(smax[0][r], smax[1][r]), fmaxf(smax[2][r], smax[3][r])), m);
+      const float corr = exp2f(m - m_new);
+      m = m_new;
 #pragma unroll
-    for (int hf = 0; hf < 2; ++hf) {
-      const unsigned char* pr = lds + p_at + r * kLatentPBytes + 2 * (32 * hf + 4 * g);
-      const u32x2_t plo = *reinterpret_cast<const u32x2_t*>(pr), phi = *reinterpret_cast<const u32x2_t*>(pr + 32);
-      const u32x4_t pf = {plo.x, plo.y, phi.x, phi.y};
+      for (int i = 0; i < 4; ++i) p[i] = exp2f(p[i] - m);
+      l = l * corr + ((p[0] + p[1]) + (p[2] + p[3]));
+      store4(reinterpret_cast<uint16_t*>(lds + p_at + r * kLatentPBytes) + 16 * wave + 4 * g, float4{p[0], p[1], p[2], p[3]});
 #pragma unroll
-      for (int t = 0; t < RT; ++t) {
-        const int tile = wave + 4 * t;
-        if (16 * tile < a.rankp) {
-          const uint32_t at = lds0 + (uint32_t)((32 * hf + 4 * g + (r >> 2)) * rb + 32 * tile + 8 * (r & 3));
-          const u32x2_t lo = pf_read_tr(at), hi = pf_read_tr(at + (uint32_t)(16 * rb));
-          u[t] = mfma16(u32x4_t{lo.x, lo.y, hi.x, hi.y}, pf, u[t]);
+      for (int t = 0; t < RT; ++t) u[t] *= corr;
+      __syncthreads();
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf) {
+        const unsigned char* pr = lds + p_at + r * kLatentPBytes + 2 * (32 * hf + 4 * g);
+        const u32x2_t plo = *reinterpret_cast<const u32x2_t*>(pr), phi = *reinterpret_cast<const u32x2_t*>(pr + 32);
+        const u32x4_t pf = {plo.x, plo.y, phi.x, phi.y};
+        const uint32_t at = lds0 + (uint32_t)((32 * hf + 4 * g + (r >> 2)) * rb + 32 * wave + 8 * (r & 3));
+        // (tiles past the latent read what else lies in LDS; their sums are not written)
+#pragma unroll
+        for (int t0 = 0; t0 < RT; t0 += 2) {
+          u32x2_t lo[2], hi[2];
+#pragma unroll
+          for (int t = 0; t < 2; ++t) {
+            lo[t] = pf_read_tr(at + 128u * (t0 + t));
+            hi[t] = pf_read_tr(at + 128u * (t0 + t) + (uint32_t)(16 * rb));
+          }
+#pragma unroll
+          for (int t = 0; t < 2; ++t) u[t0 + t] = mfma16(u32x4_t{lo[t].x, lo[t].y, hi[t].x, hi[t].y}, pf, u[t0 + t]);
         }
       }
+      __syncthreads();
     }
+    l = quad_sum(l);
+    if (g == 0) ssum[wave][r] = l;
     __syncthreads();
+    l = (ssum[0][r] + ssum[1][r]) + (ssum[2][r] + ssum[3][r]);
   }
-  l = quad_sum(l);
-  if (g == 0) ssum[wave][r] = l;
-  __syncthreads();
   if (h0 + r >= a.heads) return;
-  if (wave == 0 && g == 0)
-    *reinterpret_cast<float4*>(head_out) = float4{m, (ssum[0][r] + ssum[1][r]) + (ssum[2][r] + ssum[3][r]), 0.f, 0.f};
+  if (wave == 0 && g == 0) store4(head_out, float4{m, l, 0.f, 0.f});
 #pragma unroll
   for (int t = 0; t < RT; ++t) {
-    const int tile = wave + 4 * t;
-    if (16 * tile < a.rankp) store4(head_out + 4 + 16 * tile + 4 * g, float4{u[t][0], u[t][1], u[t][2], u[t][3]});
+    const int col = 16 * (wave + 4 * t);
+    if (col < a.rankp) store4(head_out + 4 + col + 4 * g, float4{u[t][0], u[t][1], u[t][2], u[t][3]});
   }
 }
 
@@ -412,53 +452,89 @@ struct LatentExpand {
   const float* gate;        // gate projections, [b * gate_ld + h], or null
   const uint16_t* uv;       // [H, vdimp, rankp]
   uint16_t* out;            // [B, out_ld], head h at column h * vdimp
-  int batch, heads, chunks, rankp, vdimp, gate_ld, out_ld, groups;  // groups: workgroups per head (4 tiles each)
+  int batch, heads, chunks, rankp, vdimp, gate_ld, out_ld, groups;  // groups: workgroups per head (8 tiles each)
 };
-constexpr int kLatentMaxChunks = 32;
-// Grid (H * groups, batch blocks).  Dynamic LDS: 16 x (rankp + 8) bf16 of merged sums.
-__global__ __launch_bounds__(256) void latent_expand_kernel(LatentExpand a) {
-  extern __shared__ __attribute__((aligned(16))) uint16_t merged[];
-  __shared__ float weight[kGemvBatch][kLatentMaxChunks];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
-  const int b0 = blockIdx.y * kGemvBatch, nb = min(kGemvBatch, a.batch - b0);
-  const int h = blockIdx.x / a.groups, grp = blockIdx.x % a.groups;
+constexpr int kLatentMaxChunks = 32, kExpandBatch = 4, kExpandSteps = 16;  // rankp <= 32 kExpandSteps
+// A workgroup of 8 waves per (head, 4 sequences): the chunks are merged by all threads, then every wave expands the merged
+// latents to 16 value columns; its weights are requested first.  Grid (H * groups, batch blocks).
+__global__ __launch_bounds__(512) void latent_expand_kernel(LatentExpand a) {
+  extern __shared__ __attribute__((aligned(16))) uint16_t merged[];   // [kExpandBatch][rankp + 8] bf16
+  __shared__ float weight[kExpandBatch][kLatentMaxChunks];
+  __shared__ float4 part[512];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
+  const int b0 = blockIdx.y * kExpandBatch, nb = min(kExpandBatch, a.batch - b0);
+  const int h = blockIdx.x / a.groups, tile = 8 * (blockIdx.x % a.groups) + wave;
   const int stride = a.rankp + 4, ld = a.rankp + 8;
-  for (int b = wave; b < nb; b += 4) {  // a wave per sequence, a lane per chunk
-    const float* src = a.partial + ((size_t)(b0 + b) * a.heads + h) * a.chunks * stride;
+  const u32x4_t zero = {0u, 0u, 0u, 0u};
+  const bool active = 16 * tile < a.vdimp;
+  u32x4_t w[kExpandSteps];
+  const uint16_t* wrow = a.uv + ((size_t)h * a.vdimp + (active ? 16 * tile : 0) + r) * a.rankp + 8 * g;
+#pragma unroll
+  for (int s = 0; s < kExpandSteps; ++s) {
+    w[s] = zero;
+    if (active && 32 * s + 8 * g < a.rankp) w[s] = *reinterpret_cast<const u32x4_t*>(wrow + 32 * s);
+  }
+  // merged[b] = sum over chunks; the threads of a column quad split the chunks where there are more threads than quads.
+  // The first chunks' sums are requested before the chunks' weights are known.
+  const int quads = a.rankp >> 2, items = nb * quads;
+  const int split = items <= 128 ? 4 : items <= 256 ? 2 : 1, span = 512 / split;
+  const int which = tid / span;
+  constexpr int kAhead = 8;
+  float4 ahead[kAhead];
+  auto request = [&](int i, int s0) {
+    const int b = min(i / quads, nb - 1), c = 4 * (i % quads);
+    const float* src = a.partial + ((size_t)(b0 + b) * a.heads + h) * a.chunks * stride + 4 + c;
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) ahead[k] = load4(src + (size_t)min(s0 + k * split, a.chunks - 1) * stride);
+  };
+  request(tid % span, which);
+  if (wave < nb) {  // a wave per sequence, a lane per chunk
+    const float* src = a.partial + ((size_t)(b0 + wave) * a.heads + h) * a.chunks * stride;
     const bool mine = lane < a.chunks;
     const float mx = mine ? src[lane * stride] : -INFINITY, sum = mine ? src[lane * stride + 1] : 0.f;
-    const float sink2 = a.sink ? a.sink[h] * 1.4426950408889634f : -INFINITY;
+    const float sink2 = a.sink ? a.sink[h] * kLog2eF : -INFINITY;
     const float top = fmaxf(wave_max64(mx), sink2);
-    const float w = mx == -INFINITY ? 0.f : exp2f(mx - top);
-    const float total = wave_sum64(sum * w) + (a.sink ? exp2f(sink2 - top) : 0.f);
-    if (mine) weight[b][lane] = w / total;
+    const float e = mx == -INFINITY ? 0.f : exp2f(mx - top);
+    const float total = wave_sum64(sum * e) + (a.sink ? exp2f(sink2 - top) : 0.f);
+    if (lane < kLatentMaxChunks) weight[wave][lane] = mine ? e / total : 0.f;
   }
   __syncthreads();
-  const int quads = a.rankp >> 2;
-  for (int i = threadIdx.x; i < nb * quads; i += 256) {
-    const int b = i / quads, c = 4 * (i % quads);
-    const float* src = a.partial + ((size_t)(b0 + b) * a.heads + h) * a.chunks * stride + 4 + c;
+  for (int i0 = 0; i0 < items; i0 += span) {
+    const int i = i0 + tid % span, b = min(i / quads, nb - 1);
     float4 sum = float4{0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < a.chunks; ++s) {
-      const float w = weight[b][s];
-      if (w == 0.f) continue;  // an empty chunk left no sums
-      const float4 v = load4(src + (size_t)s * stride);
-      sum.x = fmaf(v.x, w, sum.x); sum.y = fmaf(v.y, w, sum.y); sum.z = fmaf(v.z, w, sum.z); sum.w = fmaf(v.w, w, sum.w);
+    for (int s0 = which; s0 < a.chunks; s0 += kAhead * split) {
+      if (i0 > 0 || s0 > which) request(i, s0);
+#pragma unroll
+      for (int k = 0; k < kAhead; ++k) {
+        const int s = s0 + k * split;
+        const float f = s < a.chunks ? weight[b][s] : 0.f;
+        const float4 v = ahead[k];
+        sum.x = fmaf(v.x, f, sum.x); sum.y = fmaf(v.y, f, sum.y); sum.z = fmaf(v.z, f, sum.z); sum.w = fmaf(v.w, f, sum.w);
+      }
     }
-    store4(merged + b * ld + c, sum);
+    if (split > 1) {  // (one round: items <= span)
+      part[tid] = sum;
+      __syncthreads();
+      for (int o = 1; o < split; ++o) {
+        const float4 v = part[(tid + o * span) & 511];
+        sum.x += v.x; sum.y += v.y; sum.z += v.z; sum.w += v.w;
+      }
+    }
+    if (which == 0 && i < items) store4(merged + b * ld + 4 * (i % quads), sum);
   }
   __syncthreads();
-  const int tile = 4 * grp + wave;
-  if (16 * tile >= a.vdimp) return;
-  const uint16_t* wrow = a.uv + ((size_t)h * a.vdimp + 16 * tile + r) * a.rankp;
-  const uint16_t* xr = merged + min(r, nb - 1) * ld + 8 * g;
-  const f32x4_t acc = tile_steps(wrow, a.rankp, 0, (a.rankp + 31) >> 5, g, f32x4_t{0.f, 0.f, 0.f, 0.f}, [&](int s) {
-    return r < nb ? *reinterpret_cast<const u32x4_t*>(xr + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
-  });
+  if (!active) return;
+  f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int s = 0; s < kExpandSteps; ++s) {
+    u32x4_t v = zero;
+    if (r < nb && 32 * s + 8 * g < a.rankp) v = *reinterpret_cast<const u32x4_t*>(merged + r * ld + 32 * s + 8 * g);
+    acc = mfma16(w[s], v, acc);
+  }
   if (r >= nb) return;
   const float f = a.gate ? sigmoid_f32(a.gate[(size_t)(b0 + r) * a.gate_ld + h]) : 1.f;
-  *reinterpret_cast<u32x2_t*>(a.out + (size_t)(b0 + r) * a.out_ld + (size_t)h * a.vdimp + 16 * tile + 4 * g) =
-      u32x2_t{pack2_bf16(acc[0] * f, acc[1] * f), pack2_bf16(acc[2] * f, acc[3] * f)};
+  store4(a.out + (size_t)(b0 + r) * a.out_ld + (size_t)h * a.vdimp + 16 * tile + 4 * g,
+         float4{acc[0] * f, acc[1] * f, acc[2] * f, acc[3] * f});
 }
 
 }  // namespace ajq

@@ -8,6 +8,8 @@
 // Padding: every width a kernel sees is a multiple of 8; columns past the model's own width hold
 // zeros (the packed weights have zero rows and columns there), and statistics divide by the true width.
 #pragma once
+#include <type_traits>
+
 #include "ajq_common.h"
 
 namespace ajq {
@@ -182,6 +184,29 @@ __device__ __forceinline__ float rotated(const Y* v, int i, int rot, const float
   if (i < half) return to_f32(v[i]) * cosine[i] - to_f32(v[i + half]) * sine[i];
   return to_f32(v[i]) * cosine[i - half] + to_f32(v[i - half]) * sine[i - half];
 }
+// `count` vectors rotated by the threads of a workgroup, vector n from src(n) to dst(n) (rotp slots): four pairs per
+// thread where the halves allow it, one component otherwise.
+template <typename Src, typename Dst>
+__device__ __forceinline__ void rotate_all(int count, int rot, int rotp, const float* cosine, const float* sine, int tid,
+                                           int threads, Src&& src, Dst&& dst) {
+  const int half = rot >> 1;
+  if ((half & 3) == 0 && rot == rotp) {
+    const int quads = half >> 2;
+    for (int i = tid; i < count * quads; i += threads) {
+      const int n = i / quads, e = 4 * (i % quads);
+      const float4 a = load4(src(n) + e), b = load4(src(n) + half + e), c = load4(cosine + e), s = load4(sine + e);
+      store4(dst(n) + e, float4{a.x * c.x - b.x * s.x, a.y * c.y - b.y * s.y, a.z * c.z - b.z * s.z, a.w * c.w - b.w * s.w});
+      store4(dst(n) + half + e, float4{b.x * c.x + a.x * s.x, b.y * c.y + a.y * s.y, b.z * c.z + a.z * s.z, b.w * c.w + a.w * s.w});
+    }
+  } else {
+    for (int i = tid; i < count * rotp; i += threads) {
+      const int n = i / rotp, e = i % rotp;
+      const float v = rotated(src(n), e, rot, cosine, sine);
+      auto* to = dst(n) + e;
+      *to = from_f32<typename std::remove_reference<decltype(*to)>::type>(v);
+    }
+  }
+}
 
 // Projection row y[m] = (q: heads x (dimp | rotp), latent: rankp | rotp, gates: heads) of token m = (b, t):
 //   qu[m, h, 0..dimp)  = unrotated query part             (row stride qu_ld per head)
@@ -206,23 +231,26 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const Y* __restrict__
   const int dq = s.dimp + s.rotp, rot_pairs = s.rot >> 1;
   const float* cs = cosine + (size_t)p * rot_pairs;
   const float* sn = sine + (size_t)p * rot_pairs;
-  for (int i = tid; i < s.heads * dq; i += 256) {
-    const int h = i / dq, d = i % dq;
-    if (d < s.dimp)
-      qu[((size_t)m * s.heads + h) * qu_ld + d] = from_f32<T>(to_f32(row[i]));
-    else
-      qr[((size_t)m * s.heads + h) * qr_ld + (d - s.dimp)] = from_f32<T>(rotated(row + h * dq + s.dimp, d - s.dimp, s.rot, cs, sn));
+  const int quads = s.dimp >> 2;
+  for (int i = tid; i < s.heads * quads; i += 256) {
+    const int h = i / quads, d = 4 * (i % quads);
+    store4(qu + ((size_t)m * s.heads + h) * qu_ld + d, load4(row + h * dq + d));
   }
+  rotate_all(s.heads, s.rot, s.rotp, cs, sn, tid, 256, [&](int h) { return row + h * dq + s.dimp; },
+             [&](int h) { return qr + ((size_t)m * s.heads + h) * qr_ld; });
   const Y* lat = row + s.heads * dq;
   float ss = 0.f;
-  for (int i = tid; i < s.rank; i += 256) {
-    const float v = to_f32(lat[i]);
-    ss += v * v;
+  for (int i = 4 * tid; i < s.rankp; i += 1024) {  // padding columns are zero
+    const float4 v = load4(lat + i);
+    ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
   }
   const Divisor by(sqrtf(block_sum256(ss, part) / (float)s.rank + s.eps));
   T* dst = rows + (size_t)b * rows_batch + (size_t)slot * (s.rankp + s.rotp);
-  for (int i = tid; i < s.rankp; i += 256) dst[i] = from_f32<T>(by.divide(to_f32(lat[i])) * latent_gain[i]);
-  for (int i = tid; i < s.rotp; i += 256) dst[s.rankp + i] = from_f32<T>(rotated(lat + s.rankp, i, s.rot, cs, sn));
+  for (int i = 4 * tid; i < s.rankp; i += 1024) {
+    const float4 v = load4(lat + i), w = load4(latent_gain + i);
+    store4(dst + i, float4{by.divide(v.x) * w.x, by.divide(v.y) * w.y, by.divide(v.z) * w.z, by.divide(v.w) * w.w});
+  }
+  rotate_all(1, s.rot, s.rotp, cs, sn, tid, 256, [&](int) { return lat + s.rankp; }, [&](int) { return dst + s.rankp; });
   for (int h = tid; h < s.heads; h += 256) gates[(size_t)m * s.heads + h] = sigmoid_f32(to_f32(lat[s.rankp + s.rotp + h]));
 }
 

@@ -13,7 +13,7 @@
 // Scores, weights and sums are fp32; exponents are taken in base 2, scores multiplied by scale * log2(e).
 #pragma once
 #include "dense_kernels.h"
-#include "prefill_attention.h"
+#include "prefill_attention.h"  // also dma16, the fragment reads and quad_max / quad_sum
 
 namespace ajq {
 
@@ -102,21 +102,36 @@ __global__ __launch_bounds__(64) void windowed_attention_kernel(WindowedAttentio
   for (int i = lane; i < a.dv; i += 64) out[i] = from_f32<O>(acc[i] / total * factor);
 }
 
+// global -> LDS without registers (16 bytes per lane, a wave's 1 KiB contiguous in LDS), every lane with an address of
+// its own; the caller orders its completion with an explicit s_waitcnt vmcnt before a barrier (see dma16)
+#pragma clang diagnostic push
+#pragma clang diagnostic ignored "-Winline-asm"  // m0 is named as clobbered on purpose
+__device__ __forceinline__ void dma16_gather(const void* src, uint32_t lds_addr) {
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off"
+               :
+               : "s"(lds_addr), "v"(src)
+               : "memory", "m0");
+}
+#pragma clang diagnostic pop
+
 // Prompts, bf16.  The structure of attn_prefill_kernel (both products transposed so that no operand changes layout;
 // values read with transposing LDS reads; a row's reference exponent moves only when an exponent outgrows it), with
 //   * a workgroup of 4 waves on 64 U query rows of one (b, h), a wave U groups of 16;
 //   * keys of KS 32-column steps gathered from two places (the head's own columns, then the shared ones; columns past
-//     both are zero) and values of VT 16-column tiles, laid into LDS through registers one block of 64 keys ahead;
+//     both meet zero query columns) and values of VT 16-column tiles, one block of 64 rows ahead by DMA;
 //   * blocks from the first key the workgroup's first query sees to its last query's own;
 //   * the sink as the initial state of the running softmax: reference exponent sink, denominator 1.  Every row then
 //     has a finite reference from the start, also when a whole block lies outside its window.
-// LDS rows are padded: keys by 16 bytes, values by 32.
+// LDS holds key and value rows in panels of 128 bytes (64 rows x 8 chunks of 16 bytes = 8 KiB, keys first):
+//   key panel:   chunk c of row k in slot c ^ ((k >> 1) & 7)
+//   value panel: the two chunks of 32-byte segment v of row k in segment slot v ^ ((k >> 1) & 3)
+// so that a fragment read (16 rows of one chunk, or 8 rows of one segment) meets every bank once.  A DMA request fills 8
+// rows of a panel; wave w takes requests w and w + 4, which makes the chunk a lane fetches the same in every request.
+constexpr int prefill_panels(int ks, int vt) { return (ks + 1) / 2 + (vt + 3) / 4; }
 template <int KS, int VT, int U>
-__global__ __launch_bounds__(256, (KS + VT > 18) ? 1 : 2) void windowed_prefill_kernel(WindowedAttention a) {
-  constexpr int KC = 4 * KS, VC = 2 * VT;                  // 16-byte chunks per key / value row
-  constexpr int KB = 64 * KS + 16, VB = 32 * VT + 32;      // bytes per LDS row
-  constexpr int kStage = kPfBK * (KB + VB);
-  constexpr int KP = KS, VP = (kPfBK * VC + 255) / 256;    // chunks per thread and block
+__global__ __launch_bounds__(256, prefill_panels(KS, VT) > 5 ? 1 : 2) void windowed_prefill_kernel(WindowedAttention a) {
+  constexpr int KP = (KS + 1) / 2, VP = (VT + 3) / 4;      // key / value panels
+  constexpr int kPanel = kPfBK * 128, kStage = (KP + VP) * kPanel;
   extern __shared__ __attribute__((aligned(1024))) unsigned char lds[];
   const uint32_t lds0 = (uint32_t)(uintptr_t)(pf_lds_char_t*)lds;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -147,45 +162,46 @@ __global__ __launch_bounds__(256, (KS + VT > 18) ? 1 : 2) void windowed_prefill_
   const uint16_t* vv = reinterpret_cast<const uint16_t*>(a.v) + (size_t)b * a.v_batch + (size_t)h * a.v_head;
   const int c1 = a.d1 >> 3, c2 = c1 + (a.d2 >> 3), cv = a.dv >> 3;
 
-  u32x4_t kraw[KP], vraw[VP];
-  auto fetch = [&](int kb0) {
+  // ---- what this lane fetches: row 8 q + lane / 8 of a request, slot lane % 8 of its panel.  Chunks past the widths
+  // repeat the last one (finite values that meet zeros, or columns that are not written).
+  const int req_row = 8 * wave + (lane >> 3);
+  const int kslot = (lane & 7) ^ ((4 * wave + (lane >> 4)) & 7);
+  const int vslot = ((((lane & 7) >> 1) ^ ((lane >> 4) & 3)) << 1) | (lane & 1);
+  const char* kbase[KP];
+  uint32_t kstride[KP];  // bytes
 #pragma unroll
-    for (int i = 0; i < KP; ++i) {
-      const int ci = threadIdx.x + 256 * i, c = ci % KC;
-      const int row = min(kb0 + ci / KC, total - 1);  // rows past the end repeat the last one; those keys are masked
-      kraw[i] = u32x4_t{0u, 0u, 0u, 0u};
-      if (c < c2) {
-        const uint16_t* src = c < c1 ? k1 + (size_t)row * a.k1_row + 8 * c : k2 + (size_t)row * a.k2_row + 8 * (c - c1);
-        kraw[i] = *reinterpret_cast<const u32x4_t*>(src);
-      }
-    }
+  for (int p = 0; p < KP; ++p) {
+    const int c = min(8 * p + kslot, c2 - 1);
+    kbase[p] = reinterpret_cast<const char*>(c < c1 ? k1 + 8 * c : k2 + 8 * (c - c1));
+    kstride[p] = 2u * (uint32_t)(c < c1 ? a.k1_row : a.k2_row);
+  }
+  const char* vbase[VP];
 #pragma unroll
-    for (int i = 0; i < VP; ++i) {
-      const int ci = threadIdx.x + 256 * i, c = ci % VC;
-      const int row = min(kb0 + ci / VC, total - 1);
-      vraw[i] = u32x4_t{0u, 0u, 0u, 0u};
-      if (ci < kPfBK * VC && c < cv) vraw[i] = *reinterpret_cast<const u32x4_t*>(vv + (size_t)row * a.v_row + 8 * c);
-    }
-  };
-  auto lay_down = [&](int stage) {
-    unsigned char* base = lds + stage * kStage;
+  for (int p = 0; p < VP; ++p) vbase[p] = reinterpret_cast<const char*>(vv + 8 * min(8 * p + vslot, cv - 1));
+  const uint32_t vstride = 2u * (uint32_t)a.v_row;
+  auto fetch = [&](int j) {
+    const uint32_t to = lds0 + (uint32_t)((j & 1) * kStage + wave * 1024);
 #pragma unroll
-    for (int i = 0; i < KP; ++i) {
-      const int ci = threadIdx.x + 256 * i;
-      *reinterpret_cast<u32x4_t*>(base + (ci / KC) * KB + 16 * (ci % KC)) = kraw[i];
-    }
+    for (int half = 0; half < 2; ++half) {
+      // rows past the end repeat the last one; those keys are masked
+      const uint32_t row = (uint32_t)min(lo + j * kPfBK + 32 * half + req_row, total - 1);
 #pragma unroll
-    for (int i = 0; i < VP; ++i) {
-      const int ci = threadIdx.x + 256 * i;
-      if (ci < kPfBK * VC) *reinterpret_cast<u32x4_t*>(base + kPfBK * KB + (ci / VC) * VB + 16 * (ci % VC)) = vraw[i];
+      for (int p = 0; p < KP; ++p) dma16_gather(kbase[p] + (size_t)row * kstride[p], to + (uint32_t)(p * kPanel + half * 4096));
+#pragma unroll
+      for (int p = 0; p < VP; ++p) dma16_gather(vbase[p] + (size_t)row * vstride, to + (uint32_t)((KP + p) * kPanel + half * 4096));
     }
   };
-  // key fragment (16-key tile jb, step s): row 16 jb + r, columns 32 s + 8 g ..
-  uint32_t k_rd = lds0 + (uint32_t)(r * KB + 16 * g);
-  // value fragment of tile t: this lane addresses 8 bytes (piece r & 3) of key 4 g + (r >> 2)
-  uint32_t v_rd = lds0 + (uint32_t)(kPfBK * KB + (4 * g + (r >> 2)) * VB + 8 * (r & 3));
+  // ---- fragment addresses inside a stage
+  // keys (16-key tile jb, step s): row 16 jb + r, chunk 4 (s & 1) + g of panel s >> 1
+  const uint32_t k_rd[2] = {lds0 + (uint32_t)(r * 128 + 16 * (g ^ ((r >> 1) & 7))),
+                            lds0 + (uint32_t)(r * 128 + 16 * ((4 + g) ^ ((r >> 1) & 7)))};
+  // values (tile t): this lane addresses 8 bytes (piece r & 3) of key 4 g + (r >> 2), segment t & 3 of panel t >> 2
+  uint32_t v_rd[4];
+#pragma unroll
+  for (int v = 0; v < 4; ++v)
+    v_rd[v] = lds0 + (uint32_t)(KP * kPanel + (4 * g + (r >> 2)) * 128 + 32 * (v ^ ((2 * g + (r >> 3)) & 3)) + 8 * (r & 3));
 
-  fetch(lo);
+  fetch(0);
   const float scale2 = a.scale * kLog2eF;
   const float sink2 = a.sink ? a.sink[h] * kLog2eF : -1e30f;
   float m_run[U], l_run[U];
@@ -209,17 +225,12 @@ __global__ __launch_bounds__(256, (KS + VT > 18) ? 1 : 2) void windowed_prefill_
       if (c < c2) qf[u][s] = *reinterpret_cast<const u32x4_t*>(qp + 8 * c);
     }
   }
-  lay_down(0);
-  if (nblk > 1) fetch(lo + kPfBK);
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
   __syncthreads();
   for (int j = 0; j < nblk; ++j) {
-    // block j is complete in stage j & 1; block j + 1 (in registers) goes into the other stage, last read before the
-    // previous barrier, while block j + 2 starts its flight from memory
+    // block j is complete in stage j & 1; block j + 1 goes into the other stage, last read before the previous barrier
     const int kb0 = lo + j * kPfBK;
-    if (j + 1 < nblk) {
-      lay_down((j + 1) & 1);
-      if (j + 2 < nblk) fetch(kb0 + 2 * kPfBK);
-    }
+    if (j + 1 < nblk) fetch(j + 1);
     const uint32_t stage = (uint32_t)((j & 1) * kStage);
     if (kb0 <= wave_last && kb0 + kPfBK - 1 > wave_first - window) {
       f32x4_t sc[U][4];
@@ -227,7 +238,7 @@ __global__ __launch_bounds__(256, (KS + VT > 18) ? 1 : 2) void windowed_prefill_
       for (int s = 0; s < KS; ++s) {
         u32x4_t ka[4];
 #pragma unroll
-        for (int jb = 0; jb < 4; ++jb) ka[jb] = pf_read128(k_rd + stage + (uint32_t)(jb * 16 * KB + 64 * s));
+        for (int jb = 0; jb < 4; ++jb) ka[jb] = pf_read128(k_rd[s & 1] + stage + (uint32_t)((s >> 1) * kPanel + jb * 2048));
 #pragma unroll
         for (int jb = 0; jb < 4; ++jb)
 #pragma unroll
@@ -277,17 +288,28 @@ __global__ __launch_bounds__(256, (KS + VT > 18) ? 1 : 2) void windowed_prefill_
         pf[u][0] = pack8_bf16(&p[0]);
         pf[u][1] = pack8_bf16(&p[8]);
       }
+      // value fragments (two transposing reads: a half's first and second 16-key tile), kRing of them in flight
+      constexpr int kRing = VT < 4 ? VT : 4;
+      auto v_at = [&](int i) { return v_rd[(i % VT) & 3] + stage + (uint32_t)((i / VT) * 4096 + ((i % VT) >> 2) * kPanel); };
+      u32x2_t vlo[kRing], vhi[kRing];
 #pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
+      for (int i = 0; i < kRing; ++i) {
+        vlo[i] = pf_read_tr(v_at(i));
+        vhi[i] = pf_read_tr(v_at(i) + 2048u);
+      }
 #pragma unroll
-        for (int t = 0; t < VT; ++t) {
-          const uint32_t at = v_rd + stage + (uint32_t)(hf * 32 * VB + 32 * t);
-          const u32x2_t vlo = pf_read_tr(at), vhi = pf_read_tr(at + (uint32_t)(16 * VB));
-          const u32x4_t vf = {vlo.x, vlo.y, vhi.x, vhi.y};
+      for (int i = 0; i < 2 * VT; ++i) {  // i = VT half + tile
+        const u32x4_t vf = {vlo[i % kRing].x, vlo[i % kRing].y, vhi[i % kRing].x, vhi[i % kRing].y};
 #pragma unroll
-          for (int u = 0; u < U; ++u) o[u][t] = mfma16(vf, pf[u][hf], o[u][t]);
+        for (int u = 0; u < U; ++u) o[u][i % VT] = mfma16(vf, pf[u][i / VT], o[u][i % VT]);
+        if (i + kRing < 2 * VT) {
+          vlo[i % kRing] = pf_read_tr(v_at(i + kRing));
+          vhi[i % kRing] = pf_read_tr(v_at(i + kRing) + 2048u);
         }
+      }
     }
+    // the next block must have landed and every wave must be done with this one
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
   }
 #pragma unroll

@@ -32,7 +32,7 @@ from torch import nn
 from . import _lib
 from .modeling import Embedding, GatedFeedForward, Linear, RingCache, RMSNorm, build_norm, register_architecture
 
-GEMV_ROWS = 16    # rows up to which a product is a matrix-vector kernel of this library
+GEMV_ROWS = 16    # rows of a prompt up to which the head's product is a matrix-vector kernel of this library
 NORM_PROLOGUE_ROWS = 4  # rows up to which the decode products form the norms themselves
 
 
@@ -314,7 +314,8 @@ class LatentLM(nn.Module):
             raise ValueError(f"Input length {start + seq} exceeds context length {self.context_length}")
         if not static and cache is not None and start + seq > cache.max_len:
             raise ValueError(f"the cache holds {cache.max_len} positions, {start + seq} needed")
-        if cache is not None and seq == 1 and residuals is None:
+        single = cache is not None and seq == 1 and residuals is None
+        if single:
             if not static:
                 cache.position.fill_(start)
             x, delta = self._token(token_ids, cache)
@@ -332,7 +333,7 @@ class LatentLM(nn.Module):
                 rows = torch.tensor([b * seq + t for b in range(batch) for t in picks], device=x.device)
                 x = x.index_select(0, rows)
                 delta = delta.index_select(0, rows) if delta is not None else None
-        return self._logits(x, delta).view(batch, -1, self._head.shape[0])[:, :, : self.vocab_size]
+        return self._logits(x, delta, single).view(batch, -1, self._head.shape[0])[:, :, : self.vocab_size]
 
     def _embedded(self, token_ids: torch.Tensor, start: int, pos: torch.Tensor | None) -> tuple[torch.Tensor, torch.Tensor | None]:
         """The residual stream in front of the first layer run, and the embedding output where a loop needs it again."""
@@ -345,13 +346,18 @@ class LatentLM(nn.Module):
             _ptr(pos), _ptr(self._begins(0)[1]), _ptr(x), _ptr(embedded), dp, _flag(self._embed.dtype), _stream()), "embed")
         return x, embedded
 
-    def _logits(self, x: torch.Tensor, delta: torch.Tensor | None) -> torch.Tensor:
-        """``head norm(x + delta)``, fp32, columns padded to a multiple of 16."""
+    def _logits(self, x: torch.Tensor, delta: torch.Tensor | None, single: bool) -> torch.Tensor:
+        """``head norm(x + delta)``, fp32, columns padded to a multiple of 16.  ``single``: a decode step (its products are
+        this library's for any number of sequences: library kernels stay out of recorded graphs)."""
         rows, dtype = x.shape[0], self._head.dtype
+        if not single and rows > GEMV_ROWS:
+            normed, _ = _add_norms(x, delta, None, None, self._final_gain, None, self.final_norm.epsilon,
+                                   0 if isinstance(self.final_norm, RMSNorm) else 1, self.d_model, dtype)
+            return _product(normed, self._head, torch.float32)
         center = 0 if isinstance(self.final_norm, RMSNorm) else 1
         eps, gain = self.final_norm.epsilon, self._final_gain
         y = torch.empty((rows, self._head.shape[0]), dtype=torch.float32, device=x.device)
-        if dtype == torch.bfloat16 and rows <= GEMV_ROWS:
+        if dtype == torch.bfloat16:
             if delta is None and rows <= NORM_PROLOGUE_ROWS:
                 self._dense_in(x, None, None, gain, None, eps, center, self._head, None, y, None, 0, 0)
                 return y
@@ -359,10 +365,8 @@ class LatentLM(nn.Module):
             self._dense_in(None, normed, None, None, None, eps, center, self._head, None, y, None, 0, 0)
             return y
         normed, _ = _add_norms(x, delta, None, None, gain, None, eps, center, self.d_model, dtype)
-        if rows <= GEMV_ROWS:
-            _matvec(self._head, 1, normed, normed.shape[1], 0, y, y.shape[1], 0, rows)
-            return y
-        return _product(normed, self._head, torch.float32)
+        _matvec(self._head, 1, normed, normed.shape[1], 0, y, y.shape[1], 0, rows)
+        return y
 
     # ---- many tokens per sequence
     def _prompt(self, token_ids: torch.Tensor, cache: RingCache | None, start: int,
