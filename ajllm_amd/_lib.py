@@ -190,6 +190,7 @@ DENSE_SIGNATURES: dict[str, tuple] = {
     "ajqd_dense_out": (c_int, [_P, _P, _P, _P, _P, _I, _I, _I, _P]),
     "ajqd_latent_absorb": (c_int, [_P, _I, ctypes.POINTER(LatentShape), _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _P]),
     "ajqd_latent_decode_chunks": (c_int, [_I, _I, _I, _I, _I]),
+    "ajqd_latent_decode_workspace": (c_size_t, [_I, _I, _I, _I]),
     "ajqd_latent_decode": (c_int, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P]),
     "ajqd_latent_expand": (c_int, [_P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P]),
 }

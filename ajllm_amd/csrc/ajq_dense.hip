@@ -116,6 +116,12 @@ int launch_prefill_vt(int vt, const WindowedAttention& w, hipStream_t stream) {
 // ---- decode attention: (column steps, latent tiles per wave) that hold the widths
 int latent_tiles(int rankp) { const int t = (rankp + 63) / 64; return t <= 2 ? 2 : t <= 4 ? 4 : t <= 8 ? 8 : 0; }
 int latent_steps(int width) { const int s = (width + 31) / 32; return s <= 4 ? 4 : s <= 6 ? 6 : s <= 10 ? 10 : s <= 18 ? 18 : 0; }
+// the chunks' sums, then (maximum, denominator) per head and chunk
+float2* heads_at(const float* partial, int batch, int heads, int chunks, int rankp) {
+  return reinterpret_cast<float2*>(const_cast<float*>(partial) + latent_sums_at(batch, 0, 0, heads, chunks, rankp));
+}
+constexpr int kDecodeWorkgroups = 256;  // one per CU (its LDS holds two blocks of rows)
+int latent_head_groups(int heads) { return heads <= 16 ? 1 : (heads + 31) / 32; }  // one or two head tiles per workgroup
 int gemv_waves(int k) { return k >= 2048 ? 8 : k >= 256 ? 4 : 1; }
 
 }  // namespace
@@ -348,11 +354,16 @@ int ajqd_latent_decode_chunks(int batch, int heads, int rankp, int rotp, int cap
   if (batch < 1 || heads < 1 || cap < 1 || rankp < 16 || rankp % 16 || rotp < 8 || rotp % 8 || !latent_tiles(rankp) ||
       !latent_steps(rankp + rotp))
     return 0;
-  const int tiles = batch * ((heads + 15) / 16);
-  int s = (256 + tiles - 1) / tiles;
+  const int groups = batch * latent_head_groups(heads);
+  int s = (kDecodeWorkgroups + groups - 1) / groups;
   const int by_rows = (cap + kLatentRows - 1) / kLatentRows;
   if (s > by_rows) s = by_rows;
   return s < 1 ? 1 : s > kLatentMaxChunks ? kLatentMaxChunks : s;
+}
+
+size_t ajqd_latent_decode_workspace(int batch, int heads, int rankp, int chunks) {
+  if (batch < 1 || heads < 1 || rankp < 1 || chunks < 1) return 0;
+  return 4 * (size_t)latent_sums_at(batch, 0, 0, heads, chunks, rankp) + 8 * (size_t)batch * heads * chunks;
 }
 
 int ajqd_latent_decode(const void* q, const void* ring, const int64_t* pos, float* partial, int batch, int heads, int rankp,
@@ -362,23 +373,27 @@ int ajqd_latent_decode(const void* q, const void* ring, const int64_t* pos, floa
     return fail(AJQ_ERR_UNSUPPORTED, "ajqd_latent_decode: widths %d + %d are not built", rankp, rotp);
   if (chunks < 1 || chunks > kLatentMaxChunks || !(scale > 0.f))
     return fail(AJQ_ERR_SHAPE, "ajqd_latent_decode: unsupported shape (batch=%d chunks=%d)", batch, chunks);
-  LatentDecode d{(const uint16_t*)q, (const uint16_t*)ring, positions64(pos), partial, batch, heads, rankp, rankp + rotp, cap,
-                 chunks, scale * kLog2eF};
-  const long long blocks = (long long)((heads + 15) / 16) * chunks * batch;
+  LatentDecode d{(const uint16_t*)q, (const uint16_t*)ring, positions64(pos), partial,
+                 heads_at(partial, batch, heads, chunks, rankp), batch, heads, rankp, rankp + rotp, cap, chunks, scale * kLog2eF};
+  const long long blocks = (long long)latent_head_groups(heads) * chunks * batch;
   if (blocks > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_latent_decode: too many workgroups");
-  const int bytes = latent_decode_lds(rankp);
-  auto go = [&](auto kernel) {
+  const bool two = heads > 16;
+  auto go = [&](auto kernel, int ks) {
+    const int bytes = latent_decode_lds(ks, two ? 2 : 1);
     if (int e = allow_lds(kernel, bytes, "ajqd_latent_decode")) return e;
-    hipLaunchKernelGGL(kernel, dim3((unsigned)blocks), dim3(256), bytes, (hipStream_t)stream, d);
+    hipLaunchKernelGGL(kernel, dim3((unsigned)blocks), dim3(two ? 512 : 256), bytes, (hipStream_t)stream, d);
     return check_launch("ajqd_latent_decode");
   };
+  auto pick = [&](auto one, auto both, int ks) { return two ? go(both, ks) : go(one, ks); };
   const int tiles = latent_tiles(rankp);
+#define AJQD_DECODE(KS, RT) pick(latent_decode_kernel<KS, RT, 1>, latent_decode_kernel<KS, RT, 2>, KS)
   switch (latent_steps(rankp + rotp)) {
-    case 4: return go(latent_decode_kernel<4, 2>);  // (at most 128 columns: two tiles per wave)
-    case 6: return tiles == 2 ? go(latent_decode_kernel<6, 2>) : go(latent_decode_kernel<6, 4>);
-    case 10: return tiles == 2 ? go(latent_decode_kernel<10, 2>) : tiles == 4 ? go(latent_decode_kernel<10, 4>) : go(latent_decode_kernel<10, 8>);
-    default: return tiles == 2 ? go(latent_decode_kernel<18, 2>) : tiles == 4 ? go(latent_decode_kernel<18, 4>) : go(latent_decode_kernel<18, 8>);
+    case 4: return AJQD_DECODE(4, 2);  // (at most 128 columns: two tiles per wave)
+    case 6: return tiles == 2 ? AJQD_DECODE(6, 2) : AJQD_DECODE(6, 3);
+    case 10: return tiles == 2 ? AJQD_DECODE(10, 2) : tiles == 4 ? AJQD_DECODE(10, 4) : AJQD_DECODE(10, 5);
+    default: return tiles == 2 ? AJQD_DECODE(18, 2) : tiles == 4 ? AJQD_DECODE(18, 4) : AJQD_DECODE(18, 8);
   }
+#undef AJQD_DECODE
 }
 
 int ajqd_latent_expand(const float* partial, const float* sink, const float* gate, int gate_ld, const void* uv, void* out,
@@ -388,10 +403,11 @@ int ajqd_latent_expand(const float* partial, const float* sink, const float* gat
       out_ld < heads * vdimp || out_ld % 4)
     return fail(AJQ_ERR_SHAPE, "ajqd_latent_expand: unsupported shape (batch=%d heads=%d chunks=%d rankp=%d vdimp=%d)", batch,
                 heads, chunks, rankp, vdimp);
-  if (rankp > 32 * kExpandSteps) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_latent_expand: latents of %d are not built", rankp);
-  const int groups = (vdimp / 16 + 7) / 8, bytes = 2 * kExpandBatch * (rankp + 8);
-  LatentExpand d{partial, sink, gate, (const uint16_t*)uv, (uint16_t*)out, batch, heads, chunks, rankp, vdimp, gate_ld, out_ld, groups};
-  hipLaunchKernelGGL(latent_expand_kernel, dim3(heads * groups, (batch + kExpandBatch - 1) / kExpandBatch), dim3(512), bytes,
+  if (rankp > kExpandRank) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_latent_expand: latents of %d are not built", rankp);
+  const bool few = batch <= kExpandBatch;
+  const int tw = few ? 2 : 8, groups = (vdimp / 16 + tw - 1) / tw, bytes = 2 * kExpandBatch * (rankp + 8);
+  LatentExpand d{partial, heads_at(partial, batch, heads, chunks, rankp), sink, gate, (const uint16_t*)uv, (uint16_t*)out, batch, heads, chunks, rankp, vdimp, gate_ld, out_ld, groups};
+  hipLaunchKernelGGL(few ? latent_expand_kernel<2> : latent_expand_kernel<8>, dim3(heads * groups, (batch + kExpandBatch - 1) / kExpandBatch), dim3(512), bytes,
                      (hipStream_t)stream, d);
   return check_launch("ajqd_latent_expand");
 }

@@ -320,159 +320,183 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAbsorb a) {
            float4{acc[0][0][0], acc[0][0][1], acc[0][0][2], acc[0][0][3]});
 }
 
-// One chunk of cache rows against 16 heads of one sequence, in the latent space: row j of the ring
-// (latent rankp | rotated rotp) is the key, its latent part the value, for every head.  Blocks of 64 rows, a wave 16 of them:
-// the rows are loaded in the layout of the first product's A operand (S^T = K Q^T; KS column steps, queries in registers as
-// well), from there laid into LDS for the second (U^T += C^T P^T, latents read by transposing LDS reads, a wave takes every
-// fourth 16-column tile, RT of them), while the next block is on its way.
-// Partial result of (b, h, chunk): (maximum, denominator, 0, 0, rankp sums), base-2 exponents; zeros for an empty chunk.
-// Grid: chunks of sequences x head tiles; the head tiles of a chunk are 8 workgroups apart, on one XCD and its L2.
+// One chunk of cache rows against 16 HT heads of one sequence, in the latent space: row j of the ring
+// (latent rankp | rotated rotp) is the key, its latent part the value, for every head, so a row is fetched once for all of
+// the workgroup's heads and both products.  Four waves per head tile; blocks of 64 rows go into LDS by DMA, one block ahead.
+//   S^T = K Q^T:    wave w takes keys 16 (w & 3) .. of the block; KS column steps, its head tile's queries in registers
+//   U^T += C^T P^T: wave w takes every fourth 16-column tile of the latent (RT of them), latents by transposing LDS reads
+// LDS holds the rows in panels of 128 bytes (64 rows x 8 chunks): chunk c of row k in slot c ^ (k & 6 | k >> 3 & 1), so that
+// sixteen rows of one chunk and eight rows of one 32-byte segment (whose two chunks stay neighbours) meet every bank once.
+// Partial result of (b, h, chunk): maximum and denominator (base-2 exponents) in `heads_out`, and rankp sums in `sums`, which
+// holds [b][head tile][chunk][16-column tile][16 heads][16 columns] so that a wave stores whole lines; zeros for an empty chunk.
+// Grid: chunks of sequences x head groups; the groups of a chunk are 8 workgroups apart, on one XCD and its L2.
 struct LatentDecode {
   const uint16_t* q;        // [B, H, width]
   const uint16_t* ring;     // [B, cap, width]
   const long long* pos;
-  float* partial;           // [B, H, S, rankp + 4]
+  float* sums;
+  float2* heads_out;        // [B, H, S]
   int batch, heads, rankp, width, cap, chunks;
   float scale2;
 };
+__host__ __device__ constexpr long long latent_sums_at(int b, int tile, int chunk, int heads, int chunks, int rankp) {
+  return (((long long)b * ((heads + 15) / 16) + tile) * chunks + chunk) * 16 * rankp;
+}
 constexpr int kLatentRows = 64;
 constexpr int kLatentPBytes = (kLatentRows + 8) * 2;
-// bytes of a latent row in LDS: 32 past a multiple of 256, so that eight rows of one 32-byte segment meet every bank once
-__host__ __device__ constexpr int latent_row_bytes(int rankp) { return 2 * rankp + ((32 - 2 * rankp) & 255); }
-__host__ __device__ constexpr int latent_decode_lds(int rankp) { return kLatentRows * latent_row_bytes(rankp) + 16 * kLatentPBytes; }
-template <int KS, int RT>
-__global__ __launch_bounds__(256, 2) void latent_decode_kernel(LatentDecode a) {
+constexpr int latent_decode_lds(int ks, int ht) { return ks * 8192 + ht * 16 * kLatentPBytes; }  // two stages of ks / 2 panels
+template <int KS, int RT, int HT>
+__global__ __launch_bounds__(256 * HT) void latent_decode_kernel(LatentDecode a) {
+  constexpr int NP = KS / 2, kPanel = kLatentRows * 128, kStage = NP * kPanel, kWaves = 4 * HT;
+  static_assert(KS % 2 == 0, "whole panels");
   extern __shared__ __attribute__((aligned(1024))) unsigned char lds[];
-  __shared__ float smax[4][16], ssum[4][16];
+  __shared__ float smax[HT][4][16], ssum[HT][4][16];
   const uint32_t lds0 = (uint32_t)(uintptr_t)(pf_lds_char_t*)lds;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r = lane & 15, g = lane >> 4;
-  const int head_tiles = (a.heads + 15) >> 4, units = a.batch * a.chunks;
-  int unit, tile;
+  const int part = wave & 3, ht = wave >> 2;
+  const int groups = (a.heads + 16 * HT - 1) / (16 * HT), units = a.batch * a.chunks;
+  int unit, group;
   if ((units & 7) == 0) {
     const int m = (int)(blockIdx.x >> 3);
-    tile = m % head_tiles;
-    unit = 8 * (m / head_tiles) + (int)(blockIdx.x & 7);
+    group = m % groups;
+    unit = 8 * (m / groups) + (int)(blockIdx.x & 7);
   } else {
-    tile = (int)blockIdx.x % head_tiles;
-    unit = (int)blockIdx.x / head_tiles;
+    group = (int)blockIdx.x % groups;
+    unit = (int)blockIdx.x / groups;
   }
-  const int b = unit / a.chunks, chunk = unit % a.chunks, h0 = 16 * tile;
-  const int rb = latent_row_bytes(a.rankp), cw = a.width >> 3;
+  const int b = unit / a.chunks, chunk = unit % a.chunks, h0 = 16 * (HT * group + ht);
+  const int cw = a.width >> 3;
+  u32x4_t qf[KS];  // requested before the position is known
+  const uint16_t* qsrc = a.q + ((size_t)b * a.heads + min(h0 + r, a.heads - 1)) * a.width + 8 * g;
+#pragma unroll
+  for (int s = 0; s < KS; ++s) {
+    qf[s] = u32x4_t{0u, 0u, 0u, 0u};
+    if (4 * s + g < cw) qf[s] = *reinterpret_cast<const u32x4_t*>(qsrc + 32 * s);
+  }
   const int valid = (int)min(max(*a.pos, 0ll), (long long)a.cap - 1) + 1;  // rows the ring holds
   const int per = (((valid + a.chunks - 1) / a.chunks) + kLatentRows - 1) & ~(kLatentRows - 1);
   const int begin = chunk * per, end = min(valid, begin + per);
-  float* head_out = a.partial + (((size_t)b * a.heads + min(h0 + r, a.heads - 1)) * a.chunks + chunk) * (a.rankp + 4);
-  const u32x4_t zero = {0u, 0u, 0u, 0u};
   float m = -INFINITY, l = 0.f;
   f32x4_t u[RT] = {};
   if (begin < end) {
-    const uint16_t* ring = a.ring + (size_t)b * a.cap * a.width;
-    u32x4_t kf[KS], qf[KS];
-    // rows past the end repeat the last one (those keys are masked), chunks past the width the last one (zero query columns)
+    const char* ring = reinterpret_cast<const char*>(a.ring + (size_t)b * a.cap * a.width);
+    // a request fills 8 rows of a panel: this lane row lane / 8, slot lane % 8.  Rows past the end repeat the last one (those
+    // keys are masked), chunks past the width the last one (they meet zero query columns).
+    const int chunk_of = (lane & 7) ^ (((lane >> 3) & 6) | (wave & 1));  // (a wave's requests all start at rows of one parity of 8)
     auto fetch = [&](int j0) {
-      const uint32_t row = (uint32_t)min(j0 + 16 * wave + r, end - 1) * (uint32_t)a.width;
+      const uint32_t to = lds0 + (uint32_t)((((j0 - begin) / kLatentRows) & 1) * kStage);
 #pragma unroll
-      for (int s = 0; s < KS; ++s) kf[s] = *reinterpret_cast<const u32x4_t*>(ring + row + (uint32_t)min(32 * s + 8 * g, a.width - 8));
+      for (int i = 0; i < (8 * NP + kWaves - 1) / kWaves; ++i) {
+        const int req = wave + kWaves * i;  // panel req / 8, rows 8 (req % 8) ..
+        if ((8 * NP) % kWaves != 0 && req >= 8 * NP) continue;
+        const uint32_t row = (uint32_t)min(j0 + 8 * (req & 7) + (lane >> 3), end - 1);
+        const uint32_t c = (uint32_t)min(8 * (req >> 3) + chunk_of, cw - 1);
+        dma16_gather(ring + (size_t)row * (uint32_t)(2 * a.width) + 16u * c, to + (uint32_t)(req * 1024));
+      }
     };
     fetch(begin);
-    const uint16_t* qsrc = a.q + ((size_t)b * a.heads + min(h0 + r, a.heads - 1)) * a.width + 8 * g;
-#pragma unroll
-    for (int s = 0; s < KS; ++s) {
-      qf[s] = zero;
-      if (4 * s + g < cw) qf[s] = *reinterpret_cast<const u32x4_t*>(qsrc + 32 * s);
-    }
-    const uint32_t p_at = (uint32_t)(kLatentRows * rb);
+    // keys: row 16 part + r, chunk 4 (s & 1) + g of panel s / 2
+    const uint32_t k_rd[2] = {lds0 + (uint32_t)((16 * part + r) * 128 + 16 * (g ^ (r & 6 | r >> 3))),
+                              lds0 + (uint32_t)((16 * part + r) * 128 + 16 * ((4 + g) ^ (r & 6 | r >> 3)))};
+    // latents: this lane addresses 8 bytes (piece r & 3) of row 4 g + (r >> 2); tile part + 4 t is segment part of panel t
+    const int vrow = 4 * g + (r >> 2);
+    const uint32_t v_rd = lds0 + (uint32_t)(vrow * 128 + 16 * ((2 * part | (r & 3) >> 1) ^ (vrow & 6 | vrow >> 3)) + 8 * (r & 1));
+    unsigned char* p_lds = lds + 2 * kStage + ht * 16 * kLatentPBytes + r * kLatentPBytes;
     for (int j0 = begin; j0 < end; j0 += kLatentRows) {
+      // this block has landed; every wave is done with the one before, whose stage the next block goes to
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      __syncthreads();
+      if (j0 + kLatentRows < end) fetch(j0 + kLatentRows);
+      const uint32_t stage = (uint32_t)((((j0 - begin) / kLatentRows) & 1) * kStage);
       f32x4_t sc[2] = {};
 #pragma unroll
-      for (int s = 0; s < KS; ++s) sc[s & 1] = mfma16(kf[s], qf[s], sc[s & 1]);
-#pragma unroll
-      for (int s = 0; s < KS; ++s)
-        if (4 * s + g < (a.rankp >> 3)) *reinterpret_cast<u32x4_t*>(lds + (16 * wave + r) * rb + 64 * s + 16 * g) = kf[s];
-      if (j0 + kLatentRows < end) fetch(j0 + kLatentRows);
-      // score i: key j0 + 16 wave + 4 g + i, head h0 + r
+      for (int s = 0; s < KS; ++s) sc[s & 1] = mfma16(pf_read128(k_rd[s & 1] + stage + (uint32_t)((s >> 1) * kPanel)), qf[s], sc[s & 1]);
+      // score i: key j0 + 16 part + 4 g + i, head h0 + r
       float p[4], mx = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        p[i] = j0 + 16 * wave + 4 * g + i < end ? (sc[0][i] + sc[1][i]) * a.scale2 : -INFINITY;
+        p[i] = j0 + 16 * part + 4 * g + i < end ? (sc[0][i] + sc[1][i]) * a.scale2 : -INFINITY;
         mx = fmaxf(mx, p[i]);
       }
       mx = quad_max(mx);
-      if (g == 0) smax[wave][r] = mx;
+      if (g == 0) smax[ht][part][r] = mx;
       __syncthreads();
       // (finite: the block's first row is valid)
-      const float m_new = fmaxf(fmaxf(fmaxf(smax[0][r], smax[1][r]), fmaxf(smax[2][r], smax[3][r])), m);
-      const float corr = exp2f(m - m_new);
+      const float m_new = fmaxf(fmaxf(fmaxf(smax[ht][0][r], smax[ht][1][r]), fmaxf(smax[ht][2][r], smax[ht][3][r])), m);
+      const float corr = __builtin_amdgcn_exp2f(m - m_new);
       m = m_new;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) p[i] = exp2f(p[i] - m);
+      for (int i = 0; i < 4; ++i) p[i] = __builtin_amdgcn_exp2f(p[i] - m);
       l = l * corr + ((p[0] + p[1]) + (p[2] + p[3]));
-      store4(reinterpret_cast<uint16_t*>(lds + p_at + r * kLatentPBytes) + 16 * wave + 4 * g, float4{p[0], p[1], p[2], p[3]});
+      store4(reinterpret_cast<uint16_t*>(p_lds) + 16 * part + 4 * g, float4{p[0], p[1], p[2], p[3]});
 #pragma unroll
       for (int t = 0; t < RT; ++t) u[t] *= corr;
       __syncthreads();
 #pragma unroll
       for (int hf = 0; hf < 2; ++hf) {
-        const unsigned char* pr = lds + p_at + r * kLatentPBytes + 2 * (32 * hf + 4 * g);
+        const unsigned char* pr = p_lds + 2 * (32 * hf + 4 * g);
         const u32x2_t plo = *reinterpret_cast<const u32x2_t*>(pr), phi = *reinterpret_cast<const u32x2_t*>(pr + 32);
         const u32x4_t pf = {plo.x, plo.y, phi.x, phi.y};
-        const uint32_t at = lds0 + (uint32_t)((32 * hf + 4 * g + (r >> 2)) * rb + 32 * wave + 8 * (r & 3));
-        // (tiles past the latent read what else lies in LDS; their sums are not written)
+        const uint32_t at = v_rd + stage + (uint32_t)(hf * 4096);
+        // (panels past the latent hold the rotated part, or nothing of this block: their sums are not written)
+        u32x2_t lo[RT], hi[RT];
 #pragma unroll
-        for (int t0 = 0; t0 < RT; t0 += 2) {
-          u32x2_t lo[2], hi[2];
-#pragma unroll
-          for (int t = 0; t < 2; ++t) {
-            lo[t] = pf_read_tr(at + 128u * (t0 + t));
-            hi[t] = pf_read_tr(at + 128u * (t0 + t) + (uint32_t)(16 * rb));
-          }
-#pragma unroll
-          for (int t = 0; t < 2; ++t) u[t0 + t] = mfma16(u32x4_t{lo[t].x, lo[t].y, hi[t].x, hi[t].y}, pf, u[t0 + t]);
+        for (int t = 0; t < RT; ++t) {
+          lo[t] = pf_read_tr(at + (uint32_t)(t * kPanel));
+          hi[t] = pf_read_tr(at + (uint32_t)(t * kPanel + 2048));
         }
+#pragma unroll
+        for (int t = 0; t < RT; ++t) u[t] = mfma16(u32x4_t{lo[t].x, lo[t].y, hi[t].x, hi[t].y}, pf, u[t]);
       }
-      __syncthreads();
     }
     l = quad_sum(l);
-    if (g == 0) ssum[wave][r] = l;
+    if (g == 0) ssum[ht][part][r] = l;
     __syncthreads();
-    l = (ssum[0][r] + ssum[1][r]) + (ssum[2][r] + ssum[3][r]);
+    l = (ssum[ht][0][r] + ssum[ht][1][r]) + (ssum[ht][2][r] + ssum[ht][3][r]);
   }
-  if (h0 + r >= a.heads) return;
-  if (wave == 0 && g == 0) store4(head_out, float4{m, l, 0.f, 0.f});
+  if (h0 >= a.heads) return;
+  if (part == 0 && g == 0 && h0 + r < a.heads) a.heads_out[((size_t)b * a.heads + h0 + r) * a.chunks + chunk] = float2{m, l};
+  float* out = a.sums + latent_sums_at(b, h0 >> 4, chunk, a.heads, a.chunks, a.rankp) + 16 * r + 4 * g;
 #pragma unroll
   for (int t = 0; t < RT; ++t) {
-    const int col = 16 * (wave + 4 * t);
-    if (col < a.rankp) store4(head_out + 4 + col + 4 * g, float4{u[t][0], u[t][1], u[t][2], u[t][3]});
+    const int tile = part + 4 * t;
+    if (16 * tile < a.rankp) store4(out + 256 * tile, float4{u[t][0], u[t][1], u[t][2], u[t][3]});
   }
 }
 
 struct LatentExpand {
-  const float* partial;     // [B, H, S, rankp + 4]
+  const float* sums;        // as latent_decode_kernel leaves them
+  const float2* heads_in;   // [B, H, S]
   const float* sink;        // [H] or null
   const float* gate;        // gate projections, [b * gate_ld + h], or null
   const uint16_t* uv;       // [H, vdimp, rankp]
   uint16_t* out;            // [B, out_ld], head h at column h * vdimp
-  int batch, heads, chunks, rankp, vdimp, gate_ld, out_ld, groups;  // groups: workgroups per head (8 tiles each)
+  int batch, heads, chunks, rankp, vdimp, gate_ld, out_ld, groups;  // groups: workgroups per head
 };
-constexpr int kLatentMaxChunks = 32, kExpandBatch = 4, kExpandSteps = 16;  // rankp <= 32 kExpandSteps
-// A workgroup of 8 waves per (head, 4 sequences): the chunks are merged by all threads, then every wave expands the merged
-// latents to 16 value columns; its weights are requested first.  Grid (H * groups, batch blocks).
+constexpr int kLatentMaxChunks = 32, kExpandBatch = 4, kExpandRank = 512;
+// A workgroup of 8 waves per (head, TW 16-column tiles of values, 4 sequences): the chunks are merged by all threads, then
+// 8 / TW waves per tile expand the merged latents, a part of them each; their weights are requested first.  One CU takes in
+// some 40 KB per microsecond: for few sequences a head's weights (128 KB at 512 x 128) want several workgroups (TW = 2),
+// for more the merge, which every workgroup of a head repeats, wants few (TW = 8).  Grid (H * groups, batch blocks).
+template <int TW>
 __global__ __launch_bounds__(512) void latent_expand_kernel(LatentExpand a) {
+  constexpr int kParts = 8 / TW, kSteps = kExpandRank / 32 / kParts;
   extern __shared__ __attribute__((aligned(16))) uint16_t merged[];   // [kExpandBatch][rankp + 8] bf16
   __shared__ float weight[kExpandBatch][kLatentMaxChunks];
   __shared__ float4 part[512];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
   const int b0 = blockIdx.y * kExpandBatch, nb = min(kExpandBatch, a.batch - b0);
-  const int h = blockIdx.x / a.groups, tile = 8 * (blockIdx.x % a.groups) + wave;
-  const int stride = a.rankp + 4, ld = a.rankp + 8;
+  const int h = blockIdx.x / a.groups, tile = TW * (blockIdx.x % a.groups) + wave / kParts;
+  const int ld = a.rankp + 8;
   const u32x4_t zero = {0u, 0u, 0u, 0u};
   const bool active = 16 * tile < a.vdimp;
-  u32x4_t w[kExpandSteps];
-  const uint16_t* wrow = a.uv + ((size_t)h * a.vdimp + (active ? 16 * tile : 0) + r) * a.rankp + 8 * g;
+  const int k0 = 32 * kSteps * (wave % kParts) + 8 * g;
+  u32x4_t w[kSteps];
+  const uint16_t* wrow = a.uv + ((size_t)h * a.vdimp + (active ? 16 * tile : 0) + r) * a.rankp;
 #pragma unroll
-  for (int s = 0; s < kExpandSteps; ++s) {
+  for (int s = 0; s < kSteps; ++s) {
     w[s] = zero;
-    if (active && 32 * s + 8 * g < a.rankp) w[s] = *reinterpret_cast<const u32x4_t*>(wrow + 32 * s);
+    if (active && k0 + 32 * s < a.rankp) w[s] = *reinterpret_cast<const u32x4_t*>(wrow + k0 + 32 * s);
   }
   // merged[b] = sum over chunks; the threads of a column quad split the chunks where there are more threads than quads.
   // The first chunks' sums are requested before the chunks' weights are known.
@@ -483,15 +507,15 @@ __global__ __launch_bounds__(512) void latent_expand_kernel(LatentExpand a) {
   float4 ahead[kAhead];
   auto request = [&](int i, int s0) {
     const int b = min(i / quads, nb - 1), c = 4 * (i % quads);
-    const float* src = a.partial + ((size_t)(b0 + b) * a.heads + h) * a.chunks * stride + 4 + c;
+    const float* src = a.sums + latent_sums_at(b0 + b, h >> 4, 0, a.heads, a.chunks, a.rankp) + 256 * (c >> 4) + 16 * (h & 15) + (c & 15);
 #pragma unroll
-    for (int k = 0; k < kAhead; ++k) ahead[k] = load4(src + (size_t)min(s0 + k * split, a.chunks - 1) * stride);
+    for (int k = 0; k < kAhead; ++k) ahead[k] = load4(src + (size_t)min(s0 + k * split, a.chunks - 1) * (16 * a.rankp));
   };
   request(tid % span, which);
   if (wave < nb) {  // a wave per sequence, a lane per chunk
-    const float* src = a.partial + ((size_t)(b0 + wave) * a.heads + h) * a.chunks * stride;
     const bool mine = lane < a.chunks;
-    const float mx = mine ? src[lane * stride] : -INFINITY, sum = mine ? src[lane * stride + 1] : 0.f;
+    const float2 ml = mine ? a.heads_in[((size_t)(b0 + wave) * a.heads + h) * a.chunks + lane] : float2{-INFINITY, 0.f};
+    const float mx = ml.x, sum = ml.y;
     const float sink2 = a.sink ? a.sink[h] * kLog2eF : -INFINITY;
     const float top = fmaxf(wave_max64(mx), sink2);
     const float e = mx == -INFINITY ? 0.f : exp2f(mx - top);
@@ -523,13 +547,22 @@ __global__ __launch_bounds__(512) void latent_expand_kernel(LatentExpand a) {
     if (which == 0 && i < items) store4(merged + b * ld + 4 * (i % quads), sum);
   }
   __syncthreads();
-  if (!active) return;
   f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int s = 0; s < kExpandSteps; ++s) {
+  for (int s = 0; s < kSteps; ++s) {
     u32x4_t v = zero;
-    if (r < nb && 32 * s + 8 * g < a.rankp) v = *reinterpret_cast<const u32x4_t*>(merged + r * ld + 32 * s + 8 * g);
+    if (r < nb && k0 + 32 * s < a.rankp) v = *reinterpret_cast<const u32x4_t*>(merged + r * ld + k0 + 32 * s);
     acc = mfma16(w[s], v, acc);
+  }
+  if (kParts > 1) {
+    part[tid] = float4{acc[0], acc[1], acc[2], acc[3]};  // (last read before the barrier above)
+    __syncthreads();
+  }
+  if (wave % kParts != 0 || !active) return;
+#pragma unroll
+  for (int q = 1; q < kParts; ++q) {
+    const float4 v = part[tid + 64 * q];
+    acc[0] += v.x; acc[1] += v.y; acc[2] += v.z; acc[3] += v.w;
   }
   if (r >= nb) return;
   const float f = a.gate ? sigmoid_f32(a.gate[(size_t)(b0 + r) * a.gate_ld + h]) : 1.f;

@@ -33,7 +33,9 @@ from . import _lib
 from .modeling import Embedding, GatedFeedForward, Linear, RingCache, RMSNorm, build_norm, register_architecture
 
 GEMV_ROWS = 16    # rows of a prompt up to which the head's product is a matrix-vector kernel of this library
-NORM_PROLOGUE_ROWS = 4  # rows up to which the decode products form the norms themselves
+# rows up to which the decode products form the norms themselves (their workgroups each normalise every row: free at one
+# row, 7 us of 55 at two, where a norm launch costs 3)
+NORM_PROLOGUE_ROWS = 1
 
 
 @dataclass(frozen=True)
@@ -451,7 +453,7 @@ class LatentLM(nn.Module):
         _lib.check_dense(_lib.load_dense().ajqd_dense_in(ctypes.byref(args), _stream()), "dense_in")
 
     def _token_fused(self, x, delta, embedded, run: int, w: PackedBlock, ring, pos, chunks: int) -> None:
-        """One layer run in five launches (six above four sequences); x is updated in place, with what the next layer run
+        """One layer run in five launches (six for more than one sequence); x is updated in place, with what the next layer run
         adds first included."""
         lib, st, dtype, dev = _lib.load_dense(), _stream(), w.w1.dtype, x.device
         batch = x.shape[0]
@@ -470,7 +472,7 @@ class LatentLM(nn.Module):
         _lib.check_dense(lib.ajqd_latent_absorb(_ptr(y), y.shape[1], ctypes.byref(w.shape), _ptr(w.ukt), _ptr(w.latent_gain),
                                                 _ptr(w.cosine), _ptr(w.sine), self.context_length, _ptr(pos), _ptr(q), _ptr(ring),
                                                 ring.shape[1], batch, st), "latent_absorb")
-        partial = torch.empty((batch, w.heads, chunks, w.rankp + 4), dtype=torch.float32, device=dev)
+        partial = torch.empty(lib.ajqd_latent_decode_workspace(batch, w.heads, w.rankp, chunks), dtype=torch.uint8, device=dev)
         _lib.check_dense(lib.ajqd_latent_decode(_ptr(q), _ptr(ring), _ptr(pos), _ptr(partial), batch, w.heads, w.rankp, w.rotp,
                                                 ring.shape[1], chunks, w.scale, st), "latent_decode")
         gate = y.data_ptr() + 4 * w.gate_column if w.gated_heads else None

@@ -117,8 +117,9 @@ int ajqd_latent_absorb(const float* y, int ldy, const ajqd_latent_shape* shape, 
                        const float* cosine, const float* sine, int table_rows, const int64_t* pos, void* q, void* ring, int cap,
                        int batch, void* stream);
 
-/* row chunks ajqd_latent_decode uses, 0 where these widths are not built; partial: [batch, heads, chunks, rankp + 4] fp32 */
+/* row chunks ajqd_latent_decode uses, 0 where these widths are not built; bytes of the partial results it leaves */
 int ajqd_latent_decode_chunks(int batch, int heads, int rankp, int rotp, int cap);
+size_t ajqd_latent_decode_workspace(int batch, int heads, int rankp, int chunks);
 int ajqd_latent_decode(const void* q, const void* ring, const int64_t* pos, float* partial, int batch, int heads, int rankp,
                        int rotp, int cap, int chunks, float scale, void* stream);
 
