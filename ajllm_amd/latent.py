@@ -264,6 +264,8 @@ class LatentLM(nn.Module):
             raise ValueError("the model must be bfloat16 or float32")
         if weight.device.type != "cuda":
             raise ValueError("LatentLM runs on a ROCm device (there is no CPU path)")
+        if any(not isinstance(m, Linear) for layer in self.layers for m in layer.modules() if hasattr(m, "in_features")):
+            raise ValueError("LatentLM runs on dense weights (its linears have been replaced)")
         if any(p.dtype != weight.dtype or p.device != weight.device for p in self.parameters()):
             raise ValueError("all parameters must share one dtype and device")
         tables: dict = {}

@@ -17,6 +17,7 @@ Default run (what the driver calls: ``python bench.py --gpus 1 --steps K --warmu
   batch 1 and 8) in tokens/s, short form, and the Llama-3-8B-shaped W8A16 stack (4 x 2048 prefill passes,
   batch-32 decode at context 2048 with the quantized linears' share of the step), short form.
 
+``--latent`` adds the dense latent-attention decoder (its own libajq_dense.so) beside the W8A16 Transformer.
 ``--sweep`` adds the rest of the decode sweep (three shapes x M in {1, 4, 16}, W4 and W8)
 and all prefill shapes; ``--decode`` replaces the short decode leg by the long one (eager PyTorch loop
 beside it, token comparison between the two loops).  One JSON line is printed on stdout; everything else goes to stderr.
@@ -392,6 +393,9 @@ def main() -> int:
     ap.add_argument("--forms", action="store_true",
                     help="also time the decode GEMV's prologue forms against its epilogue forms (norm, gate, residual)")
     ap.add_argument("--no-cpu", action="store_true", help="skip the CPU baseline leg")
+    ap.add_argument("--latent", action="store_true",
+                    help="add the dense latent-attention decoder beside the W8A16 Transformer at two layer sizes: prompt and "
+                         "decode throughput, and every kernel's share of its roofline")
     ap.add_argument("--no-extras", action="store_true", help="timed region only")
     ap.add_argument("--no-decode", action="store_true",
                     help="skip the short end-to-end decode leg of the default line (counter-collection runs: "
@@ -505,6 +509,11 @@ def main() -> int:
         torch.cuda.empty_cache()
         extras["stack_8b_w8a16"] = bench_stack(device, log, short=not args.stack)
         torch.cuda.empty_cache()
+    if args.latent:
+        from ajllm_amd.latent_bench import bench_latent
+
+        torch.cuda.empty_cache()
+        extras["latent_attention_decoder"] = bench_latent(device, lambda name, row: log(name, json.dumps(row)))
     # a plain device-to-device copy of known size: the yardstick the FETCH_SIZE / WRITE_SIZE
     # counters of a profiling run are scaled by (64 MiB read + 64 MiB written per launch)
     calib_src = torch.empty(64 * 2**20, dtype=torch.uint8, device=device)

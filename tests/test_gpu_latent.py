@@ -237,6 +237,51 @@ def test_sinks_of_any_size(cuda, mfma):
         assert torch.isfinite(got).all() and float((got - want).abs().max()) < 2e-2
 
 
+DECODE_SHAPES = [  # batch, heads, rank, rot, vdim, rows of the ring, position
+    (1, 8, 96, 16, 80, 40, 500),       # a full ring, smaller than a block of rows
+    (3, 16, 48, 8, 32, 64, 63),        # exactly one block
+    (1, 5, 32, 16, 16, 65, 64),        # one row in the second block
+    (2, 33, 128, 24, 48, 200, 130),    # three head tiles, a ring that is partly filled
+    (5, 20, 272, 64, 64, 300, 1000),
+    (9, 32, 512, 64, 128, 1000, 5000),
+    (1, 128, 512, 64, 128, 129, 128),
+    (2, 4, 176, 8, 144, 70, 0),        # the very first token
+]
+
+
+@pytest.mark.parametrize("shape", DECODE_SHAPES)
+def test_latent_decode_and_expand_against_plain(cuda, shape):
+    """Attention in the latent space and the merge of its chunks, for every number of chunks, with one standing-out row."""
+    batch, heads, rank, rot, vdim, cap, position = shape
+    lib = _lib.load_dense()
+    g = torch.Generator().manual_seed(sum(shape))
+    bf = lambda *s: torch.randn(s, generator=g).to(torch.bfloat16)
+    q, ring, uv = bf(batch, heads, rank + rot), bf(batch, cap, rank + rot), bf(heads, vdim, rank)
+    sink, gate = torch.randn(heads, generator=g), torch.randn((batch, heads), generator=g)
+    valid = min(position, cap - 1) + 1
+    strong = valid - 1
+    ring[:, strong] *= 3
+    ring[:, valid:] = float("nan")   # never written rows must not be read
+    scale = 0.8 * (rank + rot) ** -0.5
+    scores = torch.matmul(q.double(), ring[:, :valid].double().transpose(1, 2)) * scale
+    weights = O.softmax_with_sink(scores, sink.double()[None, :].expand(batch, heads))
+    latents = torch.matmul(weights, ring[:, :valid, :rank].double())
+    want = (uv.double()[None] * latents[:, :, None, :]).sum(-1) * torch.sigmoid(gate.double())[:, :, None]
+    d = {k: v.to(cuda) for k, v in dict(q=q, ring=ring, uv=uv, sink=sink, gate=gate).items()}
+    pos = torch.tensor([position], device=cuda)
+    suggested = lib.ajqd_latent_decode_chunks(batch, heads, rank, rot, cap)
+    assert suggested >= 1
+    for chunks in sorted({1, 2, 3, 7, 32, suggested}):
+        partial = torch.full((lib.ajqd_latent_decode_workspace(batch, heads, rank, chunks),), 255, dtype=torch.uint8, device=cuda)
+        _ok(lib.ajqd_latent_decode(d["q"].data_ptr(), d["ring"].data_ptr(), pos.data_ptr(), partial.data_ptr(), batch, heads, rank, rot,
+                                   cap, chunks, scale, _st()))
+        out = torch.full((batch, heads * vdim + 8), 5.0, dtype=torch.bfloat16, device=cuda)
+        _ok(lib.ajqd_latent_expand(partial.data_ptr(), d["sink"].data_ptr(), d["gate"].data_ptr(), heads, d["uv"].data_ptr(),
+                                   out.data_ptr(), heads * vdim + 8, batch, heads, chunks, rank, vdim, _st()))
+        assert _rel(out[:, : heads * vdim], want.reshape(batch, -1)) < 8e-3, chunks
+        assert (out[:, heads * vdim:] == 5.0).all()
+
+
 # ------------------------------------------------------------------ the decoder against the plain implementation
 SHAPES = {
     "plain": {},
@@ -248,6 +293,8 @@ SHAPES = {
     "no loop": dict(loop=None, layers=2, window=[1, 2]),
     # one pass only (its vector is still added), the loop at the end, one head, a window no sequence here fills
     "one pass": dict(loop={"start": 2, "stop": 3, "times": 1}, heads=1, window=400),
+    # widths beyond the MFMA prompt kernel: operators of any width, also in bf16
+    "beyond": dict(layers=2, heads=2, dim=256, rot=16, vdim=272, loop=None, window=9),
     # wide: value tiles and key steps of a large model's layer, latents of several tiles per wave
     "wide": dict(layers=2, width=320, heads=2, dim=128, rot=64, vdim=128, rank=272, ff=520, window=70, loop={"start": 0, "stop": 1, "times": 2}),
 }
@@ -359,9 +406,9 @@ def test_a_cache_that_is_used_again_equals_a_fresh_one(cuda, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("batch", [2, 5, 17])
+@pytest.mark.parametrize("batch", [2, 5, 17, 37])
 def test_batch_rows_equal_sequences_alone(cuda, dtype, batch):
-    """Up to 4, up to 16 and more rows take different kernels; every row is its sequence's own."""
+    """One, up to 16, up to 32 and more rows take different kernels; every row is its sequence's own."""
     cfg = config(heads=3, window=[6, 20, 11])
     weights = random_weights(cfg, 17)
     model = _build(cfg, weights, cuda, dtype)
