@@ -6,9 +6,9 @@ arguments:
 * ``LatentAttention``    keys and values expanded per head from a low-rank latent, one rotated key part shared by all
                          heads, so that a position costs ``kv_rank + rot_dim`` cache elements; a sliding window (or
                          none), a learned sink per head in the softmax denominator, a sigmoid gate per head
-* ``ParallelBlock``      x + (mixer(norm1 x) + feed_forward(norm2 x))
-* ``Loop``               a span of layers that runs several times with the same weights; each pass has a cache of its own,
-                         and starts by adding a vector of its own (and, after the first, the embedding output) to x
+* ``ParallelBlock``      mixer and feed-forward side by side on two norms of the incoming stream, one sum at the end
+* ``Loop``               a span of layers traversed several times; every traversal has rings of its own in the cache and a
+                         learned offset for the stream it starts from, the later ones take the embedding in again as well
 * ``LatentLM``           the decoder: ``forward(token_ids, cache)`` is the one step function, for whole prompts, portions
                          of prompts and single tokens; ``modeling.greedy_decode`` and the decoders of ``decoding`` call it
 

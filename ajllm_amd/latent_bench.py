@@ -44,7 +44,8 @@ def build_latent(size: dict, device, seed: int = 77, dtype: torch.dtype = torch.
 
 
 def _graph_us(launches, reps: int = 20) -> float:
-    """Microseconds per launch of ``launches`` (a list of zero-argument calls), chained in a HIP graph."""
+    """Microseconds per launch of ``launches`` (a list of zero-argument calls), chained in a HIP graph of at least 48."""
+    launches = launches * max(1, 48 // len(launches))
     stream = torch.cuda.Stream()
     torch.cuda.synchronize()
     with torch.cuda.stream(stream):

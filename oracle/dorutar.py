@@ -14,12 +14,12 @@ import torch
 
 
 def embedding(tokens: list[int], table: torch.Tensor, positions: torch.Tensor, first: int = 0) -> torch.Tensor:
-    """Token row plus learned position row."""
+    """E[token] + P[position], row by row."""
     return torch.stack([table[t] + positions[first + i] for i, t in enumerate(tokens)])
 
 
 def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
-    """Mean removed, divided by the root of the mean squared deviation (+ eps), weighted; no bias."""
+    """d / sqrt(mean(d^2) + eps) * weight with d = row - mean(row)."""
     out = []
     for row in x:
         deviation = row - row.sum() / len(row)
@@ -58,7 +58,7 @@ def rotate_sequence(v: torch.Tensor, base: float, dims: int) -> torch.Tensor:
 
 
 def visible(i: int, j: int, window: int) -> bool:
-    """Whether the query at position i sees the key at position j: itself and the window - 1 tokens before it."""
+    """Whether the query at position i reads the key at position j: the last ``window`` positions up to and including i."""
     return 0 <= i - j < window
 
 
@@ -69,7 +69,7 @@ def window_mask(count: int, window: int) -> torch.Tensor:
 
 
 def softmax_with_sink(scores: torch.Tensor, sink: torch.Tensor | float) -> torch.Tensor:
-    """exp(s_j) / (exp(sink) + sum_j exp(s_j)) along the last dimension; ``sink`` broadcasts over the rest."""
+    """Softmax of (scores, sink) along the last dimension without the sink's own weight; ``sink`` broadcasts over the rest."""
     sink = torch.as_tensor(sink, dtype=scores.dtype)
     top = torch.maximum(scores.amax(dim=-1), sink)
     weights = torch.exp(scores - top.unsqueeze(-1))
@@ -102,7 +102,7 @@ def gated_relu(h: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, down: torc
 
 
 def parallel_layer(x: torch.Tensor, w: dict[str, torch.Tensor], layer: dict, eps: float) -> torch.Tensor:
-    """x + (mixer(norm1 x) + ff(norm2 x)), both from the same x."""
+    """Attention and feed-forward read the incoming stream, each through its own norm; both results join it at the end."""
     mix = {k[len("mix."):]: v for k, v in w.items() if k.startswith("mix.")}
     added = latent_attention(layer_norm(x, w["norm1"], eps), mix, layer["mixer"], eps)
     if layer.get("mlp") is not None:

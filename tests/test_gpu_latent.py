@@ -185,7 +185,7 @@ def _attention_gpu(c, prior, window, scale, cuda, dtype, mfma, sink=True, gates=
 ATTENTION_SHAPES = [  # b, h, t, prior, d1, d2, dv, window
     (1, 3, 150, 0, 16, 8, 32, 17),        # 1 key step
     (2, 4, 70, 31, 40, 8, 48, 32),        # 2 key steps, window exactly reached by the prior rows
-    (1, 8, 300, 0, 64, 24, 80, 64),       # 3
+    (1, 8, 300, 0, 72, 24, 96, 64),       # 3
     (1, 2, 129, 99, 96, 32, 112, 100),    # 4
     (1, 2, 260, 0, 128, 64, 128, 130),    # 6
     (1, 1, 90, 5, 192, 64, 256, 0),       # 8, no window
@@ -238,7 +238,7 @@ def test_sinks_of_any_size(cuda, mfma):
 
 
 DECODE_SHAPES = [  # batch, heads, rank, rot, vdim, rows of the ring, position
-    (1, 8, 96, 16, 80, 40, 500),       # a full ring, smaller than a block of rows
+    (1, 6, 112, 24, 48, 45, 500),      # a full ring, smaller than a block of rows
     (3, 16, 48, 8, 32, 64, 63),        # exactly one block
     (1, 5, 32, 16, 16, 65, 64),        # one row in the second block
     (2, 33, 128, 24, 48, 200, 130),    # three head tiles, a ring that is partly filled
@@ -290,6 +290,8 @@ SHAPES = {
     # more heads than a tile, another window per layer, a layer without a feed-forward, the loop at the start
     "heads": dict(width=96, heads=18, dim=24, rot=16, vdim=40, rank=72, ff=64, window=[5, 33, 64], mlp_missing=(1,),
                   loop={"start": 0, "stop": 3, "times": 2}),
+    # constants far from the usual: an eps that dominates, fast rotations, a large score scale
+    "constants": dict(layers=2, eps=0.4, base=3.0, scale=0.9, loop={"start": 0, "stop": 2, "times": 2}, window=[19, 20]),
     "no loop": dict(loop=None, layers=2, window=[1, 2]),
     # one pass only (its vector is still added), the loop at the end, one head, a window no sequence here fills
     "one pass": dict(loop={"start": 2, "stop": 3, "times": 1}, heads=1, window=400),
