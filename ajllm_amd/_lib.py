@@ -146,7 +146,7 @@ DENSE_LIBRARY_PATH = Path(__file__).resolve().parent / "libajq_dense.so"
 
 AJQD_BF16 = 0
 AJQD_F32 = 1
-AJQD_ACTIVATIONS = {"relu": 0, "silu": 1, "gelu_tanh": 2}
+AJQD_ACTIVATIONS = {"relu": 0, "silu": 1, "gelu_tanh": 2, "squared_relu": 3}
 
 
 class LatentShape(ctypes.Structure):
@@ -158,10 +158,10 @@ class LatentShape(ctypes.Structure):
 class WindowedAttentionArgs(ctypes.Structure):
     """``ajqd_windowed_attention_args``"""
 
-    _fields_ = ([(n, c_void_p) for n in ("q", "k1", "k2", "v", "sink", "gates", "pos", "out")]
-                + [(n, c_int64) for n in ("k1_batch", "k2_batch", "v_batch")]
-                + [(n, c_int) for n in ("k1_row", "k1_head", "k2_row", "v_row", "v_head", "d1", "d2", "dv", "batch",
-                                        "heads", "seq", "rows", "prior", "window", "out_ld")]
+    _fields_ = ([(n, c_void_p) for n in ("q", "k1", "k2", "v", "sink", "gates", "column_gates", "pos", "out")]
+                + [(n, c_int64) for n in ("k1_batch", "k2_batch", "v_batch", "k1_head", "v_head")]
+                + [(n, c_int) for n in ("k1_row", "k2_row", "v_row", "d1", "d2", "dv", "batch", "heads", "share", "seq", "rows",
+                                        "prior", "window", "keep", "gate_ld", "out_ld")]
                 + [("scale", c_float)])
 
 
@@ -169,8 +169,33 @@ class DenseInArgs(ctypes.Structure):
     """``ajqd_dense_in_args``"""
 
     _fields_ = ([(n, c_void_p) for n in ("x", "n1", "n2", "gain1", "gain2", "w1", "w2", "y1", "gated")]
-                + [(n, c_int) for n in ("batch", "true_width", "width", "tiles1", "tiles2", "gated_ld", "act", "center")]
+                + [(n, c_int) for n in ("batch", "true_width", "width", "tiles1", "tiles2", "gated_ld", "act", "center", "pairs")]
                 + [("eps", c_float)])
+
+
+class KeyValueSplitArgs(ctypes.Structure):
+    """``ajqd_key_value_split_args``"""
+
+    _fields_ = ([(n, c_void_p) for n in ("y", "q_gain", "k_gain", "half_turns", "pos", "q", "rows")]
+                + [(n, c_int64) for n in ("rows_batch", "rows_head")]
+                + [(n, c_int) for n in ("tokens", "seq", "start", "ldy", "heads", "groups", "dim", "dimp", "rot", "q_ld", "q_at", "prior",
+                                        "cap", "kept")]
+                + [("eps", c_float)])
+
+
+class ScanArgs(ctypes.Structure):
+    """``ajqd_scan_args``"""
+
+    _fields_ = ([(n, c_void_p) for n in ("x", "dt", "low", "z", "a2", "d", "dt_bias", "state", "pos", "out")]
+                + [(n, c_int) for n in ("batch", "seq", "start", "inner", "states", "dt_ld", "low_ld", "b_col", "c_col", "z_ld",
+                                        "out_ld")])
+
+
+class ScanStepArgs(ctypes.Structure):
+    """``ajqd_scan_step_args``"""
+
+    _fields_ = ([(n, c_void_p) for n in ("y", "ring", "weight", "bias", "pos", "partial", "w_dt", "dt_bias", "a2", "d", "state", "out")]
+                + [(n, c_int) for n in ("batch", "ldy", "inner", "taps", "rows", "splits", "rank", "states", "out_ld")])
 
 
 _P, _I, _F, _L = c_void_p, c_int, c_float, c_int64
@@ -180,7 +205,7 @@ DENSE_SIGNATURES: dict[str, tuple] = {
     "ajqd_add_norms": (c_int, [_P, _P, _I, _P, _P, _P, _P, _F, _I, _P, _P, _I, _I, _I, _I, _P]),
     "ajqd_latent_split": (c_int, [_P, _I, _I, ctypes.POINTER(LatentShape), _P, _P, _P, _I, _I, _I, _I, _P, _I, _I, _P, _I, _P,
                                   _I, _P, _L, _P, _I, _P]),
-    "ajqd_ring_copy": (c_int, [_P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P]),
+    "ajqd_ring_copy": (c_int, [_P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P]),
     "ajqd_gated_activation": (c_int, [_P, _I, _P, _I, _I, _I, _I, _I, _P]),
     "ajqd_matvec": (c_int, [_P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P]),
     "ajqd_windowed_attention": (c_int, [ctypes.POINTER(WindowedAttentionArgs), _I, _I, _P]),
@@ -191,8 +216,19 @@ DENSE_SIGNATURES: dict[str, tuple] = {
     "ajqd_latent_absorb": (c_int, [_P, _I, ctypes.POINTER(LatentShape), _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _P]),
     "ajqd_latent_decode_chunks": (c_int, [_I, _I, _I, _I, _I]),
     "ajqd_latent_decode_workspace": (c_size_t, [_I, _I, _I, _I]),
-    "ajqd_latent_decode": (c_int, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P]),
+    "ajqd_latent_decode": (c_int, [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P]),
     "ajqd_latent_expand": (c_int, [_P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P]),
+    "ajqd_embed_streams": (c_int, [_P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _P]),
+    "ajqd_streams_norm": (c_int, [_P, _P, _P, _P, _P, _P, _P, _F, _P, _P, _I, _I, _I, _I, _I, _P]),
+    "ajqd_dense_out_streams": (c_int, [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P]),
+    "ajqd_activation": (c_int, [_P, _P, _L, _I, _I, _P]),
+    "ajqd_key_value_split": (c_int, [ctypes.POINTER(KeyValueSplitArgs), _I, _I, _P]),
+    "ajqd_group_merge": (c_int, [_P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P]),
+    "ajqd_conv_silu": (c_int, [_P, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _P, _I, _P]),
+    "ajqd_scan": (c_int, [ctypes.POINTER(ScanArgs), _I, _P]),
+    "ajqd_scan_splits": (c_int, [_I, _I]),
+    "ajqd_scan_project": (c_int, [_P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P]),
+    "ajqd_scan_step": (c_int, [ctypes.POINTER(ScanStepArgs), _P]),
 }
 
 _lib: ctypes.CDLL | None = None

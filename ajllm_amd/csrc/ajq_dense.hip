@@ -7,6 +7,9 @@
 #include "dense_kernels.h"
 #include "latent_attention.h"
 #include "dense_gemv_kernels.h"
+#include "grouped_attention.h"
+#include "scan_kernels.h"
+#include "stream_kernels.h"
 
 using namespace ajq;
 
@@ -63,16 +66,17 @@ LatentShape device_shape(const ajqd_latent_shape* s) {
 }
 
 int check_attention(const ajqd_windowed_attention_args* a, const char* what) {
-  if (!a || !a->q || !a->k1 || !a->k2 || !a->v || !a->out) return fail(AJQ_ERR_NULL, "%s: null pointer argument", what);
-  if (a->batch < 1 || a->heads < 1 || a->seq < 1 || a->rows < 1 || a->prior < 0 || a->d1 < 8 || a->d2 < 8 || a->dv < 16 ||
-      a->d1 % 8 || a->d2 % 8 || a->dv % 16 || a->out_ld < a->heads * a->dv || a->out_ld % 4)
+  if (!a || !a->q || !a->k1 || (a->d2 && !a->k2) || !a->v || !a->out) return fail(AJQ_ERR_NULL, "%s: null pointer argument", what);
+  if (a->batch < 1 || a->heads < 1 || a->seq < 1 || a->rows < 1 || a->prior < 0 || a->d1 < 8 || a->d2 < 0 || a->dv < 16 ||
+      a->d1 % 8 || a->d2 % 8 || a->dv % 16 || a->out_ld < a->heads * a->dv || a->out_ld % 4 || a->keep < 0 || a->share < 0 ||
+      (a->share > 1 && a->heads % a->share) || (a->column_gates && (a->gate_ld < a->heads * a->dv || a->gate_ld % 4)))
     return fail(AJQ_ERR_SHAPE, "%s: unsupported shape (B=%d H=%d T=%d rows=%d prior=%d d=%d+%d dv=%d)", what, a->batch, a->heads,
                 a->seq, a->rows, a->prior, a->d1, a->d2, a->dv);
   if (a->pos ? a->seq != 1 : (long long)a->prior + a->seq > a->rows)
     return fail(AJQ_ERR_SHAPE, "%s: %d + %d queries do not fit %d rows", what, a->prior, a->seq, a->rows);
   if (!(a->scale > 0.f)) return fail(AJQ_ERR_SHAPE, "%s: the score scale must be positive", what);
   if (a->k1_row % 8 || a->k1_head % 8 || a->k2_row % 8 || a->v_row % 8 || a->v_head % 8 || a->k1_batch % 8 || a->k2_batch % 8 ||
-      a->v_batch % 8 || !aligned16(a->q) || !aligned16(a->k1) || !aligned16(a->k2) || !aligned16(a->v) || !aligned16(a->out))
+      a->v_batch % 8 || !aligned16(a->q) || !aligned16(a->k1) || !aligned16(a->k2) || !aligned16(a->v) || !aligned16(a->out) || !aligned16(a->column_gates))
     return fail(AJQ_ERR_ALIGN, "%s: rows must start on 16-byte boundaries", what);
   return AJQ_OK;
 }
@@ -84,6 +88,7 @@ WindowedAttention device_attention(const ajqd_windowed_attention_args* a) {
   w.k1_row = a->k1_row; w.k1_head = a->k1_head; w.k2_row = a->k2_row; w.v_row = a->v_row; w.v_head = a->v_head;
   w.d1 = a->d1; w.d2 = a->d2; w.dv = a->dv;
   w.batch = a->batch; w.heads = a->heads; w.seq = a->seq;
+  w.keep = a->keep; w.share = a->share > 1 ? a->share : 1; w.gate_ld = a->gate_ld; w.column_gates = a->column_gates;
   w.rows = a->rows; w.prior = a->prior; w.window = a->window; w.out_ld = a->out_ld; w.scale = a->scale;
   return w;
 }
@@ -122,6 +127,38 @@ float2* heads_at(const float* partial, int batch, int heads, int chunks, int ran
 }
 constexpr int kDecodeWorkgroups = 256;  // one per CU (its LDS holds two blocks of rows)
 int latent_head_groups(int heads) { return heads <= 16 ? 1 : (heads + 31) / 32; }  // one or two head tiles per workgroup
+// ---- several residual streams
+int stream_room(int s) { return s <= 2 ? 2 : s <= 4 ? 4 : kMaxStreams; }
+int check_streams(int streams, const char* what) {
+  if (streams < 1 || streams > kMaxStreams) return fail(AJQ_ERR_UNSUPPORTED, "%s: %d streams (1 .. %d are built)", what, streams, kMaxStreams);
+  return AJQ_OK;
+}
+
+// ---- selective scan: lanes per channel and states per lane.  More lanes than the states ask for where there are few channels:
+// the time loop is sequential, so what counts then is its length per step and not the work.
+template <typename T>
+int launch_scan(const Scan& a, int batch, hipStream_t stream) {
+  const long long lanes = (long long)batch * a.inner;
+  auto go = [&](auto kernel, int per_channel) {
+    const int channels = 256 / per_channel;
+    hipLaunchKernelGGL(kernel, dim3((a.inner + channels - 1) / channels, batch), dim3(256), 0, stream, a);
+    return check_launch("ajqd_scan");
+  };
+  const bool few = lanes * 4 < 2 * 65536, fewer = lanes * 8 < 2 * 65536;  // (65536 lanes: a wave on every SIMD)
+  const int n = a.states;
+  if (n <= 16 && fewer) return go(scan_kernel<T, 16, 1>, 16);
+  if (n <= 16 && few) return go(scan_kernel<T, 8, 2>, 8);
+  if (n <= 16) return go(scan_kernel<T, 4, 4>, 4);
+  if (n <= 32 && fewer) return go(scan_kernel<T, 16, 2>, 16);
+  if (n <= 32 && few) return go(scan_kernel<T, 8, 4>, 8);
+  if (n <= 24) return go(scan_kernel<T, 4, 6>, 4);
+  if (n <= 32) return go(scan_kernel<T, 4, 8>, 4);
+  if (n <= 64) return few ? go(scan_kernel<T, 16, 4>, 16) : go(scan_kernel<T, 8, 8>, 8);
+  if (n <= 128) return go(scan_kernel<T, 16, 8>, 16);
+  if (n <= 256) return go(scan_kernel<T, 32, 8>, 32);
+  return fail(AJQ_ERR_UNSUPPORTED, "ajqd_scan: %d states per channel (up to 256 are built)", n);
+}
+
 int gemv_waves(int k) { return k >= 2048 ? 8 : k >= 256 ? 4 : 1; }
 
 }  // namespace
@@ -188,18 +225,19 @@ int ajqd_latent_split(const void* y, int y_dtype, int ldy, const ajqd_latent_sha
   return check_launch("ajqd_latent_split");
 }
 
-int ajqd_ring_copy(void* ring, int cap, void* linear, int lines, int first_row, int position, int count, int row_bytes,
-                   int batch, int to_ring, void* stream) {
+int ajqd_ring_copy(void* ring, int cap, int kept, void* linear, int lines, int line_bytes, int first_row, int position, int count,
+                   int row_bytes, int batch, int to_ring, void* stream) {
   if (!ring || !linear) return fail(AJQ_ERR_NULL, "ajqd_ring_copy: null pointer argument");
-  if (cap < 1 || count < 1 || count > cap || first_row < 0 || (long long)first_row + count > lines || position < 0 || batch < 1 ||
-      row_bytes < 16 || row_bytes % 16)
+  if (cap < 1 || kept < 0 || kept > cap || count < 1 || first_row < 0 || (long long)first_row + count > lines || position < 0 ||
+      batch < 1 || row_bytes < 16 || row_bytes % 16 || line_bytes < row_bytes || line_bytes % 16 ||
+      (long long)position + count - (position > kept ? position : kept) > cap - kept)
     return fail(AJQ_ERR_SHAPE, "ajqd_ring_copy: unsupported shape (cap=%d lines=%d first=%d position=%d count=%d)", cap, lines,
                 first_row, position, count);
   if (!aligned16(ring) || !aligned16(linear)) return fail(AJQ_ERR_ALIGN, "ajqd_ring_copy: buffers must be 16-byte aligned");
   const long long blocks = ((long long)batch * count * (row_bytes / 16) + 255) / 256;
   if (blocks > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_ring_copy: too many elements");
-  hipLaunchKernelGGL(ring_copy_kernel, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (u32x4_t*)ring, cap,
-                     (u32x4_t*)linear, lines, first_row, position, count, row_bytes / 16, batch, to_ring);
+  hipLaunchKernelGGL(ring_copy_kernel, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (u32x4_t*)ring, cap, kept,
+                     (u32x4_t*)linear, lines, line_bytes / 16, first_row, position, count, row_bytes / 16, batch, to_ring);
   return check_launch("ajqd_ring_copy");
 }
 
@@ -208,7 +246,7 @@ int ajqd_gated_activation(const void* y, int y_dtype, void* out, int out_ld, int
   if (!y || !out) return fail(AJQ_ERR_NULL, "ajqd_gated_activation: null pointer argument");
   if (rows < 1 || width < 8 || width % 8 || out_ld < width || out_ld % 4)
     return fail(AJQ_ERR_SHAPE, "ajqd_gated_activation: unsupported shape (rows=%d width=%d out_ld=%d)", rows, width, out_ld);
-  if (!known(dtype) || !known(y_dtype) || act < 0 || act > AJQD_ACT_GELU_TANH)
+  if (!known(dtype) || !known(y_dtype) || act < 0 || act > AJQD_ACT_SQUARED_RELU)
     return fail(AJQ_ERR_UNSUPPORTED, "ajqd_gated_activation: unknown dtype or activation");
   const long long blocks = ((long long)rows * (width / 4) + 255) / 256;
   if (blocks > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_gated_activation: too many elements");
@@ -278,16 +316,16 @@ int ajqd_dense_in(const ajqd_dense_in_args* a, void* stream) {
       (a->tiles1 && (!a->w1 || !a->y1)) || (a->tiles2 && (!a->w2 || !a->gated)))
     return fail(AJQ_ERR_NULL, "ajqd_dense_in: null pointer argument");
   if (a->batch < 1 || a->true_width < 1 || a->width < a->true_width || a->width % 8 || a->tiles1 < 0 || a->tiles2 < 0 ||
-      a->tiles1 + a->tiles2 < 1 || (a->tiles2 && (a->gated_ld < 8 * a->tiles2 || a->gated_ld % 4)))
+      a->tiles1 + a->tiles2 < 1 || (a->tiles2 && (a->gated_ld < (a->pairs ? 8 : 16) * a->tiles2 || a->gated_ld % 4)))
     return fail(AJQ_ERR_SHAPE, "ajqd_dense_in: unsupported shape (batch=%d width=%d/%d tiles=%d+%d)", a->batch, a->true_width,
                 a->width, a->tiles1, a->tiles2);
-  if (a->act < 0 || a->act > AJQD_ACT_GELU_TANH) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_dense_in: unknown activation");
+  if (a->act < 0 || a->act > AJQD_ACT_SQUARED_RELU) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_dense_in: unknown activation");
   if (a->x && a->batch > 4) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_dense_in: the norm prologue takes at most 4 rows");
   DenseIn d;
   d.x = a->x; d.n1 = (const uint16_t*)a->n1; d.n2 = (const uint16_t*)a->n2; d.gain1 = a->gain1; d.gain2 = a->gain2;
   d.w1 = (const uint16_t*)a->w1; d.w2 = (const uint16_t*)a->w2; d.y1 = a->y1; d.gated = (uint16_t*)a->gated;
   d.batch = a->batch; d.D = a->true_width; d.Dp = a->width; d.tiles1 = a->tiles1; d.tiles2 = a->tiles2;
-  d.gated_ld = a->gated_ld; d.act = a->act; d.center = a->center; d.eps = a->eps;
+  d.gated_ld = a->gated_ld; d.act = a->act; d.center = a->center; d.pairs = a->pairs; d.eps = a->eps;
   // more than 16 sequences: two batch tiles and (from two tiles of rows on) two row tiles per workgroup
   const bool wide = a->batch > kGemvBatch;
   const int block = wide ? 2 * kGemvBatch : kGemvBatch;
@@ -367,14 +405,14 @@ size_t ajqd_latent_decode_workspace(int batch, int heads, int rankp, int chunks)
 }
 
 int ajqd_latent_decode(const void* q, const void* ring, const int64_t* pos, float* partial, int batch, int heads, int rankp,
-                       int rotp, int cap, int chunks, float scale, void* stream) {
+                       int rotp, int cap, int chunks, int first_column, float scale, void* stream) {
   if (!q || !ring || !pos || !partial) return fail(AJQ_ERR_NULL, "ajqd_latent_decode: null pointer argument");
   if (ajqd_latent_decode_chunks(batch, heads, rankp, rotp, cap) == 0)
     return fail(AJQ_ERR_UNSUPPORTED, "ajqd_latent_decode: widths %d + %d are not built", rankp, rotp);
-  if (chunks < 1 || chunks > kLatentMaxChunks || !(scale > 0.f))
+  if (chunks < 1 || chunks > kLatentMaxChunks || first_column < 0 || first_column >= rankp + rotp || !(scale > 0.f))
     return fail(AJQ_ERR_SHAPE, "ajqd_latent_decode: unsupported shape (batch=%d chunks=%d)", batch, chunks);
   LatentDecode d{(const uint16_t*)q, (const uint16_t*)ring, positions64(pos), partial,
-                 heads_at(partial, batch, heads, chunks, rankp), batch, heads, rankp, rankp + rotp, cap, chunks, scale * kLog2eF};
+                 heads_at(partial, batch, heads, chunks, rankp), batch, heads, rankp, rankp + rotp, cap, chunks, first_column / 32, scale * kLog2eF};
   const long long blocks = (long long)latent_head_groups(heads) * chunks * batch;
   if (blocks > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_latent_decode: too many workgroups");
   const bool two = heads > 16;
@@ -410,6 +448,210 @@ int ajqd_latent_expand(const float* partial, const float* sink, const float* gat
   hipLaunchKernelGGL(few ? latent_expand_kernel<2> : latent_expand_kernel<8>, dim3(heads * groups, (batch + kExpandBatch - 1) / kExpandBatch), dim3(512), bytes,
                      (hipStream_t)stream, d);
   return check_launch("ajqd_latent_expand");
+}
+
+// ---- several residual streams
+int ajqd_embed_streams(const int64_t* tokens, int rows, const void* table, int vocab, const float* in, float* x, float* u, int streams,
+                       int width, int dtype, void* stream) {
+  if (!tokens || !table || !x || (u && !in)) return fail(AJQ_ERR_NULL, "ajqd_embed_streams: null pointer argument");
+  if (int e = check_streams(streams, "ajqd_embed_streams")) return e;
+  if (rows < 1 || vocab < 1 || width < 8 || width % 8)
+    return fail(AJQ_ERR_SHAPE, "ajqd_embed_streams: unsupported shape (rows=%d vocab=%d width=%d)", rows, vocab, width);
+  if (!known(dtype)) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_embed_streams: unknown dtype %d", dtype);
+  with_types(dtype, dtype, [&](auto t, auto) {
+    using T = decltype(t);
+    hipLaunchKernelGGL(embed_streams_kernel<T>, dim3(rows), dim3(256), 0, (hipStream_t)stream, (const long long*)tokens, (const T*)table,
+                       vocab, in, x, u, streams, width);
+  });
+  return check_launch("ajqd_embed_streams");
+}
+
+int ajqd_streams_norm(float* x, const float* delta, const float* scale, const float* out, const float* mix, const float* in,
+                      const float* gain, float eps, void* normed, float* u, int streams, int rows, int true_width, int width, int dtype,
+                      void* stream) {
+  if (!x || (delta && (!scale || !out || !mix)) || (normed && !gain)) return fail(AJQ_ERR_NULL, "ajqd_streams_norm: null pointer argument");
+  if (int e = check_streams(streams, "ajqd_streams_norm")) return e;
+  if (rows < 1 || true_width < 1 || width < true_width || width % 8)
+    return fail(AJQ_ERR_SHAPE, "ajqd_streams_norm: unsupported shape (rows=%d width=%d of %d)", rows, true_width, width);
+  if (!known(dtype)) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_streams_norm: unknown dtype %d", dtype);
+  with_types(dtype, dtype, [&](auto t, auto) {
+    using T = decltype(t);
+    auto go = [&](auto kernel) {
+      hipLaunchKernelGGL(kernel, dim3(rows), dim3(256), 0, (hipStream_t)stream, x, delta, scale, out, mix, in, gain, eps, (T*)normed, u,
+                         streams, true_width, width);
+    };
+    switch (stream_room(streams)) {
+      case 2: go(streams_norm_kernel<T, 2>); break;
+      case 4: go(streams_norm_kernel<T, 4>); break;
+      default: go(streams_norm_kernel<T, kMaxStreams>); break;
+    }
+  });
+  return check_launch("ajqd_streams_norm");
+}
+
+int ajqd_dense_out_streams(const void* in, const void* w, float* x, const float* scale, const float* out, const float* mix,
+                           const float* next, float* u, int streams, int batch, int k, int width, void* stream) {
+  if (!in || !w || !x || !scale || !out || !mix || !u) return fail(AJQ_ERR_NULL, "ajqd_dense_out_streams: null pointer argument");
+  if (int e = check_streams(streams, "ajqd_dense_out_streams")) return e;
+  if (batch < 1 || k < 8 || k % 8 || width < 16 || width % 16)
+    return fail(AJQ_ERR_SHAPE, "ajqd_dense_out_streams: unsupported shape (batch=%d k=%d width=%d)", batch, k, width);
+  DenseOutStreams d{(const uint16_t*)in, (const uint16_t*)w, x, scale, out, mix, next, u, batch, k, width, streams};
+  const bool wide = batch > kGemvBatch;
+  const int block = wide ? 2 * kGemvBatch : kGemvBatch;
+  const int rt = wide && width % 32 == 0 && width >= 8192 ? 2 : 1;
+  const dim3 grid(width / (16 * rt), (batch + block - 1) / block);
+  auto go = [&](auto kernel, int threads) {
+    hipLaunchKernelGGL(kernel, grid, dim3(threads), 0, (hipStream_t)stream, d);
+    return check_launch("ajqd_dense_out_streams");
+  };
+  auto pick = [&](auto room) {
+    constexpr int M = decltype(room)::value;
+    const int waves = gemv_waves(k);
+    if (rt == 2) return waves == 8 ? go(dense_out_streams_kernel<8, 2, 2, M>, 512) : waves == 4 ? go(dense_out_streams_kernel<4, 2, 2, M>, 256)
+                                                                                               : go(dense_out_streams_kernel<1, 2, 2, M>, 64);
+    if (wide) return waves == 8 ? go(dense_out_streams_kernel<8, 1, 2, M>, 512) : waves == 4 ? go(dense_out_streams_kernel<4, 1, 2, M>, 256)
+                                                                                            : go(dense_out_streams_kernel<1, 1, 2, M>, 64);
+    return waves == 8 ? go(dense_out_streams_kernel<8, 1, 1, M>, 512) : waves == 4 ? go(dense_out_streams_kernel<4, 1, 1, M>, 256)
+                                                                                  : go(dense_out_streams_kernel<1, 1, 1, M>, 64);
+  };
+  switch (stream_room(streams)) {
+    case 2: return pick(std::integral_constant<int, 2>{});
+    case 4: return pick(std::integral_constant<int, 4>{});
+    default: return pick(std::integral_constant<int, kMaxStreams>{});
+  }
+}
+
+int ajqd_activation(const void* y, void* out, int64_t count, int act, int dtype, void* stream) {
+  if (!y || !out) return fail(AJQ_ERR_NULL, "ajqd_activation: null pointer argument");
+  if (count < 8 || count % 8 || count / 8 / 256 > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_activation: unsupported count %lld", (long long)count);
+  if (!aligned16(y) || !aligned16(out)) return fail(AJQ_ERR_ALIGN, "ajqd_activation: buffers must be 16-byte aligned");
+  if (!known(dtype) || act < 0 || act > AJQD_ACT_SQUARED_RELU) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_activation: unknown dtype or activation");
+  with_types(dtype, dtype, [&](auto t, auto) {
+    using T = decltype(t);
+    hipLaunchKernelGGL(activation_kernel<T>, dim3((unsigned)((count / 8 + 255) / 256)), dim3(256), 0, (hipStream_t)stream, (const T*)y, (T*)out,
+                       (long long)count / 8, act);
+  });
+  return check_launch("ajqd_activation");
+}
+
+// ---- grouped-query attention
+int ajqd_key_value_split(const ajqd_key_value_split_args* a, int y_dtype, int dtype, void* stream) {
+  if (!a || !a->y || !a->q_gain || !a->k_gain || (a->rot && !a->half_turns) || !a->q || !a->rows)
+    return fail(AJQ_ERR_NULL, "ajqd_key_value_split: null pointer argument");
+  if (a->tokens < 1 || a->seq < 1 || a->tokens % a->seq || a->heads < 1 || a->groups < 1 || a->dim < 1 || a->dimp < a->dim || a->dimp % 16 ||
+      a->rot < 0 || a->rot % 2 || a->rot > a->dim || a->start < 0 || a->ldy < (a->heads + a->groups) * a->dimp || a->ldy % 4 || a->q_at < 0 ||
+      a->q_at % 4 || a->q_ld < a->q_at + a->dimp || a->q_ld % 4 || a->prior < 0 || a->rows_batch < 0 || a->rows_head < 0 || a->rows_batch % 8 ||
+      a->rows_head % 8 || (a->pos ? (a->seq != 1 || a->cap < 1 || a->kept < 0 || a->kept >= a->cap) : (int64_t)a->start + a->seq > 0x7FFFFFFF))
+    return fail(AJQ_ERR_SHAPE, "ajqd_key_value_split: unsupported shape (tokens=%d seq=%d heads=%d groups=%d dim=%d/%d rot=%d cap=%d kept=%d)",
+                a->tokens, a->seq, a->heads, a->groups, a->dim, a->dimp, a->rot, a->cap, a->kept);
+  const int64_t need = (int64_t)(a->pos ? a->cap : a->prior + a->seq) * 2 * a->dimp;
+  if ((a->groups > 1 && a->rows_head < need) || (a->tokens > a->seq && a->rows_batch < need))
+    return fail(AJQ_ERR_SHAPE, "ajqd_key_value_split: rows of neighbouring heads or sequences overlap");
+  if (!known(dtype) || !known(y_dtype)) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_key_value_split: unknown dtype");
+  if (!aligned16(a->y) || !aligned16(a->q) || !aligned16(a->rows)) return fail(AJQ_ERR_ALIGN, "ajqd_key_value_split: rows must be 16-byte aligned");
+  KeyValueSplit k;
+  k.y = a->y; k.ldy = a->ldy; k.s = KeyValueShape{a->heads, a->groups, a->dim, a->dimp, a->rot, a->eps};
+  k.q_gain = a->q_gain; k.k_gain = a->k_gain; k.half_turns = a->half_turns; k.start = a->start; k.pos = positions64(a->pos);
+  k.seq = a->seq; k.prior = a->prior; k.cap = a->cap; k.kept = a->kept; k.q = a->q; k.q_ld = a->q_ld; k.q_at = a->q_at;
+  k.rows = a->rows; k.rows_batch = a->rows_batch; k.rows_head = a->rows_head;
+  const int bytes = 4 * 2 * ((a->rot / 2 + 3) & ~3);
+  int status = AJQ_OK;
+  with_types(y_dtype, dtype, [&](auto yt, auto t) {
+    using Y = decltype(yt);
+    using T = decltype(t);
+    auto go = [&](auto kernel) {
+      status = allow_lds(kernel, bytes, "ajqd_key_value_split");
+      if (status == AJQ_OK) hipLaunchKernelGGL(kernel, dim3(a->tokens), dim3(256), bytes, (hipStream_t)stream, k);
+    };
+    if (a->dimp <= 64) go(key_value_split_kernel<Y, T, 16>);
+    else if (a->dimp <= 128) go(key_value_split_kernel<Y, T, 32>);
+    else go(key_value_split_kernel<Y, T, 64>);
+  });
+  return status != AJQ_OK ? status : check_launch("ajqd_key_value_split");
+}
+
+int ajqd_group_merge(const float* partial, const float* gate, int gate_ld, void* out, int out_ld, int batch, int groups, int share,
+                     int chunks, int dimp, void* stream) {
+  if (!partial || !out) return fail(AJQ_ERR_NULL, "ajqd_group_merge: null pointer argument");
+  if (batch < 1 || groups < 1 || share < 1 || chunks < 1 || chunks > kLatentMaxChunks || dimp < 16 || dimp % 16 || dimp > 1024 ||
+      out_ld < groups * share * dimp || out_ld % 4 || (gate && (gate_ld < groups * share * dimp || gate_ld % 4)) ||
+      (long long)batch * groups * share > 0x7FFFFFFFll)
+    return fail(AJQ_ERR_SHAPE, "ajqd_group_merge: unsupported shape (batch=%d groups=%d share=%d chunks=%d dimp=%d)", batch, groups, share,
+                chunks, dimp);
+  GroupMerge m{partial, heads_at(partial, batch * groups, share, chunks, dimp), gate, (uint16_t*)out, groups, share, chunks, dimp, gate_ld, out_ld};
+  hipLaunchKernelGGL(group_merge_kernel, dim3(batch * groups * share), dim3(256), 0, (hipStream_t)stream, m);
+  return check_launch("ajqd_group_merge");
+}
+
+// ---- selective scan
+int ajqd_conv_silu(const void* y, int ldy, void* ring, const float* weight, const float* bias, int start, const int64_t* pos, int rows,
+                   int seq, int inner, int taps, void* out, int dtype, void* stream) {
+  if (!y || !weight || !bias || !out || (!ring && taps > 1 && (start > 0 || pos))) return fail(AJQ_ERR_NULL, "ajqd_conv_silu: null pointer argument");
+  if (rows < 1 || seq < 1 || rows % seq || inner < 8 || inner % 8 || taps < 1 || ldy < inner || ldy % 8 || start < 0 || (pos && seq != 1))
+    return fail(AJQ_ERR_SHAPE, "ajqd_conv_silu: unsupported shape (rows=%d seq=%d inner=%d taps=%d ldy=%d)", rows, seq, inner, taps, ldy);
+  if (!known(dtype)) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_conv_silu: unknown dtype %d", dtype);
+  if (!aligned16(y) || !aligned16(ring) || !aligned16(out)) return fail(AJQ_ERR_ALIGN, "ajqd_conv_silu: rows must be 16-byte aligned");
+  const long long blocks = ((long long)rows * (inner / 8) + 255) / 256;
+  if (blocks > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_conv_silu: too many elements");
+  ConvSilu c{y, ldy, ring, weight, bias, start, positions64(pos), rows, seq, inner, taps, out};
+  with_types(dtype, dtype, [&](auto t, auto) {
+    hipLaunchKernelGGL(conv_silu_kernel<decltype(t)>, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, c);
+  });
+  return check_launch("ajqd_conv_silu");
+}
+
+int ajqd_scan(const ajqd_scan_args* a, int dtype, void* stream) {
+  if (!a || !a->x || !a->dt || !a->low || !a->z || !a->a2 || !a->d || !a->dt_bias || !a->out || (!a->state && (a->start > 0 || a->pos)))
+    return fail(AJQ_ERR_NULL, "ajqd_scan: null pointer argument");
+  if (a->batch < 1 || a->batch > 65535 || a->seq < 1 || a->inner < 8 || a->inner % 8 || a->states < 4 || a->states % 4 || a->start < 0 ||
+      a->dt_ld < a->inner || a->dt_ld % 8 || a->z_ld < a->inner || a->z_ld % 8 || a->out_ld < a->inner || a->out_ld % 8 || a->b_col < 0 ||
+      a->c_col < 0 || a->low_ld < a->b_col + a->states || a->low_ld < a->c_col + a->states || (a->pos && a->seq != 1))
+    return fail(AJQ_ERR_SHAPE, "ajqd_scan: unsupported shape (batch=%d seq=%d inner=%d states=%d)", a->batch, a->seq, a->inner, a->states);
+  if (!known(dtype)) return fail(AJQ_ERR_UNSUPPORTED, "ajqd_scan: unknown dtype %d", dtype);
+  if (!aligned16(a->x) || !aligned16(a->dt) || !aligned16(a->z) || !aligned16(a->out) || !aligned16(a->d) || !aligned16(a->dt_bias))
+    return fail(AJQ_ERR_ALIGN, "ajqd_scan: rows must be 16-byte aligned");
+  Scan s{a->x, a->dt, a->low, a->z, a->a2, a->d, a->dt_bias, a->state, a->start, positions64(a->pos), a->seq, a->inner, a->states,
+         a->dt_ld, a->low_ld, a->b_col, a->c_col, a->z_ld, a->out_ld, a->out};
+  return dtype == AJQD_BF16 ? launch_scan<uint16_t>(s, a->batch, (hipStream_t)stream) : launch_scan<float>(s, a->batch, (hipStream_t)stream);
+}
+
+int ajqd_scan_splits(int batch, int inner) {
+  (void)batch;
+  const int s = inner / 512;
+  return s < 1 ? 1 : s > 8 ? 8 : s;
+}
+
+int ajqd_scan_project(const float* y, int ldy, const void* ring, const float* weight, const float* bias, const int64_t* pos, const void* w,
+                      float* partial, int batch, int inner, int taps, int rows, int splits, void* stream) {
+  if (!y || !weight || !bias || !pos || !w || !partial || (!ring && taps > 1)) return fail(AJQ_ERR_NULL, "ajqd_scan_project: null pointer argument");
+  if (batch < 1 || inner < 8 || inner % 8 || taps < 1 || rows < 16 || rows % 16 || splits < 1 || splits > 65535 || ldy < 2 * inner || ldy % 4)
+    return fail(AJQ_ERR_SHAPE, "ajqd_scan_project: unsupported shape (batch=%d inner=%d taps=%d rows=%d splits=%d)", batch, inner, taps, rows, splits);
+  ScanProject p{y, (const uint16_t*)ring, weight, bias, positions64(pos), (const uint16_t*)w, partial, batch, ldy, inner, taps, rows, splits};
+  const int rt = batch > 4 && rows >= 32 ? 2 : 1;
+  const dim3 grid((rows / 16 + rt - 1) / rt, splits, (batch + kGemvBatch - 1) / kGemvBatch);
+  if (rt == 2) hipLaunchKernelGGL(scan_project_kernel<2>, grid, dim3(256), 0, (hipStream_t)stream, p);
+  else hipLaunchKernelGGL(scan_project_kernel<1>, grid, dim3(256), 0, (hipStream_t)stream, p);
+  return check_launch("ajqd_scan_project");
+}
+
+int ajqd_scan_step(const ajqd_scan_step_args* a, void* stream) {
+  if (!a || !a->y || !a->weight || !a->bias || !a->pos || !a->partial || !a->w_dt || !a->dt_bias || !a->a2 || !a->d || !a->state || !a->out ||
+      (!a->ring && a->taps > 1))
+    return fail(AJQ_ERR_NULL, "ajqd_scan_step: null pointer argument");
+  if (a->batch < 1 || a->inner < 16 || a->inner % 16 || a->taps < 1 || a->rank < 8 || a->rank % 8 || a->states < 4 || a->states % 4 ||
+      a->rows < a->rank + 2 * a->states || a->splits < 1 || a->ldy < 2 * a->inner || a->out_ld < a->inner)
+    return fail(AJQ_ERR_SHAPE, "ajqd_scan_step: unsupported shape (batch=%d inner=%d rank=%d states=%d rows=%d)", a->batch, a->inner, a->rank,
+                a->states, a->rows);
+  ScanStep s{a->y, (uint16_t*)a->ring, a->weight, a->bias, positions64(a->pos), a->partial, (const uint16_t*)a->w_dt, a->dt_bias, a->a2, a->d,
+             a->state, (uint16_t*)a->out, a->batch, a->ldy, a->inner, a->taps, a->rows, a->splits, a->rank, a->states, a->out_ld};
+  auto go = [&](auto kernel, int ct) {
+    const int bytes = scan_step_lds(a->rank, a->states, ct);
+    if (int e = allow_lds(kernel, bytes, "ajqd_scan_step")) return e;
+    hipLaunchKernelGGL(kernel, dim3((a->inner + 64 * ct - 1) / (64 * ct), (a->batch + kScanBatch - 1) / kScanBatch), dim3(256), bytes,
+                       (hipStream_t)stream, s);
+    return check_launch("ajqd_scan_step");
+  };
+  return a->batch > kScanBatch ? go(scan_step_kernel<4>, 4) : go(scan_step_kernel<1>, 1);
 }
 
 }  // extern "C"

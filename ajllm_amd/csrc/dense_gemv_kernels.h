@@ -3,12 +3,14 @@
 //
 //   dense_in_kernel      two weight matrices that read the same fp32 residual row through norms of their own: the layer
 //                        norm is the prologue (or bf16 rows a norm launch left); the first matrix's outputs are stored
-//                        in fp32, the second's are gated pairs (8 gate rows and their 8 up rows per 16-row tile)
+//                        in fp32, the second's go through an activation: gated pairs (8 gate rows and their 8 up rows per
+//                        16-row tile), or every row by itself
 //   latent_absorb_kernel per-head products of the unrotated query with the transposed key expansion, so that attention
 //                        can run on the latents; beside them the rotation of the query, and the new cache row (RMS norm of
 //                        the latent, rotation of the shared key part)
 //   latent_expand_kernel merge of the attention's row chunks (with the sink), per-head value expansion, output gate
 //   dense_out_kernel     product with the residual add (and whatever the next layer run adds first) as epilogue
+//   dense_out_streams_kernel  product whose epilogue mixes it into several residual streams and forms what the next sublayer reads
 //
 // A 16 x 16 output tile (16 weight rows, 16 batch columns) belongs to a wave, or to kWaves waves that split K and meet in
 // LDS.  Lane l = 16 g + r loads 16 bytes of weight row r at k = 32 step + 8 g: four lanes cover 64 contiguous bytes of a
@@ -16,6 +18,7 @@
 #pragma once
 #include "dense_kernels.h"
 #include "latent_attention.h"
+#include "stream_kernels.h"
 
 namespace ajq {
 
@@ -96,10 +99,10 @@ struct DenseIn {
   const float* gain1;
   const float* gain2;
   const uint16_t* w1;       // [16 tiles1, Dp]
-  const uint16_t* w2;       // [16 tiles2, Dp], gate / up rows interleaved in blocks of 8
+  const uint16_t* w2;       // [16 tiles2, Dp]; pairs: gate / up rows interleaved in blocks of 8
   float* y1;                // [B, 16 tiles1]
-  uint16_t* gated;          // [B, gated_ld], column 8 * tile + j
-  int batch, D, Dp, tiles1, tiles2, gated_ld, act, center;
+  uint16_t* gated;          // [B, gated_ld], column 8 * tile + j (pairs) or 16 * tile + j
+  int batch, D, Dp, tiles1, tiles2, gated_ld, act, center, pairs;
   float eps;
 };
 
@@ -199,6 +202,12 @@ __global__ __launch_bounds__(64 * kWaves) void dense_in_kernel(DenseIn a) {
       if (row < nb) store4(a.y1 + (size_t)(b0 + row) * (16 * a.tiles1) + 16 * tile + 4 * g, float4{sum[0], sum[1], sum[2], sum[3]});
       continue;
     }
+    if (!a.pairs) {
+      if (row < nb)
+        store4(a.gated + (size_t)(b0 + row) * a.gated_ld + 16 * tile + 4 * g,
+               float4{activate(a.act, sum[0]), activate(a.act, sum[1]), activate(a.act, sum[2]), activate(a.act, sum[3])});
+      continue;
+    }
     // rows 0 .. 7 of the tile (lanes g < 2) are gates, rows 8 .. 15 (lanes g >= 2, 32 lanes on) the matching up rows
     float v[4];
 #pragma unroll
@@ -254,6 +263,59 @@ __global__ __launch_bounds__(64 * kWaves) void dense_out_kernel(DenseOut a) {
     const float4 v = old[kWaves > 1 ? 0 : i];
     const f32x4_t& sum = acc[i / BT][i % BT];
     store4(a.x + place(i), float4{v.x + sum[0], v.y + sum[1], v.z + sum[2], v.w + sum[3]});
+  }
+}
+
+struct DenseOutStreams {
+  const uint16_t* in;       // [B, K]
+  const uint16_t* w;        // [Dp, K]
+  float* x;                 // [B, S, Dp], updated in place
+  const float* scale;       // [Dp], a factor per column of the product
+  const float* out;         // [S]
+  const float* mix;         // [S, S]
+  const float* next;        // [S], weights of the next reader; null: the plain sum
+  float* u;                 // [B, Dp], what the next reader gets
+  int batch, K, Dp, streams;
+};
+template <int kWaves, int RT, int BT, int MAXS>
+__global__ __launch_bounds__(64 * kWaves) void dense_out_streams_kernel(DenseOutStreams a) {
+  __shared__ __attribute__((aligned(16))) float red[kWaves > 1 ? RT * BT * kWaves * 256 : 4];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const int b0 = blockIdx.y * kGemvBatch * BT, nb = min(kGemvBatch * BT, a.batch - b0);
+  const int first = blockIdx.x * RT * 16;
+  const uint16_t* wrow = a.w + (size_t)(first + r) * a.K;
+  const uint16_t* xr = a.in + (size_t)b0 * a.K + 8 * g;
+  int begin, end;
+  wave_steps(a.K, wave, kWaves, begin, end);
+  // the streams at this lane's place of tile i = (row tile, batch tile); with several waves each writes one tile and
+  // requests its streams ahead of the product
+  auto fetch = [&](int i, float4 (&v)[MAXS]) {
+    const float* x = a.x + (size_t)(b0 + min(16 * (i % BT) + r, nb - 1)) * a.streams * a.Dp + first + 16 * (i / BT) + 4 * g;
+#pragma unroll
+    for (int s = 0; s < MAXS; ++s)
+      if (s < a.streams) v[s] = load4(x + (size_t)s * a.Dp);
+  };
+  float4 v[MAXS];
+  if (kWaves > 1 && wave < RT * BT) fetch(wave, v);
+  f32x4_t acc[RT][BT] = {};
+  tile_steps<RT, BT>(wrow, a.K, begin, end, g, acc, [&](int t, int s) {
+    const int row = 16 * t + r;
+    return row < nb ? *reinterpret_cast<const u32x4_t*>(xr + (size_t)row * a.K + 32 * s) : u32x4_t{0u, 0u, 0u, 0u};
+  });
+  meet<kWaves, RT, BT>(acc, red, wave, lane);
+#pragma unroll
+  for (int i = 0; i < RT * BT; ++i) {
+    const int row = 16 * (i % BT) + r, column = first + 16 * (i / BT) + 4 * g;
+    if ((kWaves > 1 && wave != i) || row >= nb) continue;
+    if (kWaves == 1) fetch(i, v);
+    const f32x4_t& sum = acc[i / BT][i % BT];
+    const float4 f = load4(a.scale + column);
+    mix_streams<MAXS>(v, a.streams, a.out, a.mix, float4{sum[0] * f.x, sum[1] * f.y, sum[2] * f.z, sum[3] * f.w});
+    float* x = a.x + (size_t)(b0 + row) * a.streams * a.Dp + column;
+#pragma unroll
+    for (int s = 0; s < MAXS; ++s)
+      if (s < a.streams) store4(x + (size_t)s * a.Dp, v[s]);
+    store4(a.u + (size_t)(b0 + row) * a.Dp + column, read_streams<MAXS>(v, a.streams, a.next));
   }
 }
 
@@ -337,6 +399,7 @@ struct LatentDecode {
   float* sums;
   float2* heads_out;        // [B, H, S]
   int batch, heads, rankp, width, cap, chunks;
+  int key_step;             // 32-column steps ahead of it meet zero query columns and are left out of the scores
   float scale2;
 };
 __host__ __device__ constexpr long long latent_sums_at(int b, int tile, int chunk, int heads, int chunks, int rankp) {
@@ -410,7 +473,8 @@ __global__ __launch_bounds__(256 * HT) void latent_decode_kernel(LatentDecode a)
       const uint32_t stage = (uint32_t)((((j0 - begin) / kLatentRows) & 1) * kStage);
       f32x4_t sc[2] = {};
 #pragma unroll
-      for (int s = 0; s < KS; ++s) sc[s & 1] = mfma16(pf_read128(k_rd[s & 1] + stage + (uint32_t)((s >> 1) * kPanel)), qf[s], sc[s & 1]);
+      for (int s = 0; s < KS; ++s)
+        if (s >= a.key_step) sc[s & 1] = mfma16(pf_read128(k_rd[s & 1] + stage + (uint32_t)((s >> 1) * kPanel)), qf[s], sc[s & 1]);
       // score i: key j0 + 16 part + 4 g + i, head h0 + r
       float p[4], mx = -INFINITY;
 #pragma unroll

@@ -31,6 +31,32 @@ __device__ __forceinline__ void store4(uint16_t* p, float4 v) {
   *reinterpret_cast<u32x2_t*>(p) = u32x2_t{pack2_bf16(v.x, v.y), pack2_bf16(v.z, v.w)};
 }
 
+struct Float8 {
+  float v[8];
+};
+__device__ __forceinline__ Float8 load8(const float* p) {
+  const float4 a = load4(p), b = load4(p + 4);
+  return Float8{{a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w}};
+}
+__device__ __forceinline__ Float8 load8(const uint16_t* p) {
+  const u32x4_t q = *reinterpret_cast<const u32x4_t*>(p);
+  Float8 f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    f.v[2 * i] = __uint_as_float(q[i] << 16);
+    f.v[2 * i + 1] = __uint_as_float(q[i] & 0xFFFF0000u);
+  }
+  return f;
+}
+__device__ __forceinline__ void store8(float* p, const Float8& f) {
+  store4(p, float4{f.v[0], f.v[1], f.v[2], f.v[3]});
+  store4(p + 4, float4{f.v[4], f.v[5], f.v[6], f.v[7]});
+}
+__device__ __forceinline__ void store8(uint16_t* p, const Float8& f) {
+  *reinterpret_cast<u32x4_t*>(p) = u32x4_t{pack2_bf16(f.v[0], f.v[1]), pack2_bf16(f.v[2], f.v[3]), pack2_bf16(f.v[4], f.v[5]),
+                                           pack2_bf16(f.v[6], f.v[7])};
+}
+
 __device__ __forceinline__ float wave_sum64(float v) {
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off);
@@ -254,25 +280,33 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const Y* __restrict__
   for (int h = tid; h < s.heads; h += 256) gates[(size_t)m * s.heads + h] = sigmoid_f32(to_f32(lat[s.rankp + s.rotp + h]));
 }
 
-// Rows of a ring cache [B, cap, width] (slot = position % cap) from / to rows first_row .. of a linear buffer
-// [B, lines, width], starting at position `position`.  One thread per 16 bytes; chunks = bytes of a row / 16.
-__global__ __launch_bounds__(256) void ring_copy_kernel(u32x4_t* __restrict__ ring, int cap, u32x4_t* __restrict__ linear,
-                                                        int lines, int first_row, int position, int count, int chunks, int batch,
-                                                        int to_ring) {
+// Slot of a position in a ring of cap rows whose first `kept` positions stay where they are.
+__host__ __device__ __forceinline__ int ring_slot(int position, int cap, int kept) {
+  return position < kept ? position : kept + (position - kept) % (cap - kept);
+}
+// Rows of a ring cache [B, cap, width] from / to rows first_row .. of a linear buffer [B, lines, line], starting at position
+// `position`.  One thread per 16 bytes; chunks = bytes of a row / 16, line likewise.
+__global__ __launch_bounds__(256) void ring_copy_kernel(u32x4_t* __restrict__ ring, int cap, int kept, u32x4_t* __restrict__ linear,
+                                                        int lines, int line, int first_row, int position, int count, int chunks,
+                                                        int batch, int to_ring) {
   const long long idx = (long long)blockIdx.x * 256 + threadIdx.x;
   if (idx >= (long long)batch * count * chunks) return;
   const int c = (int)(idx % chunks);
   const int i = (int)((idx / chunks) % count);
   const int b = (int)(idx / ((long long)chunks * count));
-  u32x4_t* r = ring + ((size_t)b * cap + (position + i) % cap) * chunks + c;
-  u32x4_t* l = linear + ((size_t)b * lines + first_row + i) * chunks + c;
+  u32x4_t* r = ring + ((size_t)b * cap + ring_slot(position + i, cap, kept)) * chunks + c;
+  u32x4_t* l = linear + ((size_t)b * lines + first_row + i) * line + c;
   if (to_ring) *r = *l; else *l = *r;
 }
 
-enum Activation { kActRelu = 0, kActSilu = 1, kActGeluTanh = 2 };
+enum Activation { kActRelu = 0, kActSilu = 1, kActGeluTanh = 2, kActSquaredRelu = 3 };
 __device__ __forceinline__ float activate(int kind, float z) {
   if (kind == kActRelu) return fmaxf(z, 0.f);
   if (kind == kActSilu) return z * sigmoid_f32(z);
+  if (kind == kActSquaredRelu) {
+    const float r = fmaxf(z, 0.f);
+    return r * r;
+  }
   const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);  // sqrt(2 / pi)
   return 0.5f * z * (1.0f + tanhf(u));
 }
@@ -289,6 +323,17 @@ __global__ __launch_bounds__(256) void gated_activation_kernel(const Y* __restri
   const float4 a = load4(src), u = load4(src + 8);
   store4(out + (size_t)m * ldo + f, float4{activate(kind, a.x) * u.x, activate(kind, a.y) * u.y, activate(kind, a.z) * u.z,
                                            activate(kind, a.w) * u.w});
+}
+
+// out = act(y) over dense rows of eight-column multiples: one thread per 8 values.
+template <typename T>
+__global__ __launch_bounds__(256) void activation_kernel(const T* __restrict__ y, T* __restrict__ out, long long eighths, int kind) {
+  const long long idx = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= eighths) return;
+  Float8 v = load8(y + 8 * idx);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v.v[e] = activate(kind, v.v[e]);
+  store8(out + 8 * idx, v);
 }
 
 // Plain product for any type: y[b, g, n] = sum_k w[g, n, k] x[b, g, k], fp32 sums, one wave per output.

@@ -1,8 +1,10 @@
-// Attention over keys that are made of a per-head part and a part all heads share, with a sliding window, an
-// attention sink and a per-head output gate:
+// Attention over keys that are made of a per-head part and (optionally) a part all heads share, with a sliding window, first
+// rows that stay visible, an attention sink and an output gate (a factor per head, or a sigmoid per column):
 //
 //   s_j     = (qu . ku_j + qr . kr_j) * scale            over the visible rows j
 //   out     = gate * sum_j exp(s_j) v_j / (exp(sink) + sum_j exp(s_j))
+//
+// Heads may share key / value heads in groups of `share`.
 //
 // Three kernels:
 //   windowed_attention_kernel   any sizes, bf16 or fp32, one wave per (token, head): fp32 prompts and decoding
@@ -27,11 +29,16 @@ struct WindowedAttention {
   const long long* pos;     // device-side position: the first min(*pos + 1, rows) rows are visible (a ring of cap rows)
   void* out;                // [B * T, out_ld], head h at column h * dv
   long long k1_batch, k2_batch, v_batch;
-  int k1_row, k1_head, k2_row, v_row, v_head;
-  int d1, d2, dv;           // multiples of 8
+  long long k1_head, v_head;
+  int k1_row, k2_row, v_row;
+  int d1, d2, dv;           // multiples of 8; d2 may be 0
   int batch, heads, seq;    // T new tokens per sequence
   int rows, prior;          // rows a buffer holds per sequence; query t sits at row prior + t
   int window;               // <= 0: none
+  int keep;                 // rows 0 .. keep - 1 are visible whatever the window
+  int share;                // heads per key / value head
+  int gate_ld;
+  const void* column_gates; // [B * T, gate_ld], head h at column h * dv: the output's sigmoid gate before the sigmoid, or null
   int out_ld;
   float scale;
 };
@@ -58,16 +65,18 @@ __global__ __launch_bounds__(64) void windowed_attention_kernel(WindowedAttentio
     hi = a.prior + t;
     if (a.window > 0) lo = max(0, hi - a.window + 1);
   }
-  const T* k1 = reinterpret_cast<const T*>(a.k1) + (size_t)b * a.k1_batch + (size_t)h * a.k1_head;
+  const int kept = min(a.keep, lo), n_rows = kept + hi - lo + 1;  // rows 0 .. kept - 1, then lo .. hi
+  auto row_of = [&](int j) { return j < kept ? j : lo + j - kept; };
+  const T* k1 = reinterpret_cast<const T*>(a.k1) + (size_t)b * a.k1_batch + (size_t)(h / a.share) * a.k1_head;
   const T* k2 = reinterpret_cast<const T*>(a.k2) + (size_t)b * a.k2_batch;
-  const T* v = reinterpret_cast<const T*>(a.v) + (size_t)b * a.v_batch + (size_t)h * a.v_head;
+  const T* v = reinterpret_cast<const T*>(a.v) + (size_t)b * a.v_batch + (size_t)(h / a.share) * a.v_head;
   const float scale2 = a.scale * kLog2eF;
   float mx = a.sink ? a.sink[h] * kLog2eF : -INFINITY, total = a.sink ? 1.f : 0.f;
   __syncthreads();
-  for (int j0 = lo; j0 <= hi; j0 += 64) {
-    const int j = j0 + lane;
+  for (int j0 = 0; j0 < n_rows; j0 += 64) {
+    const int j = row_of(j0 + lane);
     float s = -INFINITY;
-    if (j <= hi) {
+    if (j0 + lane < n_rows) {
       float d = 0.f;
       const T* kr = k1 + (size_t)j * a.k1_row;
       for (int i = 0; i < a.d1; i += 4) {
@@ -89,17 +98,18 @@ __global__ __launch_bounds__(64) void windowed_attention_kernel(WindowedAttentio
     mx = m_new;
     weight[lane] = w;
     __syncthreads();
-    const int n = min(64, hi - j0 + 1);
+    const int n = min(64, n_rows - j0);
     for (int i = lane; i < a.dv; i += 64) {
       float o = acc[i] * corr;
-      for (int jj = 0; jj < n; ++jj) o = fmaf(weight[jj], to_f32(v[(size_t)(j0 + jj) * a.v_row + i]), o);
+      for (int jj = 0; jj < n; ++jj) o = fmaf(weight[jj], to_f32(v[(size_t)row_of(j0 + jj) * a.v_row + i]), o);
       acc[i] = o;
     }
     __syncthreads();
   }
   const float factor = a.gates ? a.gates[(size_t)m * a.heads + h] : 1.f;
   O* out = reinterpret_cast<O*>(a.out) + (size_t)m * a.out_ld + (size_t)h * a.dv;
-  for (int i = lane; i < a.dv; i += 64) out[i] = from_f32<O>(acc[i] / total * factor);
+  const T* gate = a.column_gates ? reinterpret_cast<const T*>(a.column_gates) + (size_t)m * a.gate_ld + (size_t)h * a.dv : nullptr;
+  for (int i = lane; i < a.dv; i += 64) out[i] = from_f32<O>(acc[i] / total * factor * (gate ? sigmoid_f32(to_f32(gate[i])) : 1.f));
 }
 
 // global -> LDS without registers (16 bytes per lane, a wave's 1 KiB contiguous in LDS), every lane with an address of
@@ -119,7 +129,8 @@ __device__ __forceinline__ void dma16_gather(const void* src, uint32_t lds_addr)
 //   * a workgroup of 4 waves on 64 U query rows of one (b, h), a wave U groups of 16;
 //   * keys of KS 32-column steps gathered from two places (the head's own columns, then the shared ones; columns past
 //     both meet zero query columns) and values of VT 16-column tiles, one block of 64 rows ahead by DMA;
-//   * blocks from the first key the workgroup's first query sees to its last query's own;
+//   * blocks of the first rows that stay visible, then from the first key in the window of the workgroup's first query to
+//     its last query's own;
 //   * the sink as the initial state of the running softmax: reference exponent sink, denominator 1.  Every row then
 //     has a finite reference from the start, also when a whole block lies outside its window.
 // LDS holds key and value rows in panels of 128 bytes (64 rows x 8 chunks of 16 bytes = 8 KiB, keys first):
@@ -153,13 +164,19 @@ __global__ __launch_bounds__(256, prefill_panels(KS, VT) > 5 ? 1 : 2) void windo
   const int total = a.prior + a.seq;
   const int first_q = a.prior + q0, last_q = min(total, first_q + kBQ) - 1;  // rows of the workgroup's first / last query
   const int window = a.window > 0 ? a.window : 0x3FFFFFFF;
-  const int lo = max(0, first_q - window + 1) & ~(kPfBK - 1);
-  const int nblk = (last_q - lo) / kPfBK + 1;
+  int kept_blocks = (a.keep + kPfBK - 1) / kPfBK;
+  int lo = max(0, first_q - window + 1) & ~(kPfBK - 1);
+  if (lo <= kept_blocks * kPfBK) {  // one run of blocks
+    lo = kept_blocks > 0 ? 0 : lo;
+    kept_blocks = 0;
+  }
+  const int nblk = kept_blocks + (last_q - lo) / kPfBK + 1;
+  auto block_row = [&](int j) { return j < kept_blocks ? j * kPfBK : lo + (j - kept_blocks) * kPfBK; };
   const int wave_first = first_q + 16 * U * wave, wave_last = wave_first + 16 * U - 1;
 
-  const uint16_t* k1 = reinterpret_cast<const uint16_t*>(a.k1) + (size_t)b * a.k1_batch + (size_t)h * a.k1_head;
+  const uint16_t* k1 = reinterpret_cast<const uint16_t*>(a.k1) + (size_t)b * a.k1_batch + (size_t)(h / a.share) * a.k1_head;
   const uint16_t* k2 = reinterpret_cast<const uint16_t*>(a.k2) + (size_t)b * a.k2_batch;
-  const uint16_t* vv = reinterpret_cast<const uint16_t*>(a.v) + (size_t)b * a.v_batch + (size_t)h * a.v_head;
+  const uint16_t* vv = reinterpret_cast<const uint16_t*>(a.v) + (size_t)b * a.v_batch + (size_t)(h / a.share) * a.v_head;
   const int c1 = a.d1 >> 3, c2 = c1 + (a.d2 >> 3), cv = a.dv >> 3;
 
   // ---- what this lane fetches: row 8 q + lane / 8 of a request, slot lane % 8 of its panel.  Chunks past the widths
@@ -184,7 +201,7 @@ __global__ __launch_bounds__(256, prefill_panels(KS, VT) > 5 ? 1 : 2) void windo
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
       // rows past the end repeat the last one; those keys are masked
-      const uint32_t row = (uint32_t)min(lo + j * kPfBK + 32 * half + req_row, total - 1);
+      const uint32_t row = (uint32_t)min(block_row(j) + 32 * half + req_row, total - 1);
 #pragma unroll
       for (int p = 0; p < KP; ++p) dma16_gather(kbase[p] + (size_t)row * kstride[p], to + (uint32_t)(p * kPanel + half * 4096));
 #pragma unroll
@@ -229,10 +246,10 @@ __global__ __launch_bounds__(256, prefill_panels(KS, VT) > 5 ? 1 : 2) void windo
   __syncthreads();
   for (int j = 0; j < nblk; ++j) {
     // block j is complete in stage j & 1; block j + 1 goes into the other stage, last read before the previous barrier
-    const int kb0 = lo + j * kPfBK;
+    const int kb0 = block_row(j);
     if (j + 1 < nblk) fetch(j + 1);
     const uint32_t stage = (uint32_t)((j & 1) * kStage);
-    if (kb0 <= wave_last && kb0 + kPfBK - 1 > wave_first - window) {
+    if (kb0 <= wave_last && (kb0 + kPfBK - 1 > wave_first - window || kb0 < a.keep)) {
       f32x4_t sc[U][4];
 #pragma unroll
       for (int s = 0; s < KS; ++s) {
@@ -254,7 +271,7 @@ __global__ __launch_bounds__(256, prefill_panels(KS, VT) > 5 ? 1 : 2) void windo
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
               const int key = kb0 + 16 * jb + 4 * g + i;
-              if (key > qrow[u] || key <= qrow[u] - window) sc[u][jb][i] = -INFINITY;
+              if (key > qrow[u] || (key <= qrow[u] - window && key >= a.keep)) sc[u][jb][i] = -INFINITY;
             }
       }
       u32x4_t pf[U][2];
@@ -320,11 +337,17 @@ __global__ __launch_bounds__(256, prefill_panels(KS, VT) > 5 ? 1 : 2) void windo
     const size_t m = (size_t)b * a.seq + t0;
     const float factor = (a.gates ? a.gates[m * a.heads + h] : 1.f) / l;
     uint16_t* dst = reinterpret_cast<uint16_t*>(a.out) + m * a.out_ld + (size_t)h * a.dv + 4 * g;
+    const uint16_t* gate = a.column_gates ? reinterpret_cast<const uint16_t*>(a.column_gates) + m * a.gate_ld + (size_t)h * a.dv + 4 * g : nullptr;
 #pragma unroll
     for (int t = 0; t < VT; ++t)
-      if (16 * t < a.dv)
-        *reinterpret_cast<u32x2_t*>(dst + 16 * t) =
-            u32x2_t{pack2_bf16(o[u][t][0] * factor, o[u][t][1] * factor), pack2_bf16(o[u][t][2] * factor, o[u][t][3] * factor)};
+      if (16 * t < a.dv) {
+        float4 v = float4{o[u][t][0] * factor, o[u][t][1] * factor, o[u][t][2] * factor, o[u][t][3] * factor};
+        if (gate) {
+          const float4 z = load4(gate + 16 * t);
+          v.x *= sigmoid_f32(z.x); v.y *= sigmoid_f32(z.y); v.z *= sigmoid_f32(z.z); v.w *= sigmoid_f32(z.w);
+        }
+        store4(dst + 16 * t, v);
+      }
   }
 }
 

@@ -1,0 +1,357 @@
+// Selective scan (a diagonal linear recurrence per channel whose decay, input and output weights depend on the token):
+//
+//   x   = silu(conv(x))                               causal, per channel, `taps` wide
+//   S  <- exp(dt A) S + (dt x) B,   y = S C + D x     S [channels, states] fp32, dt = softplus(raw + bias) per channel
+//   out = y silu(z)
+//
+// Prompts (any number of tokens, from any position; also one token on any operand type):
+//   conv_silu_kernel, scan_kernel
+// One token in bf16:
+//   scan_project_kernel, scan_step_kernel
+//
+// States and a2 = A log2(e) (decays are taken in base 2) are stored in planes of four: [states / 4][channels][4], so that threads
+// of neighbouring channels load whole lines; `states` is a multiple of 4 (states past a model's own are zero).
+//
+// Whatever the operand type: convolution sums, dt and its softplus, decays, states and y are fp32.  A
+// sequence's first token (position 0) starts from zeros whatever the buffers hold.
+#pragma once
+#include "dense_gemv_kernels.h"
+
+namespace ajq {
+
+__device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
+__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+
+struct ConvSilu {
+  const void* y;            // [B * seq, ldy], the convolved columns first
+  int ldy;
+  void* ring;               // [B, taps - 1, inner]: position p in slot p % (taps - 1); null: the sequence starts here
+  const float* weight;      // [taps, inner], the last row meets the token itself
+  const float* bias;        // [inner]
+  int start;
+  const long long* pos;     // device-side position (seq = 1): the token's own column goes into the ring as well
+  int rows, seq, inner, taps;
+  void* out;                // [B * seq, inner]
+};
+// A thread makes 8 channels of one token.
+template <typename T>
+__global__ __launch_bounds__(256) void conv_silu_kernel(ConvSilu a) {
+  const int vectors = a.inner >> 3;
+  const long long idx = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= (long long)a.rows * vectors) return;
+  const int m = (int)(idx / vectors), c = 8 * (int)(idx % vectors), b = m / a.seq, t = m % a.seq, reach = a.taps - 1;
+  const int p = clamped_position(a.pos, a.start + t, 0x7FFFFFFF);
+  const T* y = reinterpret_cast<const T*>(a.y) + (size_t)m * a.ldy + c;
+  T* ring = reinterpret_cast<T*>(a.ring) + (size_t)b * reach * a.inner + c;
+  Float8 sum = load8(a.bias + c);
+  const Float8 own = load8(y);
+  for (int j = min(reach, p); j >= 0; --j) {
+    const Float8 w = load8(a.weight + (size_t)(reach - j) * a.inner + c);
+    Float8 v = own;
+    if (j > t) v = load8(ring + (size_t)((p - j) % reach) * a.inner);
+    else if (j > 0) v = load8(y - (size_t)j * a.ldy);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sum.v[e] = fmaf(w.v[e], v.v[e], sum.v[e]);
+  }
+  if (a.pos && reach > 0) store8(ring + (size_t)(p % reach) * a.inner, own);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) sum.v[e] = silu_f32(sum.v[e]);
+  store8(reinterpret_cast<T*>(a.out) + (size_t)m * a.inner + c, sum);
+}
+
+template <int kCtrl>
+__device__ __forceinline__ float dpp_add(float v) {
+  return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), kCtrl, 0xF, 0xF, true));
+}
+// sum over L neighbouring lanes (L a power of two), in every one of them
+template <int L>
+__device__ __forceinline__ float team_sum(float v) {
+  if (L > 1) v = dpp_add<0xB1>(v);    // quad_perm [1, 0, 3, 2]
+  if (L > 2) v = dpp_add<0x4E>(v);    // quad_perm [2, 3, 0, 1]
+  if (L > 4) v = dpp_add<0x141>(v);   // row_half_mirror: quads are uniform by now
+  if (L > 8) v = dpp_add<0x140>(v);   // row_mirror
+  if (L > 16) v += __shfl_xor(v, 16);
+  if (L > 32) v += __shfl_xor(v, 32);
+  return v;
+}
+
+struct Scan {
+  const void* x;            // [B * seq, inner] behind the convolution
+  const void* dt;           // [B * seq, dt_ld] raw
+  const void* low;          // [B * seq, low_ld]: B at column b_col, C at c_col, `states` each
+  const void* z;            // [B * seq, z_ld]
+  const float *a2, *d, *dt_bias;  // [states / 4, inner, 4], [inner], [inner]
+  float* state;             // [B, states / 4, inner, 4] or null
+  int start;
+  const long long* pos;
+  int seq, inner, states, dt_ld, low_ld, b_col, c_col, z_ld, out_ld;
+  void* out;                // [B * seq, out_ld]
+};
+// L lanes share a channel, NS states each (states <= L NS; the ones past the end stay zero), so that a small model or batch
+// still fills the chip: the time loop is sequential, and its length is what a wave costs.  256 / L channels per workgroup.
+// A tile of kT tokens is staged in LDS: dt and dt x (the softplus is taken once per channel and token there), B and C; y takes
+// dt x's place.  The next tile's operands are requested ahead of the current one's time loop.
+template <int L, int NS>
+constexpr int scan_tile() {
+  int t = 8 * L;
+  while (t * L * NS > 4096) t /= 2;
+  return t;
+}
+template <typename T, int L, int NS>
+__global__ __launch_bounds__(256) void scan_kernel(Scan a) {
+  constexpr int CH = 256 / L, kT = scan_tile<L, NS>(), kN = L * NS, kVec = kT * CH / 8, kPitch = CH + 4, kTogether = 4;
+  static_assert(kT % kTogether == 0, "whole groups of tokens");
+  static_assert(kVec >= 1 && kVec <= 256, "at most one vector of 8 channels per thread");
+  __shared__ __attribute__((aligned(16))) float dt_s[kT * kPitch], dx_s[kT * kPitch], b_s[kT * kN], c_s[kT * kN];
+  const int tid = threadIdx.x, ch = tid / L, part = tid % L;
+  const int b = blockIdx.y, c0 = blockIdx.x * CH, c = c0 + ch;
+  const bool mine = c < a.inner;
+  float s[NS], a2[NS];
+  const bool carried = a.state && (a.start > 0 || (a.pos && *a.pos > 0));
+  float* state = a.state + (size_t)b * a.inner * a.states;
+  auto place = [&](int n) { return ((size_t)(n >> 2) * a.inner + c) * 4 + (n & 3); };
+#pragma unroll
+  for (int i = 0; i < NS; ++i) {
+    const int n = part * NS + i;
+    const bool real = mine && n < a.states;
+    a2[i] = real ? a.a2[place(n)] : 0.f;
+    s[i] = real && carried ? state[place(n)] : 0.f;
+  }
+  // this thread's vector of a tile: token vt, channels vc ..
+  const int vt = tid / (CH / 8), vl = 8 * (tid % (CH / 8)), vc = c0 + vl;
+  const bool stages = tid < kVec && vc < a.inner;
+  const T* xp = reinterpret_cast<const T*>(a.x) + (size_t)b * a.seq * a.inner + vc;
+  const T* dp = reinterpret_cast<const T*>(a.dt) + (size_t)b * a.seq * a.dt_ld + vc;
+  const T* zp = reinterpret_cast<const T*>(a.z) + (size_t)b * a.seq * a.z_ld + vc;
+  const T* lp = reinterpret_cast<const T*>(a.low) + (size_t)b * a.seq * a.low_ld;
+  T* op = reinterpret_cast<T*>(a.out) + (size_t)b * a.seq * a.out_ld + vc;
+  constexpr int kLow = (kT * kN + 255) / 256;
+  Float8 nx, nd, nz, bias, skip;
+  float nb[kLow], nc[kLow];
+  if (stages) {
+    bias = load8(a.dt_bias + vc);
+    skip = load8(a.d + vc);
+  }
+  auto request = [&](int t0) {
+    const int t = t0 + vt;
+    if (stages && t < a.seq) {
+      nx = load8(xp + (size_t)t * a.inner);
+      nd = load8(dp + (size_t)t * a.dt_ld);
+      nz = load8(zp + (size_t)t * a.z_ld);
+    }
+#pragma unroll
+    for (int k = 0; k < kLow; ++k) {
+      const int i = tid + 256 * k, u = t0 + i / kN, n = i % kN;
+      nb[k] = nc[k] = 0.f;
+      if (i < kT * kN && u < a.seq && n < a.states) {
+        nb[k] = to_f32(lp[(size_t)u * a.low_ld + a.b_col + n]);
+        nc[k] = to_f32(lp[(size_t)u * a.low_ld + a.c_col + n]);
+      }
+    }
+  };
+  request(0);
+  for (int t0 = 0; t0 < a.seq; t0 += kT) {
+    const int count = min(kT, a.seq - t0);
+    const Float8 x = nx, z = nz;
+    if (tid < kVec) {
+      float* dts = dt_s + vt * kPitch + vl;
+      float* dxs = dx_s + vt * kPitch + vl;
+      Float8 d, dx;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        d.v[e] = stages && vt < count ? softplus_f32(nd.v[e] + bias.v[e]) : 0.f;
+        dx.v[e] = stages && vt < count ? d.v[e] * x.v[e] : 0.f;
+      }
+      store8(dts, d);
+      store8(dxs, dx);
+    }
+#pragma unroll
+    for (int k = 0; k < kLow; ++k) {
+      const int i = tid + 256 * k;
+      if (i < kT * kN) {
+        b_s[i] = nb[k];
+        c_s[i] = nc[k];
+      }
+    }
+    __syncthreads();
+    if (t0 + kT < a.seq) request(t0 + kT);
+    for (int u = 0; u < count; u += kTogether) {  // (tokens past the end: dt = 0 leaves the states alone)
+      float y[kTogether];
+#pragma unroll
+      for (int k = 0; k < kTogether; ++k) {
+        const int t = u + k;
+        const float dt = dt_s[t * kPitch + ch], dx = dx_s[t * kPitch + ch];
+        const float* bt = b_s + t * kN + part * NS;
+        const float* ct = c_s + t * kN + part * NS;
+        y[k] = 0.f;
+#pragma unroll
+        for (int i = 0; i < NS; ++i) {
+          s[i] = fmaf(__builtin_amdgcn_exp2f(dt * a2[i]), s[i], dx * bt[i]);
+          y[k] = fmaf(s[i], ct[i], y[k]);
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < kTogether; ++k) y[k] = team_sum<L>(y[k]);
+      if (part == 0)
+#pragma unroll
+        for (int k = 0; k < kTogether; ++k) dx_s[(u + k) * kPitch + ch] = y[k];
+    }
+    __syncthreads();
+    if (stages && vt < count) {
+      const float* ys = dx_s + vt * kPitch + vl;
+      Float8 o;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o.v[e] = fmaf(skip.v[e], x.v[e], ys[e]) * silu_f32(z.v[e]);
+      store8(op + (size_t)(t0 + vt) * a.out_ld, o);
+    }
+    __syncthreads();
+  }
+  if (a.state && mine)
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+      if (part * NS + i < a.states) state[place(part * NS + i)] = s[i];
+}
+
+// ---- one token per sequence, bf16
+// The projection of the convolved columns to (dt rank | B | C): `rows` weight rows (a multiple of 16), K = inner cut into
+// `splits` parts whose sums scan_step_kernel adds.  A lane convolves the eight channels of its own operand fragment, so the
+// convolved row exists in registers only; every group of RT row tiles repeats that.  Grid (row groups, splits, batch blocks).
+struct ScanProject {
+  const float* y;           // [B, ldy]: convolved columns, then z
+  const uint16_t* ring;     // [B, taps - 1, inner]
+  const float* weight;      // [taps, inner]
+  const float* bias;
+  const long long* pos;
+  const uint16_t* w;        // [rows, inner]
+  float* partial;           // [splits, B, rows]
+  int batch, ldy, inner, taps, rows, splits;
+};
+template <int RT>
+__global__ __launch_bounds__(256) void scan_project_kernel(ScanProject a) {
+  __shared__ __attribute__((aligned(16))) float red[RT * 4 * 256];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const int b0 = blockIdx.z * kGemvBatch, nb = min(kGemvBatch, a.batch - b0);
+  const int tile0 = max(0, min(RT * (int)blockIdx.x, a.rows / 16 - RT));  // (the last group may repeat its neighbour's rows)
+  const int reach = a.taps - 1, p = clamped_position(a.pos, 0, 0x7FFFFFFF);
+  const int steps = (a.inner + 31) >> 5, per = (steps + a.splits - 1) / a.splits;
+  const int lo = min(steps, (int)blockIdx.y * per), hi = min(steps, lo + per), quarter = (hi - lo + 3) >> 2;
+  const int begin = min(hi, lo + wave * quarter), end = min(hi, begin + quarter);
+  const float* y = a.y + (size_t)(b0 + min(r, nb - 1)) * a.ldy;
+  const uint16_t* ring = a.ring + (size_t)(b0 + min(r, nb - 1)) * reach * a.inner;
+  f32x4_t acc[RT][1] = {};
+  tile_steps<RT, 1>(a.w + (size_t)(16 * tile0 + r) * a.inner, a.inner, begin, end, g, acc, [&](int, int s) {
+    u32x4_t packed = {0u, 0u, 0u, 0u};
+    if (r < nb) {
+      const int c = 32 * s + 8 * g;
+      Float8 sum = load8(a.bias + c);
+      for (int j = min(reach, p); j >= 0; --j) {
+        const Float8 w = load8(a.weight + (size_t)(reach - j) * a.inner + c);
+        Float8 v;
+        if (j > 0) {
+          v = load8(ring + (size_t)((p - j) % reach) * a.inner + c);
+        } else {  // (as the ring will hold it)
+          v = load8(y + c);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) v.v[e] = to_f32(f32_to_bf16_rne(v.v[e]));
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum.v[e] = fmaf(w.v[e], v.v[e], sum.v[e]);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) packed[e] = pack2_bf16(silu_f32(sum.v[2 * e]), silu_f32(sum.v[2 * e + 1]));
+    }
+    return packed;
+  });
+  meet<4, RT, 1>(acc, red, wave, lane);
+#pragma unroll
+  for (int i = 0; i < RT; ++i)
+    if (wave == i && r < nb)
+      store4(a.partial + ((size_t)blockIdx.y * a.batch + b0 + r) * a.rows + 16 * (tile0 + i) + 4 * g,
+             float4{acc[i][0][0], acc[i][0][1], acc[i][0][2], acc[i][0][3]});
+}
+
+// The rest of the step for 64 CT channels of kScanBatch sequences: the parts of (dt rank | B | C) are added, dt comes from a
+// product on MFMA (a wave per CT tiles of 16 channels), then a thread per (sequence, channel) convolves its channel, moves the
+// channel's states on and writes the gated output and the ring's new row.  Grid (channel blocks, batch blocks).
+constexpr int kScanBatch = 4;
+struct ScanStep {
+  const float* y;           // [B, ldy]: convolved columns, z from column inner on
+  uint16_t* ring;
+  const float *weight, *bias;
+  const long long* pos;
+  const float* partial;     // [splits, B, rows]: dt rank from 0, B from rank, C from rank + states
+  const uint16_t* w_dt;     // [inner, rank]
+  const float *dt_bias, *a2, *d;
+  float* state;             // [B, states / 4, inner, 4]
+  uint16_t* out;            // [B, out_ld]
+  int batch, ldy, inner, taps, rows, splits, rank, states, out_ld;
+};
+__host__ __device__ constexpr int scan_step_lds(int rank, int states, int ct) {
+  return kScanBatch * (2 * (rank + 8) + 4 * 2 * states + 4 * 64 * ct);
+}
+template <int CT>
+__global__ __launch_bounds__(256) void scan_step_kernel(ScanStep a) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char scan_lds[];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
+  const int b0 = blockIdx.y * kScanBatch, nb = min(kScanBatch, a.batch - b0), c0 = blockIdx.x * 64 * CT;
+  const int ld = a.rank + 8;
+  float* bc = reinterpret_cast<float*>(scan_lds);                    // [kScanBatch][2 states]
+  float* dt_s = bc + kScanBatch * 2 * a.states;                      // [kScanBatch][64 CT]
+  uint16_t* low = reinterpret_cast<uint16_t*>(dt_s + kScanBatch * 64 * CT);  // [kScanBatch][rank + 8]
+  const int used = a.rank + 2 * a.states;
+  for (int i = tid; i < nb * used; i += 256) {
+    const int b = i / used, n = i % used;
+    float v = 0.f;
+    for (int s = 0; s < a.splits; ++s) v += a.partial[((size_t)s * a.batch + b0 + b) * a.rows + n];
+    if (n < a.rank) low[b * ld + n] = f32_to_bf16_rne(v);
+    else bc[b * 2 * a.states + n - a.rank] = v;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int t = 0; t < CT; ++t) {
+    const int c = 16 * (CT * wave + t);
+    if (c0 + c >= a.inner) continue;
+    f32x4_t acc[1][1] = {};
+    tile_steps<1, 1>(a.w_dt + (size_t)(c0 + c + r) * a.rank, a.rank, 0, (a.rank + 31) >> 5, g, acc, [&](int, int s) {
+      return r < nb ? *reinterpret_cast<const u32x4_t*>(low + r * ld + 32 * s + 8 * g) : u32x4_t{0u, 0u, 0u, 0u};
+    });
+    if (r < nb) {
+      const float4 bias = load4(a.dt_bias + c0 + c + 4 * g);
+      store4(dt_s + r * 64 * CT + c + 4 * g, float4{softplus_f32(acc[0][0][0] + bias.x), softplus_f32(acc[0][0][1] + bias.y),
+                                                    softplus_f32(acc[0][0][2] + bias.z), softplus_f32(acc[0][0][3] + bias.w)});
+    }
+  }
+  __syncthreads();
+  const int reach = a.taps - 1, p = clamped_position(a.pos, 0, 0x7FFFFFFF);
+  for (int i = tid; i < nb * 64 * CT; i += 256) {
+    const int b = i / (64 * CT), local = i % (64 * CT), c = c0 + local;
+    if (c >= a.inner) continue;
+    const float* y = a.y + (size_t)(b0 + b) * a.ldy;
+    uint16_t* ring = a.ring + (size_t)(b0 + b) * reach * a.inner + c;
+    const uint16_t own = f32_to_bf16_rne(y[c]);
+    float x = a.bias[c];
+    for (int j = min(reach, p); j >= 0; --j)
+      x = fmaf(a.weight[(size_t)(reach - j) * a.inner + c], to_f32(j > 0 ? ring[(size_t)((p - j) % reach) * a.inner] : own), x);
+    if (reach > 0) ring[(size_t)(p % reach) * a.inner] = own;
+    x = silu_f32(x);
+    const float dt = dt_s[b * 64 * CT + local], dx = dt * x;
+    float* state = a.state + ((size_t)(b0 + b) * a.states * a.inner) + 4 * c;
+    const float* bs = bc + b * 2 * a.states;
+    float out = a.d[c] * x;
+#pragma unroll 4
+    for (int n = 0; n < a.states; n += 4) {
+      const float4 f = load4(a.a2 + (size_t)n * a.inner + 4 * c);
+      float4 s = p > 0 ? load4(state + (size_t)n * a.inner) : float4{0.f, 0.f, 0.f, 0.f};
+      const float4 bn = load4(bs + n), cn = load4(bs + a.states + n);
+      s.x = fmaf(__builtin_amdgcn_exp2f(dt * f.x), s.x, dx * bn.x);
+      s.y = fmaf(__builtin_amdgcn_exp2f(dt * f.y), s.y, dx * bn.y);
+      s.z = fmaf(__builtin_amdgcn_exp2f(dt * f.z), s.z, dx * bn.z);
+      s.w = fmaf(__builtin_amdgcn_exp2f(dt * f.w), s.w, dx * bn.w);
+      store4(state + (size_t)n * a.inner, s);
+      out = fmaf(s.x, cn.x, fmaf(s.y, cn.y, fmaf(s.z, cn.z, fmaf(s.w, cn.w, out))));
+    }
+    a.out[(size_t)(b0 + b) * a.out_ld + c] = f32_to_bf16_rne(out * silu_f32(y[a.inner + c]));
+  }
+}
+
+}  // namespace ajq

@@ -14,12 +14,12 @@ import ctypes
 
 import torch
 
-from . import _lib, latent, modeling
+from . import _lib, dense, modeling
 from .quant import QuantLinear, repack_w4, repack_w8, w4a16_matmul, w8a16_matmul
 
 
 class GraphDecoder:
-    def __init__(self, model: modeling.TransformerLM | latent.LatentLM, batch: int, max_len: int,
+    def __init__(self, model: modeling.TransformerLM | dense.DenseLM, batch: int, max_len: int,
                  kv_dtype: torch.dtype | None = None) -> None:
         if max_len > model.context_length:
             raise ValueError(f"max_len {max_len} exceeds the model's context length {model.context_length}")
@@ -748,12 +748,12 @@ class FusedDecoder(GraphDecoder):
         return self.logits_full[:, : self.vocab]
 
 
-class LatentDecoder(GraphDecoder):
-    """GraphDecoder for a ``latent.LatentLM``, whose step is this library's kernels already: the choice of the token
+class DenseDecoder(GraphDecoder):
+    """GraphDecoder for a ``dense.DenseLM``, whose step is this library's kernels already: the choice of the token
     and the step's two counters are one launch as well (``ajq_greedy_pick`` / ``ajq_sample_pick``), and eight steps make
     a graph.  A prompt may be given in portions of ``tokens_per_pass``."""
 
-    def __init__(self, model: latent.LatentLM, batch: int, max_len: int, kv_dtype: torch.dtype | None = None) -> None:
+    def __init__(self, model: dense.DenseLM, batch: int, max_len: int, kv_dtype: torch.dtype | None = None) -> None:
         super().__init__(model, batch, max_len, kv_dtype)
         self.steps_per_graph = 8
         # cache position and output column advance together, at the end of a step (see FusedDecoder)
@@ -798,8 +798,8 @@ class LatentDecoder(GraphDecoder):
 
 def decoder_for(model: torch.nn.Module, fused: bool = False) -> type[GraphDecoder]:
     """The decoder class that serves ``model``."""
-    if isinstance(model, latent.LatentLM):
-        return LatentDecoder
+    if isinstance(model, dense.DenseLM):
+        return DenseDecoder
     return FusedDecoder if fused else GraphDecoder
 
 

@@ -9,8 +9,7 @@ arguments:
 * ``ParallelBlock``      mixer and feed-forward side by side on two norms of the incoming stream, one sum at the end
 * ``Loop``               a span of layers traversed several times; every traversal has rings of its own in the cache and a
                          learned offset for the stream it starts from, the later ones take the embedding in again as well
-* ``LatentLM``           the decoder: ``forward(token_ids, cache)`` is the one step function, for whole prompts, portions
-                         of prompts and single tokens; ``modeling.greedy_decode`` and the decoders of ``decoding`` call it
+* ``LatentLM``           the decoder (``dense.DenseLM``)
 
 All of it runs on the operators of ``libajq_dense.so`` on a ROCm device, weights and activations in bf16 or fp32 (plain
 matrix products of prompts are the vendor library's).  There is no CPU path.  The residual stream, norms, angles,
@@ -23,28 +22,15 @@ moves its query into the latent space instead and attends to the cached latents 
 from __future__ import annotations
 
 import ctypes
-from dataclasses import dataclass
 from typing import Any
 
 import torch
 from torch import nn
 
 from . import _lib
+from .dense import (NORM_PROLOGUE_ROWS, DenseLM, Loop, _add_norms, _flag, _matvec, _padded, _product, _ptr, _stream, _up,
+                    rotary_frequencies)
 from .modeling import Embedding, GatedFeedForward, Linear, RingCache, RMSNorm, build_norm, register_architecture
-
-GEMV_ROWS = 16    # rows of a prompt up to which the head's product is a matrix-vector kernel of this library
-# rows up to which the decode products form the norms themselves (their workgroups each normalise every row: free at one
-# row, 7 us of 55 at two, where a norm launch costs 3)
-NORM_PROLOGUE_ROWS = 1
-
-
-@dataclass(frozen=True)
-class Loop:
-    """Layers ``start .. stop - 1`` run ``times`` times in a row."""
-
-    start: int
-    stop: int
-    times: int
 
 
 class LatentAttention(nn.Module):
@@ -78,22 +64,8 @@ class ParallelBlock(nn.Module):
 
 def rotary_tables(base: float, dims: int, length: int) -> tuple[torch.Tensor, torch.Tensor]:
     """cos and sin of p * base^(-2 i / dims), ``[length, dims / 2]`` fp32 (angles formed in double on the host)."""
-    i = torch.arange(dims // 2, dtype=torch.float64)
-    angles = torch.arange(length, dtype=torch.float64)[:, None] * torch.pow(torch.tensor(base, dtype=torch.float64), -2.0 * i / dims)
+    angles = torch.arange(length, dtype=torch.float64)[:, None] * rotary_frequencies(base, dims)
     return torch.cos(angles).float(), torch.sin(angles).float()
-
-
-def _up(n: int, to: int) -> int:
-    return (n + to - 1) // to * to
-
-
-def _padded(t: torch.Tensor, *sizes: int) -> torch.Tensor:
-    """``t`` with zeros appended up to ``sizes``."""
-    if tuple(t.shape) == sizes:
-        return t.contiguous()
-    out = torch.zeros(sizes, dtype=t.dtype, device=t.device)
-    out[tuple(slice(0, n) for n in t.shape)] = t
-    return out
 
 
 def interleave_gate(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
@@ -154,54 +126,14 @@ class PackedBlock:
         self.shape = _lib.LatentShape(heads, self.dimp, mix.rot_dim, self.rotp, mix.kv_rank, self.rankp, mix.dkv_norm.epsilon)
 
 
-def _ptr(t: torch.Tensor | None) -> int | None:
-    return t.data_ptr() if t is not None else None
-
-
-def _flag(dtype: torch.dtype) -> int:
-    return _lib.AJQD_BF16 if dtype == torch.bfloat16 else _lib.AJQD_F32
-
-
-def _stream() -> int:
-    return torch.cuda.current_stream().cuda_stream
-
-
-def _product(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
-    """``x w^T`` of many rows (the vendor library's product, fp32 accumulation)."""
-    if x.dtype == out_dtype:
-        return torch.mm(x, w.t())
-    return torch.mm(x, w.t(), out_dtype=out_dtype)
-
-
-def _add_norms(x: torch.Tensor, delta: torch.Tensor | None, again: torch.Tensor | None, step: torch.Tensor | None,
-               gain1: torch.Tensor | None, gain2: torch.Tensor | None, eps: float, center: int, true_width: int,
-               dtype: torch.dtype) -> tuple[torch.Tensor | None, torch.Tensor | None]:
-    """``x += delta + again + step`` in place; the normed rows for each gain given."""
-    out1 = torch.empty(x.shape, dtype=dtype, device=x.device) if gain1 is not None else None
-    out2 = torch.empty(x.shape, dtype=dtype, device=x.device) if gain2 is not None else None
-    _lib.check_dense(_lib.load_dense().ajqd_add_norms(
-        _ptr(x), _ptr(delta), _flag(delta.dtype) if delta is not None else _lib.AJQD_F32, _ptr(again), _ptr(step), _ptr(gain1),
-        _ptr(gain2), eps, center, _ptr(out1), _ptr(out2), x.shape[0], true_width, x.shape[1], _flag(dtype), _stream()), "add_norms")
-    return out1, out2
-
-
-def _matvec(w: torch.Tensor, groups: int, x: torch.Tensor, x_batch: int, x_group: int, y: torch.Tensor, y_batch: int,
-            y_group: int, batch: int) -> None:
-    """``y[b, g] = w[g] x[b, g]`` for ``w [groups * n, k]``; strides in elements."""
-    _lib.check_dense(_lib.load_dense().ajqd_matvec(
-        _ptr(w), _ptr(x), x_batch, x_group, _ptr(y), y_batch, y_group, groups, w.shape[0] // groups, w.shape[1], batch,
-        _flag(w.dtype), _flag(y.dtype), _stream()), "matvec")
-
-
-class LatentLM(nn.Module):
+class LatentLM(DenseLM):
     """The decoder.  ``blocks``: one ``(mixer arguments, feed-forward (width, activation) or None)`` per layer."""
 
     def __init__(self, vocab_size: int, context_length: int, d_model: int, blocks: list[tuple[dict[str, Any], tuple[int, str] | None]],
                  loop: Loop | None = None, norm: str = "layernorm", epsilon: float = 1e-5) -> None:
         super().__init__()
-        if loop is not None and not (0 <= loop.start < loop.stop <= len(blocks) and loop.times >= 1):
-            raise ValueError(f"the loop {loop} does not fit {len(blocks)} layers")
         self.vocab_size, self.context_length, self.d_model, self.loop = vocab_size, context_length, d_model, loop
+        self._check_loop(len(blocks))
         self.token_embeddings = Embedding(vocab_size, d_model)
         self.position_embeddings = Embedding(context_length, d_model)
         self.layers = nn.ModuleList([
@@ -212,17 +144,6 @@ class LatentLM(nn.Module):
         self.loop_step = nn.Parameter(torch.zeros(loop.times, d_model)) if loop is not None else None
         self.final_norm = build_norm(norm, d_model, epsilon)
         self.lm_head = Linear(d_model, vocab_size)
-        self._packed: tuple | None = None
-
-    # ---- structure
-    @property
-    def runs(self) -> list[tuple[int, int | None]]:
-        """``(layer, pass)`` in running order; the pass is given on the layer run that begins it."""
-        if self.loop is None:
-            return [(i, None) for i in range(len(self.layers))]
-        lo, hi = self.loop.start, self.loop.stop
-        inner = [(i, t if i == lo else None) for t in range(self.loop.times) for i in range(lo, hi)]
-        return [(i, None) for i in range(lo)] + inner + [(i, None) for i in range(hi, len(self.layers))]
 
     def checkpoint_names(self) -> dict[str, str]:
         """State-dict key -> tensor name in a checkpoint file."""
@@ -255,89 +176,27 @@ class LatentLM(nn.Module):
         return RingCache([min(m.window or max_len, max_len) for m in mixers],
                          [_up(m.kv_rank, 16) + _up(m.rot_dim, 8) for m in mixers], batch, max_len, weight.device, weight.dtype)
 
-    # ---- weights as the kernels read them
-    def prepare(self) -> None:
-        """(Re)build the packed weights from the parameters; done by itself at the first call.  Call it again after
-        changing parameters in place."""
+    def _pack(self) -> None:
         weight = self.token_embeddings.weight
-        if weight.dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError("the model must be bfloat16 or float32")
-        if weight.device.type != "cuda":
-            raise ValueError("LatentLM runs on a ROCm device (there is no CPU path)")
-        if any(not isinstance(m, Linear) for layer in self.layers for m in layer.modules() if hasattr(m, "in_features")):
-            raise ValueError("LatentLM runs on dense weights (its linears have been replaced)")
-        if any(p.dtype != weight.dtype or p.device != weight.device for p in self.parameters()):
-            raise ValueError("all parameters must share one dtype and device")
         tables: dict = {}
         blocks = []
-        with torch.no_grad():
-            for layer in self.layers:
-                key = (layer.mixer.rot_base, layer.mixer.rot_dim)
-                if key not in tables:
-                    tables[key] = tuple(t.to(weight.device) for t in rotary_tables(*key, self.context_length))
-                blocks.append(PackedBlock(layer, tables[key]))
-            dp = _up(self.d_model, 16)
-            self._blocks = blocks
-            self._embed = _padded(weight.detach(), self.vocab_size, dp)
-            self._pos = _padded(self.position_embeddings.weight.detach(), self.context_length, dp)
-            self._steps = _padded(self.loop_step.detach().float(), self.loop.times, dp) if self.loop is not None else None
-            self._final_gain = _padded(self.final_norm.weight.detach().float(), dp)
-            self._head = _padded(self.lm_head.weight.detach(), _up(self.vocab_size, 16), dp)
-        self._packed = (weight.data_ptr(), weight.dtype, weight.device)
-
-    def _ready(self) -> None:
-        weight = self.token_embeddings.weight
-        if self._packed != (weight.data_ptr(), weight.dtype, weight.device):
-            self.prepare()
+        for layer in self.layers:
+            key = (layer.mixer.rot_base, layer.mixer.rot_dim)
+            if key not in tables:
+                tables[key] = tuple(t.to(weight.device) for t in rotary_tables(*key, self.context_length))
+            blocks.append(PackedBlock(layer, tables[key]))
+        dp = _up(self.d_model, 16)
+        self._blocks = blocks
+        self._embed = _padded(weight.detach(), self.vocab_size, dp)
+        self._pos = _padded(self.position_embeddings.weight.detach(), self.context_length, dp)
+        self._steps = _padded(self.loop_step.detach().float(), self.loop.times, dp) if self.loop is not None else None
+        self._final_gain = _padded(self.final_norm.weight.detach().float(), dp)
+        self._head = _padded(self.lm_head.weight.detach(), _up(self.vocab_size, 16), dp)
 
     def _begins(self, run: int) -> tuple[bool, torch.Tensor | None]:
         """What is added to x ahead of a layer run: whether the embedding output is, and the pass's vector."""
         t = self.runs[run][1] if run < len(self.runs) else None
         return (t is not None and t > 0), (self._steps[t] if t is not None else None)
-
-    # ---- the step
-    @torch.no_grad()
-    def forward(self, token_ids: torch.Tensor, cache: RingCache | None = None, last_token_only: bool = False,
-                want: torch.Tensor | None = None, residuals: list | None = None) -> torch.Tensor:
-        """Logits (fp32) ``[B, n, V]`` of the new tokens ``token_ids [B, T]``, which continue at ``cache.length``
-        (``cache.position`` for a static cache).  ``last_token_only``, or ``want`` (a list of places among the T tokens,
-        possibly empty) selects the places whose logits are formed.  ``residuals`` collects copies of the residual
-        stream after every layer run (prompts only)."""
-        batch, seq = token_ids.shape
-        self._ready()
-        if not token_ids.is_cuda:
-            raise ValueError("LatentLM takes token ids on the model's device")
-        token_ids = token_ids.contiguous()
-        static = cache is not None and cache.static
-        if static and seq != 1:
-            raise ValueError("a static cache takes one token per call")
-        if cache is not None and cache.batch != batch:
-            raise ValueError(f"the cache holds {cache.batch} sequences, {batch} given")
-        start = cache.length if cache is not None and not static else 0
-        if not static and start + seq > self.context_length:
-            raise ValueError(f"Input length {start + seq} exceeds context length {self.context_length}")
-        if not static and cache is not None and start + seq > cache.max_len:
-            raise ValueError(f"the cache holds {cache.max_len} positions, {start + seq} needed")
-        single = cache is not None and seq == 1 and residuals is None
-        if single:
-            if not static:
-                cache.position.fill_(start)
-            x, delta = self._token(token_ids, cache)
-        else:
-            x, delta = self._prompt(token_ids, cache, start, residuals)
-        if cache is not None and not static:
-            cache.length = start + seq
-        if last_token_only:
-            want = [seq - 1]
-        if want is not None:
-            picks = list(want)
-            if not picks:
-                return torch.empty((batch, 0, self.vocab_size), dtype=torch.float32, device=x.device)
-            if not (seq == 1 and len(picks) == 1):
-                rows = torch.tensor([b * seq + t for b in range(batch) for t in picks], device=x.device)
-                x = x.index_select(0, rows)
-                delta = delta.index_select(0, rows) if delta is not None else None
-        return self._logits(x, delta, single).view(batch, -1, self._head.shape[0])[:, :, : self.vocab_size]
 
     def _embedded(self, token_ids: torch.Tensor, start: int, pos: torch.Tensor | None) -> tuple[torch.Tensor, torch.Tensor | None]:
         """The residual stream in front of the first layer run, and the embedding output where a loop needs it again."""
@@ -349,28 +208,6 @@ class LatentLM(nn.Module):
             _ptr(token_ids), batch * seq, seq, _ptr(self._embed), self.vocab_size, _ptr(self._pos), self.context_length, start,
             _ptr(pos), _ptr(self._begins(0)[1]), _ptr(x), _ptr(embedded), dp, _flag(self._embed.dtype), _stream()), "embed")
         return x, embedded
-
-    def _logits(self, x: torch.Tensor, delta: torch.Tensor | None, single: bool) -> torch.Tensor:
-        """``head norm(x + delta)``, fp32, columns padded to a multiple of 16.  ``single``: a decode step (its products are
-        this library's for any number of sequences: library kernels stay out of recorded graphs)."""
-        rows, dtype = x.shape[0], self._head.dtype
-        if not single and rows > GEMV_ROWS:
-            normed, _ = _add_norms(x, delta, None, None, self._final_gain, None, self.final_norm.epsilon,
-                                   0 if isinstance(self.final_norm, RMSNorm) else 1, self.d_model, dtype)
-            return _product(normed, self._head, torch.float32)
-        center = 0 if isinstance(self.final_norm, RMSNorm) else 1
-        eps, gain = self.final_norm.epsilon, self._final_gain
-        y = torch.empty((rows, self._head.shape[0]), dtype=torch.float32, device=x.device)
-        if dtype == torch.bfloat16:
-            if delta is None and rows <= NORM_PROLOGUE_ROWS:
-                self._dense_in(x, None, None, gain, None, eps, center, self._head, None, y, None, 0, 0)
-                return y
-            normed, _ = _add_norms(x, delta, None, None, gain, None, eps, center, self.d_model, dtype)
-            self._dense_in(None, normed, None, None, None, eps, center, self._head, None, y, None, 0, 0)
-            return y
-        normed, _ = _add_norms(x, delta, None, None, gain, None, eps, center, self.d_model, dtype)
-        _matvec(self._head, 1, normed, normed.shape[1], 0, y, y.shape[1], 0, rows)
-        return y
 
     # ---- many tokens per sequence
     def _prompt(self, token_ids: torch.Tensor, cache: RingCache | None, start: int,
@@ -391,8 +228,8 @@ class LatentLM(nn.Module):
             ring = cache.rings[run] if cache is not None else None
             row_bytes = w.width * rows.element_size()
             if reach > 0:
-                _lib.check_dense(lib.ajqd_ring_copy(_ptr(ring), ring.shape[1], _ptr(rows), reach + seq, 0, start - reach, reach,
-                                                    row_bytes, batch, 0, st), "ring_copy")
+                _lib.check_dense(lib.ajqd_ring_copy(_ptr(ring), ring.shape[1], 0, _ptr(rows), reach + seq, row_bytes, 0,
+                                                    start - reach, reach, row_bytes, batch, 0, st), "ring_copy")
             q = torch.empty((m, w.heads, w.dimp + w.rotp), dtype=dtype, device=dev)
             gates = torch.empty((m, w.heads), dtype=torch.float32, device=dev)
             _lib.check_dense(lib.ajqd_latent_split(
@@ -419,7 +256,7 @@ class LatentLM(nn.Module):
             delta = _product(joined, w.wo, torch.float32)
             if ring is not None:
                 keep = min(seq, ring.shape[1])
-                _lib.check_dense(lib.ajqd_ring_copy(_ptr(ring), ring.shape[1], _ptr(rows), reach + seq, reach + seq - keep,
+                _lib.check_dense(lib.ajqd_ring_copy(_ptr(ring), ring.shape[1], 0, _ptr(rows), reach + seq, row_bytes, reach + seq - keep,
                                                     start + seq - keep, keep, row_bytes, batch, 1, st), "ring_copy")
             if residuals is not None:
                 residuals.append((x + delta)[:, : self.d_model].view(batch, seq, -1))
@@ -446,14 +283,6 @@ class LatentLM(nn.Module):
                 delta = self._token_plain(x, delta, embedded, run, w, ring, cache.position)
         return x, delta
 
-    def _dense_in(self, x, n1, n2, gain1, gain2, eps, center, w1, w2, y1, gated, gated_ld, act) -> None:
-        batch = x.shape[0] if x is not None else n1.shape[0]
-        args = _lib.DenseInArgs(
-            x=_ptr(x), n1=_ptr(n1), n2=_ptr(n2), gain1=_ptr(gain1), gain2=_ptr(gain2), w1=_ptr(w1), w2=_ptr(w2), y1=_ptr(y1),
-            gated=gated, batch=batch, true_width=self.d_model, width=w1.shape[1], tiles1=w1.shape[0] // 16,
-            tiles2=w2.shape[0] // 16 if w2 is not None else 0, gated_ld=gated_ld, act=act, center=center, eps=eps)
-        _lib.check_dense(_lib.load_dense().ajqd_dense_in(ctypes.byref(args), _stream()), "dense_in")
-
     def _token_fused(self, x, delta, embedded, run: int, w: PackedBlock, ring, pos, chunks: int) -> None:
         """One layer run in five launches (six for more than one sequence); x is updated in place, with what the next layer run
         adds first included."""
@@ -476,7 +305,7 @@ class LatentLM(nn.Module):
                                                 ring.shape[1], batch, st), "latent_absorb")
         partial = torch.empty(lib.ajqd_latent_decode_workspace(batch, w.heads, w.rankp, chunks), dtype=torch.uint8, device=dev)
         _lib.check_dense(lib.ajqd_latent_decode(_ptr(q), _ptr(ring), _ptr(pos), _ptr(partial), batch, w.heads, w.rankp, w.rotp,
-                                                ring.shape[1], chunks, w.scale, st), "latent_decode")
+                                                ring.shape[1], chunks, 0, w.scale, st), "latent_decode")
         gate = y.data_ptr() + 4 * w.gate_column if w.gated_heads else None
         _lib.check_dense(lib.ajqd_latent_expand(_ptr(partial), _ptr(w.sink), gate, y.shape[1], _ptr(w.uv), _ptr(joined),
                                                 w.joined, batch, w.heads, chunks, w.rankp, w.vdimp, st), "latent_expand")

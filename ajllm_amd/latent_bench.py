@@ -105,7 +105,7 @@ def bench_whole(size: dict, device, log=print, batches=(1, 8, 32), steps: int = 
     out: dict = {"layer_runs": runs, "prompt": {"tokens": PROMPT_ROWS * CONTEXT, "latent_ms": seconds * 1e3,
                                                 "latent_tok/s": PROMPT_ROWS * CONTEXT / seconds}, "decode": []}
     for batch in batches:
-        dec = decoding.LatentDecoder(model, batch, CONTEXT + steps + 16)
+        dec = decoding.DenseDecoder(model, batch, CONTEXT + steps + 16)
         dec.prefill(prompt[:batch], rows_per_pass=PROMPT_ROWS)
         dec.generate(12)
         t0 = time.perf_counter()
@@ -205,7 +205,7 @@ def bench_kernels(size: dict, device, log=print, batches=(1, 8, 32)) -> list[dic
         chunks = lib.ajqd_latent_decode_chunks(batch, heads, w0.rankp, w0.rotp, window)
         partial = torch.empty(lib.ajqd_latent_decode_workspace(batch, heads, w0.rankp, chunks), dtype=torch.uint8, device=device)
         attend = lambda r: _lib.check_dense(lib.ajqd_latent_decode(q.data_ptr(), r.data_ptr(), pos.data_ptr(), partial.data_ptr(), batch, heads,
-                                                                   w0.rankp, w0.rotp, window, chunks, w0.scale, _st()), "latent_decode")
+                                                                   w0.rankp, w0.rotp, window, chunks, 0, w0.scale, _st()), "latent_decode")
         # the other model's decode attention over a bf16 cache of about as many bytes
         hd, hkv = d // heads, size["kv_heads"]
         context = max(16, ring_bytes // (4 * batch * hkv * hd))

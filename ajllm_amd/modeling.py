@@ -57,6 +57,8 @@ class Embedding(nn.Module):
 class RMSNorm(nn.Module):
     """x / sqrt(mean(x^2) + eps) * gain, computed in fp32 and cast back."""
 
+    zero_centered = False    # whether the gain is 1 + weight
+
     def __init__(self, d_model: int, epsilon: float = 1e-5, device=None, dtype=None) -> None:
         super().__init__()
         self.epsilon = epsilon
@@ -66,6 +68,21 @@ class RMSNorm(nn.Module):
         x = inputs.float()
         rms = torch.sqrt(torch.mean(x.square(), dim=-1, keepdim=True) + self.epsilon)
         return ((x / rms) * self.weight).to(inputs.dtype)
+
+
+class ZeroCenteredRMSNorm(RMSNorm):
+    """RMS norm whose gain is 1 + weight."""
+
+    zero_centered = True
+
+    def __init__(self, d_model: int, epsilon: float = 1e-5, device=None, dtype=None) -> None:
+        super().__init__(d_model, epsilon, device, dtype)
+        nn.init.zeros_(self.weight)
+
+    def forward(self, inputs: torch.Tensor) -> torch.Tensor:
+        x = inputs.float()
+        rms = torch.sqrt(torch.mean(x.square(), dim=-1, keepdim=True) + self.epsilon)
+        return ((x / rms) * (1.0 + self.weight.float())).to(inputs.dtype)
 
 
 class LayerNorm(nn.Module):
@@ -85,6 +102,8 @@ class LayerNorm(nn.Module):
 def build_norm(kind: str, d_model: int, epsilon: float = 1e-5) -> nn.Module:
     if kind == "rmsnorm":
         return RMSNorm(d_model, epsilon)
+    if kind == "zero_centered_rmsnorm":
+        return ZeroCenteredRMSNorm(d_model, epsilon)
     if kind == "layernorm":
         return LayerNorm(d_model, epsilon)
     if kind == "none":
@@ -99,6 +118,7 @@ def silu(inputs: torch.Tensor) -> torch.Tensor:
 ACTIVATIONS = {
     "silu": silu,
     "relu": torch.relu,
+    "squared_relu": lambda z: torch.relu(z).square(),
     "gelu_tanh": lambda z: 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3))),
 }
 
@@ -126,16 +146,26 @@ class SwiGLU(GatedFeedForward):
         super().__init__(d_model, d_ff, "silu")
 
 
-class SiLUFeedForward(nn.Module):
-    """w2(silu(w1 x))"""
+class PlainFeedForward(nn.Module):
+    """w2(act(w1 x))"""
 
-    def __init__(self, d_model: int, d_ff: int) -> None:
+    def __init__(self, d_model: int, d_ff: int, activation: str = "silu") -> None:
         super().__init__()
+        if activation not in ACTIVATIONS:
+            raise ValueError(f"Unsupported activation: {activation}")
+        self.activation = activation
         self.w1 = Linear(d_model, d_ff)
         self.w2 = Linear(d_ff, d_model)
 
     def forward(self, inputs: torch.Tensor) -> torch.Tensor:
-        return self.w2(silu(self.w1(inputs)))
+        return self.w2(ACTIVATIONS[self.activation](self.w1(inputs)))
+
+
+class SiLUFeedForward(PlainFeedForward):
+    """w2(silu(w1 x))"""
+
+    def __init__(self, d_model: int, d_ff: int) -> None:
+        super().__init__(d_model, d_ff, "silu")
 
 
 def build_feed_forward(kind: str, d_model: int, d_ff: int) -> nn.Module:
@@ -145,6 +175,8 @@ def build_feed_forward(kind: str, d_model: int, d_ff: int) -> nn.Module:
         return SiLUFeedForward(d_model, d_ff)
     if kind == "reglu":
         return GatedFeedForward(d_model, d_ff, "relu")
+    if kind == "squared_relu":
+        return PlainFeedForward(d_model, d_ff, "squared_relu")
     raise ValueError(f"Unsupported feed-forward type: {kind}")
 
 
@@ -222,17 +254,28 @@ class KVCache:
 
 
 class RingCache:
-    """Cache of a model whose layer runs keep one row per position and look a bounded number of positions back:
-    ``rings[run]`` is ``[B, capacity, width]``, position p in slot p % capacity, so a run holds its window and no more
-    (``capacities[run] = min(window, max_len)``; a run without a window keeps every position).  A layer that runs
-    several times has a ring per pass.
+    """Cache of a model whose layer runs keep rows of the last positions, a state, or both.
+
+    ``rings[run]`` is ``[B, capacity, width]``, or ``[B, groups, capacity, width]`` where ``groups`` gives a number: position p
+    lies in slot p % capacity, so a run holds its window and no more (``capacities[run] = min(window, max_len)``; a run
+    without a window keeps every position).  The first ``kept[run]`` positions keep slots of their own, ahead of the
+    others': p stays in slot p there, and in slot kept + (p - kept) % (capacity - kept) behind.  ``states[run]`` is an fp32
+    tensor ``[B, ...]`` a recurrent layer carries along (None: it has none); what it holds counts from position 1 on.  A
+    layer that runs several times has all of this per pass.
 
     The two modes are ``KVCache``'s: dynamic (``length``, calls of any number of tokens) and static (one token per
     call at the device-side ``position``, fixed shapes for a recorded graph; the caller advances it)."""
 
-    def __init__(self, capacities: list[int], widths: list[int], batch: int, max_len: int, device, dtype) -> None:
-        self.rings = [torch.zeros(batch, rows, width, device=device, dtype=dtype)
-                      for rows, width in zip(capacities, widths)]
+    def __init__(self, capacities: list[int], widths: list[int], batch: int, max_len: int, device, dtype,
+                 groups: list[int | None] | None = None, kept: list[int] | None = None,
+                 states: list[tuple[int, ...] | None] | None = None) -> None:
+        runs = len(capacities)
+        groups = groups or [None] * runs
+        self.rings = [torch.zeros((batch, rows, width) if g is None else (batch, g, rows, width), device=device, dtype=dtype)
+                      for rows, width, g in zip(capacities, widths, groups)]
+        self.kept = kept or [0] * runs
+        self.states = [torch.zeros((batch, *shape), device=device) if shape is not None else None
+                       for shape in states or [None] * runs]
         self.batch = batch
         self.length = 0
         self.max_len = max_len
@@ -243,6 +286,8 @@ class RingCache:
         """A cache over sequences ``start .. stop - 1`` of this one, sharing its storage (dynamic mode, empty)."""
         view = object.__new__(RingCache)
         view.rings = [ring[start:stop] for ring in self.rings]
+        view.kept = self.kept
+        view.states = [state[start:stop] if state is not None else None for state in self.states]
         view.batch = stop - start
         view.length = 0
         view.max_len = self.max_len
@@ -251,7 +296,8 @@ class RingCache:
         return view
 
     def reset(self) -> None:
-        """Give the cache to another sequence: a position is read only after it has been written again."""
+        """Give the cache to another sequence: a position is read only after it has been written again, and a state is
+        not read at position 0."""
         self.length = 0
         self.static = False
 
@@ -450,7 +496,7 @@ def build_model(config: dict[str, Any], vocab_size: int | None = None) -> nn.Mod
     """Model from a config dict: one that names an ``architecture`` goes to that architecture's builder, any other is
     a reference-style dict (keys as in the reference's model YAML)."""
     if "architecture" in config:
-        from . import latent  # noqa: F401  (registers its architectures)
+        from . import hybrid, latent  # noqa: F401  (they register their architectures)
         name = config["architecture"]
         if name not in ARCHITECTURES:
             raise ValueError(f"Unsupported architecture: {name} (known: {', '.join(sorted(ARCHITECTURES))})")

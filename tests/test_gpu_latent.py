@@ -126,9 +126,9 @@ def test_matvec(cuda, k):
 def test_ring_copy_both_ways(cuda):
     ring = torch.zeros((2, 7, 16), device=cuda)
     line = torch.arange(2 * 9 * 16, dtype=torch.float32, device=cuda).view(2, 9, 16)
-    _ok(_lib.load_dense().ajqd_ring_copy(ring.data_ptr(), 7, line.data_ptr(), 9, 3, 12, 6, 64, 2, 1, _st()))
+    _ok(_lib.load_dense().ajqd_ring_copy(ring.data_ptr(), 7, 0, line.data_ptr(), 9, 64, 3, 12, 6, 64, 2, 1, _st()))
     back = torch.zeros_like(line)
-    _ok(_lib.load_dense().ajqd_ring_copy(ring.data_ptr(), 7, back.data_ptr(), 9, 1, 12, 6, 64, 2, 0, _st()))
+    _ok(_lib.load_dense().ajqd_ring_copy(ring.data_ptr(), 7, 0, back.data_ptr(), 9, 64, 1, 12, 6, 64, 2, 0, _st()))
     for i in range(6):
         assert torch.equal(ring[:, (12 + i) % 7], line[:, 3 + i])
     assert (ring[:, (12 + 6) % 7] == 0).all()
@@ -274,7 +274,7 @@ def test_latent_decode_and_expand_against_plain(cuda, shape):
     for chunks in sorted({1, 2, 3, 7, 32, suggested}):
         partial = torch.full((lib.ajqd_latent_decode_workspace(batch, heads, rank, chunks),), 255, dtype=torch.uint8, device=cuda)
         _ok(lib.ajqd_latent_decode(d["q"].data_ptr(), d["ring"].data_ptr(), pos.data_ptr(), partial.data_ptr(), batch, heads, rank, rot,
-                                   cap, chunks, scale, _st()))
+                                   cap, chunks, 0, scale, _st()))
         out = torch.full((batch, heads * vdim + 8), 5.0, dtype=torch.bfloat16, device=cuda)
         _ok(lib.ajqd_latent_expand(partial.data_ptr(), d["sink"].data_ptr(), d["gate"].data_ptr(), heads, d["uv"].data_ptr(),
                                    out.data_ptr(), heads * vdim + 8, batch, heads, chunks, rank, vdim, _st()))
@@ -465,7 +465,7 @@ def test_greedy_generation_through_the_decoders(cuda, dtype, batch):
     new = 75
     graph = decoding.greedy_decode_graph(model, prompts, new)
     eager = modeling.greedy_decode(model, prompts, new)
-    dec = decoding.LatentDecoder(model, batch, 37 + new)
+    dec = decoding.DenseDecoder(model, batch, 37 + new)
     dec.prefill(prompts, tokens_per_pass=8)
     portions = dec.generate(new)
     for i in range(batch):
@@ -478,7 +478,7 @@ def test_graph_replays_equal_the_eager_step(cuda):
     """The same decoder used for two prompts (the second from a used cache), with other work between the replays."""
     cfg = config()
     model = _build(cfg, random_weights(cfg, 23), cuda, torch.bfloat16)
-    dec = decoding.LatentDecoder(model, 2, 120)
+    dec = decoding.DenseDecoder(model, 2, 120)
     for seed in (1, 2, 3):
         prompts = torch.tensor([_tokens(cfg, 20, seed), _tokens(cfg, 20, seed + 9)], device=cuda)
         dec.prefill(prompts)
@@ -502,16 +502,16 @@ def test_sampling_and_stop_token(cuda):
     prompts = torch.tensor([_tokens(cfg, 12, 3)], device=cuda)
 
     def draw(seed):
-        dec = decoding.LatentDecoder(model, 1, 80)
+        dec = decoding.DenseDecoder(model, 1, 80)
         dec.set_sampling(1.0, 0.9, seed)
         dec.prefill(prompts)
         return dec.generate(60)
 
     assert torch.equal(draw(1), draw(1)) and not torch.equal(draw(1), draw(2))
-    dec = decoding.LatentDecoder(model, 1, 80)
+    dec = decoding.DenseDecoder(model, 1, 80)
     dec.prefill(prompts)
     tokens = dec.generate(60)[0].tolist()
-    dec = decoding.LatentDecoder(model, 1, 80)
+    dec = decoding.DenseDecoder(model, 1, 80)
     dec.prefill(prompts)
     stop = tokens[30]
     assert dec.generate(60, eos_token_id=stop)[0].tolist() == tokens[: tokens.index(stop) + 1]

@@ -234,7 +234,7 @@ def test_dense_library_refuses_bad_arguments_before_any_launch():
     assert lib.ajqd_embed(p, 3, 3, p, 4, p, 8, 6, None, None, p, None, 16, 0, None) == -2      # positions 6 .. 8 of 8
     assert lib.ajqd_embed(p, 1, 1, p, 4, p, 8, 0, None, None, p, None, 16, 7, None) == -4      # unknown dtype
     assert lib.ajqd_add_norms(p, None, 1, None, None, p, None, 1e-5, 1, p, None, 1, 12, 12, 0, None) == -2
-    assert lib.ajqd_ring_copy(p, 4, p, 8, 0, 0, 5, 32, 1, 1, None) == -2                        # more rows than the ring has
+    assert lib.ajqd_ring_copy(p, 4, 0, p, 8, 32, 0, 0, 5, 32, 1, 1, None) == -2                        # more rows than the ring has
     assert lib.ajqd_matvec(p, p, 8, 0, p, 4, 0, 1, 4, 12, 1, 0, 1, None) == -2
     assert lib.ajqd_dense_out(p, p, p, None, None, 1, 8, 24, None) == -2
     args = _lib.WindowedAttentionArgs(q=p, k1=p, k2=p, v=p, out=p, k1_row=16, k1_head=8, k2_row=8, v_row=16, v_head=16, d1=8,
