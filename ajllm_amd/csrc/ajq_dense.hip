@@ -120,7 +120,7 @@ int launch_prefill_vt(int vt, const WindowedAttention& w, hipStream_t stream) {
 
 // ---- decode attention: (column steps, latent tiles per wave) that hold the widths
 int latent_tiles(int rankp) { const int t = (rankp + 63) / 64; return t <= 2 ? 2 : t <= 4 ? 4 : t <= 8 ? 8 : 0; }
-int latent_steps(int width) { const int s = (width + 31) / 32; return s <= 4 ? 4 : s <= 6 ? 6 : s <= 10 ? 10 : s <= 18 ? 18 : 0; }
+int latent_steps(int width) { const int s = (width + 31) / 32; return s <= 4 ? 4 : s <= 6 ? 6 : s <= 8 ? 8 : s <= 10 ? 10 : s <= 18 ? 18 : 0; }
 // the chunks' sums, then (maximum, denominator) per head and chunk
 float2* heads_at(const float* partial, int batch, int heads, int chunks, int rankp) {
   return reinterpret_cast<float2*>(const_cast<float*>(partial) + latent_sums_at(batch, 0, 0, heads, chunks, rankp));
@@ -291,7 +291,7 @@ int ajqd_windowed_attention(const ajqd_windowed_attention_args* args, int dtype,
 }
 
 int ajqd_windowed_prefill_supported(int d1, int d2, int dv) {
-  return d1 >= 8 && d2 >= 8 && d1 % 8 == 0 && d2 % 8 == 0 && dv >= 16 && dv % 16 == 0 && prefill_ks(d1 + d2) && prefill_vt(dv);
+  return d1 >= 8 && d2 >= 0 && d1 % 8 == 0 && d2 % 8 == 0 && dv >= 16 && dv % 16 == 0 && prefill_ks(d1 + d2) && prefill_vt(dv);
 }
 
 int ajqd_windowed_prefill(const ajqd_windowed_attention_args* args, void* stream) {
@@ -428,6 +428,7 @@ int ajqd_latent_decode(const void* q, const void* ring, const int64_t* pos, floa
   switch (latent_steps(rankp + rotp)) {
     case 4: return AJQD_DECODE(4, 2);  // (at most 128 columns: two tiles per wave)
     case 6: return tiles == 2 ? AJQD_DECODE(6, 2) : AJQD_DECODE(6, 3);
+    case 8: return tiles == 2 ? AJQD_DECODE(8, 2) : AJQD_DECODE(8, 4);
     case 10: return tiles == 2 ? AJQD_DECODE(10, 2) : tiles == 4 ? AJQD_DECODE(10, 4) : AJQD_DECODE(10, 5);
     default: return tiles == 2 ? AJQD_DECODE(18, 2) : tiles == 4 ? AJQD_DECODE(18, 4) : AJQD_DECODE(18, 8);
   }

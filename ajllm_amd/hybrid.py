@@ -506,7 +506,8 @@ def build_purusun(config: dict[str, Any]) -> HybridLM:
         if layer["type"] == "attention":
             if m.get("vdim", m["dim"]) != m["dim"]:
                 raise ValueError(f"layer {i}: vdim must equal dim (the values are the keys)")
-            mask, rot, s = m.get("mask") or {}, m["rot"], m["rot"].get("scaling")
+            mask, rot = m.get("mask") or {}, m.get("rot") or {"dims": 0, "base": 1.0}
+            s = rot.get("scaling")
             mixer = dict(num_heads=int(m["heads"]), num_kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), scale=float(m["scale"]),
                          rot_dim=int(rot["dims"]), rot_base=float(rot["base"]),
                          scaling=FrequencyScaling(float(s["factor"]), float(s["low"]), float(s["high"]), float(s["original"])) if s else None,
