@@ -18,6 +18,8 @@ Default run (what the driver calls: ``python bench.py --gpus 1 --steps K --warmu
   batch-32 decode at context 2048 with the quantized linears' share of the step), short form.
 
 ``--latent`` adds the dense latent-attention decoder (its own libajq_dense.so) beside the W8A16 Transformer.
+``--hybrid`` adds the decoder of key-value attention and selective scans on several residual streams beside the
+latent-attention decoder.
 ``--sweep`` adds the rest of the decode sweep (three shapes x M in {1, 4, 16}, W4 and W8)
 and all prefill shapes; ``--decode`` replaces the short decode leg by the long one (eager PyTorch loop
 beside it, token comparison between the two loops).  One JSON line is printed on stdout; everything else goes to stderr.
@@ -396,6 +398,9 @@ def main() -> int:
     ap.add_argument("--latent", action="store_true",
                     help="add the dense latent-attention decoder beside the W8A16 Transformer at two layer sizes: prompt and "
                          "decode throughput, and every kernel's share of its roofline")
+    ap.add_argument("--hybrid", action="store_true",
+                    help="add the decoder of key-value attention and selective scans beside the dense latent-attention decoder at two "
+                         "layer sizes: prompt and decode throughput, and every kernel's share of its roofline")
     ap.add_argument("--no-extras", action="store_true", help="timed region only")
     ap.add_argument("--no-decode", action="store_true",
                     help="skip the short end-to-end decode leg of the default line (counter-collection runs: "
@@ -514,6 +519,11 @@ def main() -> int:
 
         torch.cuda.empty_cache()
         extras["latent_attention_decoder"] = bench_latent(device, lambda name, row: log(name, json.dumps(row)))
+    if args.hybrid:
+        from ajllm_amd.hybrid_bench import bench_hybrid
+
+        torch.cuda.empty_cache()
+        extras["hybrid_decoder"] = bench_hybrid(device, lambda name, row: log(name, json.dumps(row)))
     # a plain device-to-device copy of known size: the yardstick the FETCH_SIZE / WRITE_SIZE
     # counters of a profiling run are scaled by (64 MiB read + 64 MiB written per launch)
     calib_src = torch.empty(64 * 2**20, dtype=torch.uint8, device=device)

@@ -453,7 +453,7 @@ def test_decode_step_of_the_scan(cuda, shape):
         dt = O.softplus(low[:, :rank] @ w_dt.double().T + dt_bias.double())
         want, end = O.recurrence(x, dt, -torch.exp(a_log.double()), low[:, rank:rank + states], low[:, rank + states:rank + 2 * states], skip.double())
         want = want * O.silu(y[:, b, inner:].double())
-        assert _rel(torch.stack([o[b] for o in got]), want) < 1e-2 and _rel(state[b], hybrid.state_planes(end)) < 1e-2
+        assert _rel(torch.stack([o[b] for o in got]), want) < 2e-2 and _rel(state[b], hybrid.state_planes(end)) < 2e-2
 
 
 # ------------------------------------------------------------------ the decoder against the plain implementation
@@ -548,10 +548,11 @@ def test_a_far_token_shows_through_the_state(cuda, dtype):
     weights = random_weights(cfg, 12)
     weights["l0.mix.A_log"].fill_(-9.0)
     weights["l0.mix.dt.b"].fill_(-1.0)
-    weights["l0.mix.o"] *= 4
-    tokens = _tokens(cfg, 300, 4)
-    tokens[0] = 0
-    weights["embed"][0] *= 8
+    weights["embed"][:, 7] = 0        # a column that tells token 0, which comes first and nowhere else, from the others
+    weights["embed"][0] = 0
+    weights["embed"][0, 7] = 30
+    weights["l0.mix.in"][:32, 7] = 3  # its input and B are large
+    tokens = [0] + [t or 2 for t in _tokens(cfg, 299, 4)]
     want = O.forward(cfg, weights, tokens)
     assert _rel(O.forward(cfg, weights, [1] + tokens[1:])[250:], want[250:]) > 2 * LOGIT_TOL[torch.bfloat16]
     model = _build(cfg, weights, cuda, dtype)
@@ -571,9 +572,7 @@ def test_a_kept_token_shows_far_away(cuda, dtype):
     weights["l0.mix.q.norm"].fill_(1.0)
     weights["l0.mix.k.norm"].fill_(1.0)
     weights["l0.hc1.in"].fill_(0.5)
-    tokens = [1] + [int(t) or 2 for t in _tokens(cfg, 400, 5)]
-    tokens = [t if t != 0 else 3 for t in tokens]
-    tokens[1] = 0                     # position 1 is the last one kept; token 0 occurs nowhere else
+    tokens = [1, 0] + [t or 2 for t in _tokens(cfg, 399, 5)]   # position 1 is the last one kept; token 0 occurs nowhere else
     unit = torch.zeros(16)
     unit[5] = 1.0
     axis = torch.zeros(cfg["width"])
