@@ -560,13 +560,22 @@ int ajqd_key_value_split(const ajqd_key_value_split_args* a, int y_dtype, int dt
   with_types(y_dtype, dtype, [&](auto yt, auto t) {
     using Y = decltype(yt);
     using T = decltype(t);
-    auto go = [&](auto kernel) {
+    const bool quads = (a->rot / 2) % 4 == 0 && a->dimp <= 256;
+    auto go = [&](auto lanes, auto whole) {
+      constexpr int L = decltype(lanes)::value;
+      auto kernel = key_value_split_kernel<Y, T, L, decltype(whole)::value>;
+      // few tokens: a head per team, so that the heads of a token go side by side
+      const int teams = 256 / L, slices = a->tokens < 256 ? (a->heads + a->groups + teams - 1) / teams : 1;
       status = allow_lds(kernel, bytes, "ajqd_key_value_split");
-      if (status == AJQ_OK) hipLaunchKernelGGL(kernel, dim3(a->tokens), dim3(256), bytes, (hipStream_t)stream, k);
+      if (status == AJQ_OK) hipLaunchKernelGGL(kernel, dim3(a->tokens, slices), dim3(256), bytes, (hipStream_t)stream, k);
     };
-    if (a->dimp <= 64) go(key_value_split_kernel<Y, T, 16>);
-    else if (a->dimp <= 128) go(key_value_split_kernel<Y, T, 32>);
-    else go(key_value_split_kernel<Y, T, 64>);
+    auto pick = [&](auto whole) {
+      if (a->dimp <= 64) go(std::integral_constant<int, 16>{}, whole);
+      else if (a->dimp <= 128) go(std::integral_constant<int, 32>{}, whole);
+      else go(std::integral_constant<int, 64>{}, whole);
+    };
+    if (quads) pick(std::true_type{});
+    else pick(std::false_type{});
   });
   return status != AJQ_OK ? status : check_launch("ajqd_key_value_split");
 }
@@ -595,8 +604,14 @@ int ajqd_conv_silu(const void* y, int ldy, void* ring, const float* weight, cons
   const long long blocks = ((long long)rows * (inner / 8) + 255) / 256;
   if (blocks > 0x7FFFFFFFll) return fail(AJQ_ERR_SHAPE, "ajqd_conv_silu: too many elements");
   ConvSilu c{y, ldy, ring, weight, bias, start, positions64(pos), rows, seq, inner, taps, out};
+  const long long run_blocks = ((long long)(rows / seq) * ((seq + kConvTokens - 1) / kConvTokens) * (inner / 8) + 255) / 256;
   with_types(dtype, dtype, [&](auto t, auto) {
-    hipLaunchKernelGGL(conv_silu_kernel<decltype(t)>, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, c);
+    using T = decltype(t);
+    auto run = [&](auto kernel) { hipLaunchKernelGGL(kernel, dim3((unsigned)run_blocks), dim3(256), 0, (hipStream_t)stream, c); };
+    if (!pos && taps == 2) return run(conv_silu_run_kernel<T, 2>);
+    if (!pos && taps == 3) return run(conv_silu_run_kernel<T, 3>);
+    if (!pos && taps == 4) return run(conv_silu_run_kernel<T, 4>);
+    hipLaunchKernelGGL(conv_silu_kernel<T>, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, c);
   });
   return check_launch("ajqd_conv_silu");
 }
@@ -618,7 +633,7 @@ int ajqd_scan(const ajqd_scan_args* a, int dtype, void* stream) {
 
 int ajqd_scan_splits(int batch, int inner) {
   (void)batch;
-  const int s = inner / 512;
+  const int s = (inner + kScanBlock - 1) / kScanBlock;
   return s < 1 ? 1 : s > 8 ? 8 : s;
 }
 
@@ -630,8 +645,9 @@ int ajqd_scan_project(const float* y, int ldy, const void* ring, const float* we
   ScanProject p{y, (const uint16_t*)ring, weight, bias, positions64(pos), (const uint16_t*)w, partial, batch, ldy, inner, taps, rows, splits};
   const int rt = batch > 4 && rows >= 32 ? 2 : 1;
   const dim3 grid((rows / 16 + rt - 1) / rt, splits, (batch + kGemvBatch - 1) / kGemvBatch);
-  if (rt == 2) hipLaunchKernelGGL(scan_project_kernel<2>, grid, dim3(256), 0, (hipStream_t)stream, p);
-  else hipLaunchKernelGGL(scan_project_kernel<1>, grid, dim3(256), 0, (hipStream_t)stream, p);
+  auto go = [&](auto kernel) { hipLaunchKernelGGL(kernel, grid, dim3(256), 0, (hipStream_t)stream, p); };
+  if (taps == 4) rt == 2 ? go(scan_project_kernel<2, 4>) : go(scan_project_kernel<1, 4>);
+  else rt == 2 ? go(scan_project_kernel<2, 0>) : go(scan_project_kernel<1, 0>);
   return check_launch("ajqd_scan_project");
 }
 
@@ -645,14 +661,13 @@ int ajqd_scan_step(const ajqd_scan_step_args* a, void* stream) {
                 a->states, a->rows);
   ScanStep s{a->y, (uint16_t*)a->ring, a->weight, a->bias, positions64(a->pos), a->partial, (const uint16_t*)a->w_dt, a->dt_bias, a->a2, a->d,
              a->state, (uint16_t*)a->out, a->batch, a->ldy, a->inner, a->taps, a->rows, a->splits, a->rank, a->states, a->out_ld};
-  auto go = [&](auto kernel, int ct) {
-    const int bytes = scan_step_lds(a->rank, a->states, ct);
+  auto go = [&](auto kernel, int bb) {
+    const int bytes = scan_step_lds(a->rank, a->states, bb);
     if (int e = allow_lds(kernel, bytes, "ajqd_scan_step")) return e;
-    hipLaunchKernelGGL(kernel, dim3((a->inner + 64 * ct - 1) / (64 * ct), (a->batch + kScanBatch - 1) / kScanBatch), dim3(256), bytes,
-                       (hipStream_t)stream, s);
+    hipLaunchKernelGGL(kernel, dim3((a->inner + 63) / 64, (a->batch + bb - 1) / bb), dim3(256), bytes, (hipStream_t)stream, s);
     return check_launch("ajqd_scan_step");
   };
-  return a->batch > kScanBatch ? go(scan_step_kernel<4>, 4) : go(scan_step_kernel<1>, 1);
+  return a->batch > 16 ? go(scan_step_kernel<8>, 8) : go(scan_step_kernel<4>, 4);
 }
 
 }  // extern "C"

@@ -23,8 +23,8 @@ struct KeyValueShape {
   float eps;
 };
 
-// One head of a projection row, normed over dim and rotated, by a team of LPH lanes: four columns per lane and turn, through
-// put(column, values); columns dim .. dimp are zero and stay so (the gain is zero there).
+// One head of a projection row, normed over dim and rotated, of any width and with any pairs, by a team of LPH lanes: four columns
+// per lane and turn, through put(column, values); columns dim .. dimp are zero and stay so (the gain is zero there).
 template <int LPH, typename Y, typename Put>
 __device__ __forceinline__ void norm_rotate(const Y* __restrict__ src, const KeyValueShape& s, const float* __restrict__ gain,
                                             const float* cosine, const float* sine, int lane, Put&& put) {
@@ -37,31 +37,13 @@ __device__ __forceinline__ void norm_rotate(const Y* __restrict__ src, const Key
   for (int off = LPH / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off);
   const Divisor by(sqrtf(ss / (float)s.dim + s.eps));
   const int half = s.rot >> 1;
-  const bool quads = (half & 3) == 0;
   auto one = [&](int i) { return by.divide(to_f32(src[i])) * gain[i]; };
   auto turned = [&](int i) {
     if (i >= s.rot) return one(i);
     if (i < half) return one(i) * cosine[i] - one(i + half) * sine[i];
     return one(i) * cosine[i - half] + one(i - half) * sine[i - half];
   };
-  for (int i = 4 * lane; i < s.dimp; i += 4 * LPH) {
-    if (i < s.rot && !quads) {  // a pair may straddle four columns
-      put(i, float4{turned(i), turned(i + 1), turned(i + 2), turned(i + 3)});
-      continue;
-    }
-    const float4 v = load4(src + i), g = load4(gain + i);
-    float4 a = float4{by.divide(v.x) * g.x, by.divide(v.y) * g.y, by.divide(v.z) * g.z, by.divide(v.w) * g.w};
-    if (i < s.rot) {
-      const bool first = i < half;
-      const int o = first ? i + half : i - half, e = first ? i : o;
-      const float4 w = load4(src + o), h = load4(gain + o), c = load4(cosine + e);
-      float4 n = load4(sine + e);
-      if (first) n = float4{-n.x, -n.y, -n.z, -n.w};
-      a = float4{a.x * c.x + by.divide(w.x) * h.x * n.x, a.y * c.y + by.divide(w.y) * h.y * n.y,
-                 a.z * c.z + by.divide(w.z) * h.z * n.z, a.w * c.w + by.divide(w.w) * h.w * n.w};
-    }
-    put(i, a);
-  }
+  for (int i = 4 * lane; i < s.dimp; i += 4 * LPH) put(i, float4{turned(i), turned(i + 1), turned(i + 2), turned(i + 3)});
 }
 
 struct KeyValueSplit {
@@ -78,29 +60,81 @@ struct KeyValueSplit {
   void* rows;               // row slot of (b, group) at b * rows_batch + group * rows_head + slot * 2 dimp
   long long rows_batch, rows_head;
 };
-// One workgroup per token; a team of LPH lanes per head.
-template <typename Y, typename T, int LPH>
+// Grid (tokens, slices): the heads of a token are dealt to the teams of LPH lanes of its workgroups.  QUADS: four columns per lane
+// hold a head, and its pairs too (dimp <= 4 LPH, half the rotated width a multiple of 4): a head is read once, the first one
+// before the angles are known, every other one ahead of the arithmetic of the one before; gains and angles stay in registers.
+template <typename Y, typename T, int LPH, bool QUADS>
 __global__ __launch_bounds__(256) void key_value_split_kernel(KeyValueSplit a) {
   extern __shared__ __attribute__((aligned(16))) float trig[];
+  constexpr int kTeams = 256 / LPH;
   const KeyValueShape s = a.s;
   const int m = blockIdx.x, b = m / a.seq, t = m % a.seq;
-  const int half = s.rot >> 1, pitch = (half + 3) & ~3;
+  const int half = s.rot >> 1, pitch = (half + 3) & ~3, all = s.heads + s.groups, stride = kTeams * gridDim.y;
   const int p = clamped_position(a.pos, a.start + t, 0x7FFFFFFF);
   const int slot = a.pos ? ring_slot(p, a.cap, a.kept) : a.prior + t;
-  angles(a.half_turns, half, p, trig, trig + pitch);
-  __syncthreads();
-  const int lane = threadIdx.x % LPH;
+  const int lane = threadIdx.x % LPH, first = kTeams * blockIdx.y + threadIdx.x / LPH;
   const Y* row = reinterpret_cast<const Y*>(a.y) + (size_t)m * a.ldy;
-  for (int n = threadIdx.x / LPH; n < s.heads + s.groups; n += 256 / LPH) {
-    const Y* src = row + n * s.dimp;
-    if (n < s.heads) {
-      T* dst = reinterpret_cast<T*>(a.q) + ((size_t)m * s.heads + n) * a.q_ld;
-      for (int i = 4 * lane; i < a.q_at; i += 4 * LPH) store4(dst + i, float4{0.f, 0.f, 0.f, 0.f});
-      norm_rotate<LPH>(src, s, a.q_gain, trig, trig + pitch, lane, [&](int i, float4 v) { store4(dst + a.q_at + i, v); });
-    } else {
-      T* dst = reinterpret_cast<T*>(a.rows) + (size_t)b * a.rows_batch + (size_t)(n - s.heads) * a.rows_head + (size_t)slot * (2 * s.dimp);
-      for (int i = 4 * lane; i < s.dimp; i += 4 * LPH) store4(dst + i, load4(src + i));
-      norm_rotate<LPH>(src, s, a.k_gain, trig, trig + pitch, lane, [&](int i, float4 v) { store4(dst + s.dimp + i, v); });
+  auto query = [&](int n) { return reinterpret_cast<T*>(a.q) + ((size_t)m * s.heads + n) * a.q_ld; };
+  auto key = [&](int n) {
+    return reinterpret_cast<T*>(a.rows) + (size_t)b * a.rows_batch + (size_t)(n - s.heads) * a.rows_head + (size_t)slot * (2 * s.dimp);
+  };
+  if constexpr (QUADS) {
+    const float4 zero = float4{0.f, 0.f, 0.f, 0.f};
+    const int i = 4 * lane, o = i < half ? i + half : i - half, e = i < half ? i : o;
+    const bool mine = i < s.dimp, pairs = mine && i < s.rot;
+    auto read = [&](int n, float4& v, float4& w) {
+      v = w = zero;
+      if (n < all && mine) v = load4(row + n * s.dimp + i);
+      if (n < all && pairs) w = load4(row + n * s.dimp + o);
+    };
+    float4 v, w, gq = zero, hq = zero, gk = zero, hk = zero, c = float4{1.f, 1.f, 1.f, 1.f}, d = zero;
+    read(first, v, w);
+    if (mine) { gq = load4(a.q_gain + i); gk = load4(a.k_gain + i); }
+    if (pairs) { hq = load4(a.q_gain + o); hk = load4(a.k_gain + o); }
+    angles(a.half_turns, half, p, trig, trig + pitch);
+    __syncthreads();
+    if (pairs) {
+      c = load4(trig + e);
+      d = load4(trig + pitch + e);
+      if (i < half) d = float4{-d.x, -d.y, -d.z, -d.w};
+    }
+    for (int n = first; n < all; n += stride) {
+      float4 nv, nw;
+      read(n + stride, nv, nw);
+      float ss = (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+#pragma unroll
+      for (int off = LPH / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off);
+      const Divisor by(sqrtf(ss / (float)s.dim + s.eps));
+      const bool is_query = n < s.heads;
+      const float4 g = is_query ? gq : gk, h = is_query ? hq : hk;
+      const float4 out = float4{by.divide(v.x) * g.x * c.x + by.divide(w.x) * h.x * d.x, by.divide(v.y) * g.y * c.y + by.divide(w.y) * h.y * d.y,
+                                by.divide(v.z) * g.z * c.z + by.divide(w.z) * h.z * d.z, by.divide(v.w) * g.w * c.w + by.divide(w.w) * h.w * d.w};
+      if (is_query) {
+        T* dst = query(n);
+        for (int k = i; k < a.q_at; k += 4 * LPH) store4(dst + k, zero);
+        if (mine) store4(dst + a.q_at + i, out);
+      } else if (mine) {
+        T* dst = key(n);
+        store4(dst + i, v);
+        store4(dst + s.dimp + i, out);
+      }
+      v = nv;
+      w = nw;
+    }
+  } else {
+    angles(a.half_turns, half, p, trig, trig + pitch);
+    __syncthreads();
+    for (int n = first; n < all; n += stride) {
+      const Y* src = row + n * s.dimp;
+      if (n < s.heads) {
+        T* dst = query(n);
+        for (int i = 4 * lane; i < a.q_at; i += 4 * LPH) store4(dst + i, float4{0.f, 0.f, 0.f, 0.f});
+        norm_rotate<LPH>(src, s, a.q_gain, trig, trig + pitch, lane, [&](int i, float4 v) { store4(dst + a.q_at + i, v); });
+      } else {
+        T* dst = key(n);
+        for (int i = 4 * lane; i < s.dimp; i += 4 * LPH) store4(dst + i, load4(src + i));
+        norm_rotate<LPH>(src, s, a.k_gain, trig, trig + pitch, lane, [&](int i, float4 v) { store4(dst + s.dimp + i, v); });
+      }
     }
   }
 }

@@ -20,7 +20,18 @@
 namespace ajq {
 
 __device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
-__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// For operands in bf16: the hardware's exponential and reciprocal (one ulp each; the argument's rounding makes it |z| ulps).
+template <typename T>
+__device__ __forceinline__ float silu_for(float z) {
+  if (sizeof(T) == 4) return silu_f32(z);
+  return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
+// max(z, 0) + log(1 + e) with e = exp(-|z|).  1 + e is rounded to u, which log(u) e / (u - 1) makes good (u - 1 is exact).
+__device__ __forceinline__ float softplus_f32(float z) {
+  const float e = expf(-fabsf(z)), u = 1.0f + e, d = u - 1.0f;
+  const float l = d == 0.f ? e : 0.6931471805599453f * __builtin_amdgcn_logf(u) * (e * __builtin_amdgcn_rcpf(d));
+  return fmaxf(z, 0.f) + l;
+}
 
 struct ConvSilu {
   const void* y;            // [B * seq, ldy], the convolved columns first
@@ -55,8 +66,52 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvSilu a) {
   }
   if (a.pos && reach > 0) store8(ring + (size_t)(p % reach) * a.inner, own);
 #pragma unroll
-  for (int e = 0; e < 8; ++e) sum.v[e] = silu_f32(sum.v[e]);
+  for (int e = 0; e < 8; ++e) sum.v[e] = silu_for<T>(sum.v[e]);
   store8(reinterpret_cast<T*>(a.out) + (size_t)m * a.inner + c, sum);
+}
+
+// The same for prompts (no device-side position): a thread makes 8 channels of kConvTokens tokens, its weights and the last
+// TAPS - 1 rows in registers.
+constexpr int kConvTokens = 8;
+template <typename T, int TAPS>
+__global__ __launch_bounds__(256) void conv_silu_run_kernel(ConvSilu a) {
+  constexpr int kReach = TAPS - 1;
+  const int vectors = a.inner >> 3, runs = (a.seq + kConvTokens - 1) / kConvTokens;
+  const long long idx = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= (long long)(a.rows / a.seq) * runs * vectors) return;
+  const int c = 8 * (int)(idx % vectors), run = (int)((idx / vectors) % runs), b = (int)(idx / ((long long)vectors * runs));
+  const int t0 = run * kConvTokens, count = min(kConvTokens, a.seq - t0);
+  const T* y = reinterpret_cast<const T*>(a.y) + ((size_t)b * a.seq + t0) * a.ldy + c;
+  const T* ring = reinterpret_cast<const T*>(a.ring) + (size_t)b * kReach * a.inner + c;
+  T* out = reinterpret_cast<T*>(a.out) + ((size_t)b * a.seq + t0) * a.inner + c;
+  Float8 now[kConvTokens], last[kReach], w[TAPS];  // last[j]: j + 1 tokens back
+#pragma unroll
+  for (int k = 0; k < kConvTokens; ++k)
+    if (k < count) now[k] = load8(y + (size_t)k * a.ldy);
+#pragma unroll
+  for (int j = 0; j < kReach; ++j) {
+    const int t = t0 - 1 - j, p = a.start + t;
+    last[j] = Float8{};
+    if (t >= 0) last[j] = load8(y - (size_t)(j + 1) * a.ldy);
+    else if (p >= 0) last[j] = load8(ring + (size_t)(p % kReach) * a.inner);
+  }
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) w[j] = load8(a.weight + (size_t)(kReach - j) * a.inner + c);
+  const Float8 bias = load8(a.bias + c);
+#pragma unroll
+  for (int k = 0; k < kConvTokens; ++k) {
+    if (k >= count) break;
+    Float8 sum = bias;
+#pragma unroll
+    for (int j = kReach; j >= 0; --j) {
+      const Float8& v = j <= k ? now[j <= k ? k - j : 0] : last[j > k ? j - k - 1 : 0];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) sum.v[e] = fmaf(w[j].v[e], v.v[e], sum.v[e]);
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sum.v[e] = silu_for<T>(sum.v[e]);
+    store8(out + (size_t)k * a.inner, sum);
+  }
 }
 
 template <int kCtrl>
@@ -91,6 +146,10 @@ struct Scan {
 // still fills the chip: the time loop is sequential, and its length is what a wave costs.  256 / L channels per workgroup.
 // A tile of kT tokens is staged in LDS: dt and dt x (the softplus is taken once per channel and token there), B and C; y takes
 // dt x's place.  The next tile's operands are requested ahead of the current one's time loop.
+template <int K, int NS>
+struct Operands {
+  float dt[K], dx[K], b[K][NS], c[K][NS];
+};
 template <int L, int NS>
 constexpr int scan_tile() {
   int t = 8 * L;
@@ -175,19 +234,36 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan a) {
     }
     __syncthreads();
     if (t0 + kT < a.seq) request(t0 + kT);
-    for (int u = 0; u < count; u += kTogether) {  // (tokens past the end: dt = 0 leaves the states alone)
-      float y[kTogether];
+    // (tokens past the end: dt = 0 leaves the states alone)  A group's operands are read ahead of the arithmetic of the one before.
+    Operands<kTogether, NS> next;
+    auto read = [&](int u) {
 #pragma unroll
       for (int k = 0; k < kTogether; ++k) {
-        const int t = u + k;
-        const float dt = dt_s[t * kPitch + ch], dx = dx_s[t * kPitch + ch];
-        const float* bt = b_s + t * kN + part * NS;
-        const float* ct = c_s + t * kN + part * NS;
+        next.dt[k] = dt_s[(u + k) * kPitch + ch];
+        next.dx[k] = dx_s[(u + k) * kPitch + ch];
+#pragma unroll
+        for (int i = 0; i < NS; ++i) {
+          next.b[k][i] = b_s[(u + k) * kN + part * NS + i];
+          next.c[k][i] = c_s[(u + k) * kN + part * NS + i];
+        }
+      }
+    };
+    read(0);
+    for (int u = 0; u < count; u += kTogether) {
+      const Operands<kTogether, NS> now = next;
+      read(min(u + kTogether, kT - kTogether));
+      float y[kTogether], f[kTogether][NS];
+#pragma unroll
+      for (int k = 0; k < kTogether; ++k)
+#pragma unroll
+        for (int i = 0; i < NS; ++i) f[k][i] = __builtin_amdgcn_exp2f(now.dt[k] * a2[i]);
+#pragma unroll
+      for (int k = 0; k < kTogether; ++k) {
         y[k] = 0.f;
 #pragma unroll
         for (int i = 0; i < NS; ++i) {
-          s[i] = fmaf(__builtin_amdgcn_exp2f(dt * a2[i]), s[i], dx * bt[i]);
-          y[k] = fmaf(s[i], ct[i], y[k]);
+          s[i] = fmaf(f[k][i], s[i], now.dx[k] * now.b[k][i]);
+          y[k] = fmaf(s[i], now.c[k][i], y[k]);
         }
       }
 #pragma unroll
@@ -201,7 +277,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan a) {
       const float* ys = dx_s + vt * kPitch + vl;
       Float8 o;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o.v[e] = fmaf(skip.v[e], x.v[e], ys[e]) * silu_f32(z.v[e]);
+      for (int e = 0; e < 8; ++e) o.v[e] = fmaf(skip.v[e], x.v[e], ys[e]) * silu_for<T>(z.v[e]);
       store8(op + (size_t)(t0 + vt) * a.out_ld, o);
     }
     __syncthreads();
@@ -213,9 +289,16 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan a) {
 }
 
 // ---- one token per sequence, bf16
+// Slot of the column `back` tokens (1 .. reach) ahead of the one whose own slot is `slot`.
+__device__ __forceinline__ int column_slot(int slot, int back, int reach) {
+  const int s = slot - back;
+  return s < 0 ? s + reach : s;
+}
+
 // The projection of the convolved columns to (dt rank | B | C): `rows` weight rows (a multiple of 16), K = inner cut into
-// `splits` parts whose sums scan_step_kernel adds.  A lane convolves the eight channels of its own operand fragment, so the
-// convolved row exists in registers only; every group of RT row tiles repeats that.  Grid (row groups, splits, batch blocks).
+// `splits` parts whose sums scan_step_kernel adds.  A workgroup takes RT row tiles and a part of K in blocks of kScanBlock
+// channels: a wave requests its weights, all threads convolve the block's channels into LDS (a thread 8 channels of every
+// second sequence, its weights in registers), then the product.  Grid (row groups, splits, batch blocks).
 struct ScanProject {
   const float* y;           // [B, ldy]: convolved columns, then z
   const uint16_t* ring;     // [B, taps - 1, inner]
@@ -226,42 +309,77 @@ struct ScanProject {
   float* partial;           // [splits, B, rows]
   int batch, ldy, inner, taps, rows, splits;
 };
-template <int RT>
+constexpr int kScanBlock = 1024;
+// TAPS: the convolution's width, or 0 for any
+template <int RT, int TAPS>
 __global__ __launch_bounds__(256) void scan_project_kernel(ScanProject a) {
+  constexpr int kSteps = kScanBlock / 32 / 4, kLd = kScanBlock + 8;
+  __shared__ __attribute__((aligned(16))) uint16_t conv[kGemvBatch * kLd];
   __shared__ __attribute__((aligned(16))) float red[RT * 4 * 256];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
   const int b0 = blockIdx.z * kGemvBatch, nb = min(kGemvBatch, a.batch - b0);
   const int tile0 = max(0, min(RT * (int)blockIdx.x, a.rows / 16 - RT));  // (the last group may repeat its neighbour's rows)
-  const int reach = a.taps - 1, p = clamped_position(a.pos, 0, 0x7FFFFFFF);
+  const int reach = (TAPS ? TAPS : a.taps) - 1, p = clamped_position(a.pos, 0, 0x7FFFFFFF), slot = reach > 0 ? p % reach : 0;
   const int steps = (a.inner + 31) >> 5, per = (steps + a.splits - 1) / a.splits;
-  const int lo = min(steps, (int)blockIdx.y * per), hi = min(steps, lo + per), quarter = (hi - lo + 3) >> 2;
-  const int begin = min(hi, lo + wave * quarter), end = min(hi, begin + quarter);
-  const float* y = a.y + (size_t)(b0 + min(r, nb - 1)) * a.ldy;
-  const uint16_t* ring = a.ring + (size_t)(b0 + min(r, nb - 1)) * reach * a.inner;
+  const int lo = min(steps, (int)blockIdx.y * per), hi = min(steps, lo + per);
+  const uint16_t* wrow = a.w + (size_t)(16 * tile0 + r) * a.inner;
+  const int vl = 8 * (tid & 127);
   f32x4_t acc[RT][1] = {};
-  tile_steps<RT, 1>(a.w + (size_t)(16 * tile0 + r) * a.inner, a.inner, begin, end, g, acc, [&](int, int s) {
-    u32x4_t packed = {0u, 0u, 0u, 0u};
-    if (r < nb) {
-      const int c = 32 * s + 8 * g;
-      Float8 sum = load8(a.bias + c);
-      for (int j = min(reach, p); j >= 0; --j) {
-        const Float8 w = load8(a.weight + (size_t)(reach - j) * a.inner + c);
-        Float8 v;
-        if (j > 0) {
-          v = load8(ring + (size_t)((p - j) % reach) * a.inner + c);
-        } else {  // (as the ring will hold it)
-          v = load8(y + c);
+  for (int s0 = lo; s0 < hi; s0 += kScanBlock / 32) {
+    const int mine = s0 + kSteps * wave;
+    u32x4_t w[kSteps][RT];
 #pragma unroll
-          for (int e = 0; e < 8; ++e) v.v[e] = to_f32(f32_to_bf16_rne(v.v[e]));
+    for (int i = 0; i < kSteps; ++i)
+#pragma unroll
+      for (int n = 0; n < RT; ++n) {
+        const int k = 32 * (mine + i) + 8 * g;
+        w[i][n] = u32x4_t{0u, 0u, 0u, 0u};
+        if (mine + i < hi && k < a.inner) w[i][n] = *reinterpret_cast<const u32x4_t*>(wrow + (size_t)n * 16 * a.inner + k);
+      }
+    const int c = 32 * s0 + vl;
+    if (c < min(32 * hi, a.inner)) {
+      const Float8 bias = load8(a.bias + c);
+      Float8 f[TAPS ? TAPS : 1];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) f[j] = load8(a.weight + (size_t)(reach - j) * a.inner + c);
+      for (int b = tid >> 7; b < nb; b += 2) {
+        const uint16_t* ring = a.ring + (size_t)(b0 + b) * reach * a.inner + c;
+        Float8 sum = bias, own = load8(a.y + (size_t)(b0 + b) * a.ldy + c);
+        auto tap = [&](const Float8& weight, const Float8& v) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) sum.v[e] = fmaf(weight.v[e], v.v[e], sum.v[e]);
+        };
+        if (TAPS > 0) {
+          Float8 held[TAPS > 1 ? TAPS : 1];
+#pragma unroll
+          for (int j = TAPS - 1; j > 0; --j)
+            if (j <= p) held[j] = load8(ring + (size_t)column_slot(slot, j, reach) * a.inner);
+#pragma unroll
+          for (int j = TAPS - 1; j > 0; --j)
+            if (j <= p) tap(f[j], held[j]);
+        } else {
+          for (int j = min(reach, p); j > 0; --j)
+            tap(load8(a.weight + (size_t)(reach - j) * a.inner + c), load8(ring + (size_t)column_slot(slot, j, reach) * a.inner));
         }
 #pragma unroll
-        for (int e = 0; e < 8; ++e) sum.v[e] = fmaf(w.v[e], v.v[e], sum.v[e]);
-      }
+        for (int e = 0; e < 8; ++e) own.v[e] = to_f32(f32_to_bf16_rne(own.v[e]));  // (as the ring will hold it)
+        tap(TAPS ? f[0] : load8(a.weight + (size_t)reach * a.inner + c), own);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) packed[e] = pack2_bf16(silu_f32(sum.v[2 * e]), silu_f32(sum.v[2 * e + 1]));
+        for (int e = 0; e < 8; ++e) sum.v[e] = silu_for<uint16_t>(sum.v[e]);
+        store8(conv + b * kLd + vl, sum);
+      }
     }
-    return packed;
-  });
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < kSteps; ++i) {
+      const int local = 32 * (kSteps * wave + i) + 8 * g;
+      u32x4_t v = {0u, 0u, 0u, 0u};
+      if (r < nb && mine + i < hi && 32 * s0 + local < a.inner) v = *reinterpret_cast<const u32x4_t*>(conv + r * kLd + local);
+#pragma unroll
+      for (int n = 0; n < RT; ++n) acc[n][0] = mfma16(w[i][n], v, acc[n][0]);
+    }
+    __syncthreads();
+  }
   meet<4, RT, 1>(acc, red, wave, lane);
 #pragma unroll
   for (int i = 0; i < RT; ++i)
@@ -270,10 +388,10 @@ __global__ __launch_bounds__(256) void scan_project_kernel(ScanProject a) {
              float4{acc[i][0][0], acc[i][0][1], acc[i][0][2], acc[i][0][3]});
 }
 
-// The rest of the step for 64 CT channels of kScanBatch sequences: the parts of (dt rank | B | C) are added, dt comes from a
-// product on MFMA (a wave per CT tiles of 16 channels), then a thread per (sequence, channel) convolves its channel, moves the
-// channel's states on and writes the gated output and the ring's new row.  Grid (channel blocks, batch blocks).
-constexpr int kScanBatch = 4;
+// The rest of the step for 64 channels of BB sequences: the parts of (dt rank | B | C) are added, dt comes from a product on
+// MFMA (a wave per 16 channels), then a lane per channel, a wave per sequence and turn: it convolves the channel, moves the
+// channel's states on and writes the gated output and the ring's new row.  Everything that does not hang on the parts is
+// requested behind them, ahead of the first barrier.  Grid (channel blocks, batch blocks).
 struct ScanStep {
   const float* y;           // [B, ldy]: convolved columns, z from column inner on
   uint16_t* ring;
@@ -286,71 +404,121 @@ struct ScanStep {
   uint16_t* out;            // [B, out_ld]
   int batch, ldy, inner, taps, rows, splits, rank, states, out_ld;
 };
-__host__ __device__ constexpr int scan_step_lds(int rank, int states, int ct) {
-  return kScanBatch * (2 * (rank + 8) + 4 * 2 * states + 4 * 64 * ct);
+__host__ __device__ constexpr int scan_step_lds(int rank, int states, int bb) {
+  return bb * (2 * (rank + 8) + 4 * 2 * states + 4 * 64);
 }
-template <int CT>
+template <int BB>
 __global__ __launch_bounds__(256) void scan_step_kernel(ScanStep a) {
+  constexpr int kTurns = BB / 4, kPlanes = 4, kSteps = 8, kAhead = 8;
   extern __shared__ __attribute__((aligned(16))) unsigned char scan_lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
-  const int b0 = blockIdx.y * kScanBatch, nb = min(kScanBatch, a.batch - b0), c0 = blockIdx.x * 64 * CT;
-  const int ld = a.rank + 8;
-  float* bc = reinterpret_cast<float*>(scan_lds);                    // [kScanBatch][2 states]
-  float* dt_s = bc + kScanBatch * 2 * a.states;                      // [kScanBatch][64 CT]
-  uint16_t* low = reinterpret_cast<uint16_t*>(dt_s + kScanBatch * 64 * CT);  // [kScanBatch][rank + 8]
-  const int used = a.rank + 2 * a.states;
-  for (int i = tid; i < nb * used; i += 256) {
-    const int b = i / used, n = i % used;
-    float v = 0.f;
-    for (int s = 0; s < a.splits; ++s) v += a.partial[((size_t)s * a.batch + b0 + b) * a.rows + n];
-    if (n < a.rank) low[b * ld + n] = f32_to_bf16_rne(v);
-    else bc[b * 2 * a.states + n - a.rank] = v;
+  const int b0 = blockIdx.y * BB, nb = min(BB, a.batch - b0), c0 = blockIdx.x * 64, c = c0 + lane;
+  const int ld = a.rank + 8, used = a.rank + 2 * a.states, quads = used >> 2;
+  float* bc = reinterpret_cast<float*>(scan_lds);                  // [BB][2 states]
+  float* dt_s = bc + BB * 2 * a.states;                            // [BB][64]
+  uint16_t* low = reinterpret_cast<uint16_t*>(dt_s + BB * 64);     // [BB][rank + 8]
+  const int reach = a.taps - 1, p = clamped_position(a.pos, 0, 0x7FFFFFFF), slot = reach > 0 ? p % reach : 0;
+  float4 ahead[kAhead];
+  auto request = [&](int i, int s0) {
+    const float* src = a.partial + (size_t)(b0 + i / quads) * a.rows + 4 * (i % quads);
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k)
+      if (s0 + k < a.splits) ahead[k] = load4(src + (size_t)(s0 + k) * a.batch * a.rows);
+  };
+  if (tid < nb * quads) request(tid, 0);
+  // this wave's 16 channels of the step size product
+  const bool tile = c0 + 16 * wave < a.inner;
+  const uint16_t* wrow = a.w_dt + (size_t)(c0 + 16 * wave + r) * a.rank;
+  u32x4_t w[kSteps];
+#pragma unroll
+  for (int s = 0; s < kSteps; ++s) {
+    w[s] = u32x4_t{0u, 0u, 0u, 0u};
+    if (tile && 32 * s + 8 * g < a.rank) w[s] = *reinterpret_cast<const u32x4_t*>(wrow + 32 * s + 8 * g);
+  }
+  // this lane's channel: the convolution, the gate, the first planes of its decays and states
+  float x[kTurns], z[kTurns], skip = 0.f;
+  uint16_t own[kTurns];
+  float4 f[kPlanes], st[kTurns][kPlanes];
+  if (c < a.inner) {
+    skip = a.d[c];
+#pragma unroll
+    for (int n = 0; n < kPlanes; ++n)
+      if (4 * n < a.states) f[n] = load4(a.a2 + ((size_t)n * a.inner + c) * 4);
+  }
+#pragma unroll
+  for (int t = 0; t < kTurns; ++t) {
+    const int b = wave + 4 * t;
+    if (c >= a.inner || b >= nb) continue;
+    const float* y = a.y + (size_t)(b0 + b) * a.ldy + c;
+    const uint16_t* ring = a.ring + (size_t)(b0 + b) * reach * a.inner + c;
+    const float* state = a.state + (size_t)(b0 + b) * a.states * a.inner + 4 * c;
+#pragma unroll
+    for (int n = 0; n < kPlanes; ++n)
+      if (4 * n < a.states) st[t][n] = p > 0 ? load4(state + (size_t)n * a.inner * 4) : float4{0.f, 0.f, 0.f, 0.f};
+    own[t] = f32_to_bf16_rne(y[0]);
+    z[t] = y[a.inner];
+    x[t] = a.bias[c];
+#pragma unroll 4
+    for (int j = min(reach, p); j > 0; --j)
+      x[t] = fmaf(a.weight[(size_t)(reach - j) * a.inner + c], to_f32(ring[(size_t)column_slot(slot, j, reach) * a.inner]), x[t]);
+    x[t] = fmaf(a.weight[(size_t)reach * a.inner + c], to_f32(own[t]), x[t]);
+  }
+  for (int i = tid; i < nb * quads; i += 256) {
+    float4 v = float4{0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < a.splits; s0 += kAhead) {
+      if (i != tid || s0 > 0) request(i, s0);
+#pragma unroll
+      for (int k = 0; k < kAhead; ++k)
+        if (s0 + k < a.splits) {
+          v.x += ahead[k].x; v.y += ahead[k].y; v.z += ahead[k].z; v.w += ahead[k].w;
+        }
+    }
+    const int b = i / quads, n = 4 * (i % quads);
+    if (n < a.rank) store4(low + b * ld + n, v);
+    else store4(bc + b * 2 * a.states + n - a.rank, v);
+  }
+  __syncthreads();
+  if (tile) {
+    f32x4_t acc[1][1] = {};
+    auto operand = [&](int, int s) {
+      return r < nb ? *reinterpret_cast<const u32x4_t*>(low + r * ld + 32 * s + 8 * g) : u32x4_t{0u, 0u, 0u, 0u};
+    };
+#pragma unroll
+    for (int s = 0; s < kSteps; ++s)
+      if (32 * s < a.rank) acc[0][0] = mfma16(w[s], 32 * s + 8 * g < a.rank ? operand(0, s) : u32x4_t{0u, 0u, 0u, 0u}, acc[0][0]);
+    tile_steps<1, 1>(wrow, a.rank, kSteps, (a.rank + 31) >> 5, g, acc, operand);
+    if (r < nb) {
+      const float4 bias = load4(a.dt_bias + c0 + 16 * wave + 4 * g);
+      store4(dt_s + r * 64 + 16 * wave + 4 * g, float4{softplus_f32(acc[0][0][0] + bias.x), softplus_f32(acc[0][0][1] + bias.y),
+                                                       softplus_f32(acc[0][0][2] + bias.z), softplus_f32(acc[0][0][3] + bias.w)});
+    }
   }
   __syncthreads();
 #pragma unroll
-  for (int t = 0; t < CT; ++t) {
-    const int c = 16 * (CT * wave + t);
-    if (c0 + c >= a.inner) continue;
-    f32x4_t acc[1][1] = {};
-    tile_steps<1, 1>(a.w_dt + (size_t)(c0 + c + r) * a.rank, a.rank, 0, (a.rank + 31) >> 5, g, acc, [&](int, int s) {
-      return r < nb ? *reinterpret_cast<const u32x4_t*>(low + r * ld + 32 * s + 8 * g) : u32x4_t{0u, 0u, 0u, 0u};
-    });
-    if (r < nb) {
-      const float4 bias = load4(a.dt_bias + c0 + c + 4 * g);
-      store4(dt_s + r * 64 * CT + c + 4 * g, float4{softplus_f32(acc[0][0][0] + bias.x), softplus_f32(acc[0][0][1] + bias.y),
-                                                    softplus_f32(acc[0][0][2] + bias.z), softplus_f32(acc[0][0][3] + bias.w)});
-    }
-  }
-  __syncthreads();
-  const int reach = a.taps - 1, p = clamped_position(a.pos, 0, 0x7FFFFFFF);
-  for (int i = tid; i < nb * 64 * CT; i += 256) {
-    const int b = i / (64 * CT), local = i % (64 * CT), c = c0 + local;
-    if (c >= a.inner) continue;
-    const float* y = a.y + (size_t)(b0 + b) * a.ldy;
-    uint16_t* ring = a.ring + (size_t)(b0 + b) * reach * a.inner + c;
-    const uint16_t own = f32_to_bf16_rne(y[c]);
-    float x = a.bias[c];
-    for (int j = min(reach, p); j >= 0; --j)
-      x = fmaf(a.weight[(size_t)(reach - j) * a.inner + c], to_f32(j > 0 ? ring[(size_t)((p - j) % reach) * a.inner] : own), x);
-    if (reach > 0) ring[(size_t)(p % reach) * a.inner] = own;
-    x = silu_f32(x);
-    const float dt = dt_s[b * 64 * CT + local], dx = dt * x;
-    float* state = a.state + ((size_t)(b0 + b) * a.states * a.inner) + 4 * c;
+  for (int t = 0; t < kTurns; ++t) {
+    const int b = wave + 4 * t;
+    if (c >= a.inner || b >= nb) continue;
+    if (reach > 0) a.ring[((size_t)(b0 + b) * reach + slot) * a.inner + c] = own[t];
+    const float v = silu_for<uint16_t>(x[t]), dt = dt_s[b * 64 + lane], dx = dt * v;
+    float* state = a.state + (size_t)(b0 + b) * a.states * a.inner + 4 * c;
     const float* bs = bc + b * 2 * a.states;
-    float out = a.d[c] * x;
-#pragma unroll 4
-    for (int n = 0; n < a.states; n += 4) {
-      const float4 f = load4(a.a2 + (size_t)n * a.inner + 4 * c);
-      float4 s = p > 0 ? load4(state + (size_t)n * a.inner) : float4{0.f, 0.f, 0.f, 0.f};
-      const float4 bn = load4(bs + n), cn = load4(bs + a.states + n);
-      s.x = fmaf(__builtin_amdgcn_exp2f(dt * f.x), s.x, dx * bn.x);
-      s.y = fmaf(__builtin_amdgcn_exp2f(dt * f.y), s.y, dx * bn.y);
-      s.z = fmaf(__builtin_amdgcn_exp2f(dt * f.z), s.z, dx * bn.z);
-      s.w = fmaf(__builtin_amdgcn_exp2f(dt * f.w), s.w, dx * bn.w);
-      store4(state + (size_t)n * a.inner, s);
+    float out = skip * v;
+    auto move = [&](int n, float4 s, const float4& k) {
+      const float4 bn = load4(bs + 4 * n), cn = load4(bs + a.states + 4 * n);
+      s.x = fmaf(__builtin_amdgcn_exp2f(dt * k.x), s.x, dx * bn.x);
+      s.y = fmaf(__builtin_amdgcn_exp2f(dt * k.y), s.y, dx * bn.y);
+      s.z = fmaf(__builtin_amdgcn_exp2f(dt * k.z), s.z, dx * bn.z);
+      s.w = fmaf(__builtin_amdgcn_exp2f(dt * k.w), s.w, dx * bn.w);
+      store4(state + (size_t)n * a.inner * 4, s);
       out = fmaf(s.x, cn.x, fmaf(s.y, cn.y, fmaf(s.z, cn.z, fmaf(s.w, cn.w, out))));
-    }
-    a.out[(size_t)(b0 + b) * a.out_ld + c] = f32_to_bf16_rne(out * silu_f32(y[a.inner + c]));
+    };
+#pragma unroll
+    for (int n = 0; n < kPlanes; ++n)
+      if (4 * n < a.states) move(n, st[t][n], f[n]);
+#pragma unroll 4
+    for (int n = kPlanes; n < a.states / 4; ++n)
+      move(n, p > 0 ? load4(state + (size_t)n * a.inner * 4) : float4{0.f, 0.f, 0.f, 0.f}, load4(a.a2 + ((size_t)n * a.inner + c) * 4));
+    a.out[(size_t)(b0 + b) * a.out_ld + c] = f32_to_bf16_rne(out * silu_for<uint16_t>(z[t]));
   }
 }
 
