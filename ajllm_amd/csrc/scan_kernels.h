@@ -26,11 +26,14 @@ __device__ __forceinline__ float silu_for(float z) {
   if (sizeof(T) == 4) return silu_f32(z);
   return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
 }
-// max(z, 0) + log(1 + e) with e = exp(-|z|).  1 + e is rounded to u, which log(u) e / (u - 1) makes good (u - 1 is exact).
+// max(z, 0) + log(1 + e) with e = exp(-|z|), the exponential in base 2 with the part of its exponent that the product rounded
+// away.  1 + e is rounded to u, which log(u) e / (u - 1) makes good (u - 1 is exact).  No branch.
 __device__ __forceinline__ float softplus_f32(float z) {
-  const float e = expf(-fabsf(z)), u = 1.0f + e, d = u - 1.0f;
-  const float l = d == 0.f ? e : 0.6931471805599453f * __builtin_amdgcn_logf(u) * (e * __builtin_amdgcn_rcpf(d));
-  return fmaxf(z, 0.f) + l;
+  constexpr float kLog2e = 1.4426950408889634f, kLn2 = 0.6931471805599453f;
+  const float x = -fminf(fabsf(z), 100.f), h = x * kLog2e, rest = fmaf(x, kLog2e, -h);
+  const float e0 = __builtin_amdgcn_exp2f(h), e = fmaf(e0, rest * kLn2, e0), u = 1.0f + e, d = u - 1.0f;
+  const float l = kLn2 * __builtin_amdgcn_logf(u) * (e * __builtin_amdgcn_rcpf(d == 0.f ? 1.f : d));
+  return fmaxf(z, 0.f) + (d == 0.f ? e : l);
 }
 
 struct ConvSilu {
@@ -185,7 +188,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan a) {
   const T* lp = reinterpret_cast<const T*>(a.low) + (size_t)b * a.seq * a.low_ld;
   T* op = reinterpret_cast<T*>(a.out) + (size_t)b * a.seq * a.out_ld + vc;
   constexpr int kLow = (kT * kN + 255) / 256;
-  Float8 nx, nd, nz, bias, skip;
+  Float8 nx{}, nd{}, nz{}, bias{}, skip{};
   float nb[kLow], nc[kLow];
   if (stages) {
     bias = load8(a.dt_bias + vc);
@@ -216,10 +219,12 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan a) {
       float* dts = dt_s + vt * kPitch + vl;
       float* dxs = dx_s + vt * kPitch + vl;
       Float8 d, dx;
+      const bool real = stages && vt < count;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        d.v[e] = stages && vt < count ? softplus_f32(nd.v[e] + bias.v[e]) : 0.f;
-        dx.v[e] = stages && vt < count ? d.v[e] * x.v[e] : 0.f;
+        const float step = softplus_f32(nd.v[e] + bias.v[e]);
+        d.v[e] = real ? step : 0.f;
+        dx.v[e] = real ? step * x.v[e] : 0.f;
       }
       store8(dts, d);
       store8(dxs, dx);
