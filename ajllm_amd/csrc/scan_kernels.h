@@ -5,7 +5,7 @@
 //   out = y silu(z)
 //
 // Prompts (any number of tokens, from any position; also one token on any operand type):
-//   conv_silu_kernel, scan_kernel
+//   conv_silu_kernel, conv_silu_run_kernel (prompts with usual widths), scan_kernel
 // One token in bf16:
 //   scan_project_kernel, scan_step_kernel
 //
