@@ -417,7 +417,7 @@ def test_scan_portions_equal_the_whole(cuda, dtype):
 
 
 STEPS = [  # batch, inner, states, rank, taps
-    (1, 48, 8, 8, 4), (3, 384, 24, 16, 4), (1, 1552, 16, 40, 2), (5, 80, 40, 8, 1), (17, 640, 16, 24, 3), (20, 2048, 4, 128, 4), (33, 32, 64, 8, 7),
+    (1, 48, 8, 8, 4), (3, 400, 28, 16, 4), (1, 1552, 16, 40, 2), (5, 80, 40, 8, 1), (17, 640, 16, 24, 3), (20, 2048, 4, 128, 4), (33, 32, 64, 8, 7),
 ]
 
 
